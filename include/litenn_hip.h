@@ -334,6 +334,59 @@ int litenn_hip_llama_generate(litenn_hip_llama* model, const int32_t* prompt, si
 /* Copies the first `past` cache rows of one layer to host as f32 [past, n_kv_head*head_dim]. */
 int litenn_hip_llama_get_kv(litenn_hip_llama* model, int layer, float* k, float* v);
 
+/* ---- group 3b: resident models of any registered design ----------------- */
+
+/* A resident decoder whatever its layers are.  One handle is one sequence: its caches and states
+ * belong to the tokens evaluated since the last reset.  As with litenn_hip_llama, a handle is used
+ * by one thread at a time. */
+typedef struct litenn_hip_model litenn_hip_model;
+
+/* The handle of a LLaMA decoder as a model (the same object: free it through either, once). */
+litenn_hip_model* litenn_hip_llama_model(litenn_hip_llama* model);
+
+/* Loads `path` and picks the model class from what it finds: a folder with config.json and
+ * model.safetensors (the class by config.json's "architecture"), a GGUF file or a LiteNN archive
+ * (LLaMA).  dtype BF16 (or F16) runs a model with the precisions it is served with (matrix operands
+ * and caches in 16 bits); F32 keeps every operand and cache in 32 bits.  context_length bounds the
+ * positions of a sequence; <= 0 takes the file's, or 32768 where the file has none.  What a layer
+ * with a sliding window or a recurrent state holds does not grow with it. */
+int litenn_hip_model_load(int dev, const char* path, int dtype, int32_t context_length, litenn_hip_model** out);
+
+/* A host tensor of a model under construction: matrices BFloat16 [out, in], vectors BFloat16 or Float32. */
+typedef struct litenn_hip_model_tensor
+{
+	const char* name;
+	int dtype;
+	size_t rank;
+	size_t shape[4]; /* slowest dimension first */
+	const void* data;
+} litenn_hip_model_tensor;
+
+/* The same from a configuration's text and tensors in host memory (copied to the device). */
+int litenn_hip_model_create(int dev, const char* config_json, const litenn_hip_model_tensor* tensors, size_t count,
+                            int dtype, int32_t context_length, litenn_hip_model** out);
+int litenn_hip_model_free(litenn_hip_model* model);
+/* Forgets the sequence: positions count from zero again, recurrent states are zero. */
+int litenn_hip_model_reset(litenn_hip_model* model);
+int litenn_hip_model_past(const litenn_hip_model* model);
+
+typedef struct litenn_hip_model_info
+{
+	const char* architecture; /* valid while the model lives */
+	int32_t vocab_size, context_length, dtype;
+} litenn_hip_model_info;
+int litenn_hip_model_get_info(const litenn_hip_model* model, litenn_hip_model_info* out);
+
+/* Feeds `count` tokens (host I32) behind those the model has seen.  want lists n_want places among
+ * them (in any order) whose logits go to `logits` (host f32 [n_want, vocab], in the order of want);
+ * want == NULL means every place (logits may be NULL then: none).  flags as for
+ * litenn_hip_llama_eval; a model whose dtype was chosen at load time ignores them. */
+int litenn_hip_model_eval(litenn_hip_model* model, const int32_t* tokens, size_t count, const int32_t* want,
+                          size_t n_want, float* logits, unsigned flags);
+/* litenn_hip_llama_generate for any model. */
+int litenn_hip_model_generate(litenn_hip_model* model, const int32_t* prompt, size_t n_prompt, size_t n_new,
+                              int32_t* out_tokens, unsigned flags, double* prefill_ms, double* decode_ms);
+
 /* ---- group 4: weight container readers (host side) --------------------- */
 
 /* A dependency-free reader of the GGUF container (versions 2 and 3), producing what

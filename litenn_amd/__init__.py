@@ -12,7 +12,9 @@ from .device import (HIP, DeviceTraits, HIPDeviceCount, IsHIPDeviceAvailable, Te
                      MATMUL_PRECISE)
 from .llama import LLaMA
 from .gguf import GGUFFile
+from .model import Model, create_model, load_model
 
 __all__ = ["formats", "synth", "LiteNNHipError", "LIB_PATH", "HIP", "DeviceTraits", "HIPDeviceCount",
            "IsHIPDeviceAvailable", "Tensor", "argmax", "attn_decode", "attn_decode_noalloc", "attn_rows", "flash_attn_ext", "dequantize", "get_rows_q", "kv_append",
-           "mul_mat_q", "linear_group", "rmsnorm", "rope_interleaved", "silu_mul", "MATMUL_PRECISE", "LLaMA", "GGUFFile"]
+           "mul_mat_q", "linear_group", "rmsnorm", "rope_interleaved", "silu_mul", "MATMUL_PRECISE", "LLaMA", "GGUFFile", "Model",
+           "create_model", "load_model"]

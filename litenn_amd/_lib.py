@@ -44,6 +44,17 @@ class GgufTensor(C.Structure):
     ]
 
 
+class ModelTensor(C.Structure):
+    """litenn_hip_model_tensor: a host tensor of a model under construction."""
+    _fields_ = [("name", C.c_char_p), ("dtype", C.c_int), ("rank", C.c_size_t), ("shape", C.c_size_t * 4),
+                ("data", C.c_void_p)]
+
+
+class ModelInfo(C.Structure):
+    _fields_ = [("architecture", C.c_char_p), ("vocab_size", C.c_int32), ("context_length", C.c_int32),
+                ("dtype", C.c_int32)]
+
+
 _vp, _sz, _i, _u, _d = C.c_void_p, C.c_size_t, C.c_int, C.c_uint, C.c_double
 _szp = C.POINTER(C.c_size_t)
 _ex = C.POINTER(Exec)
@@ -92,6 +103,15 @@ SIGNATURES = {
     "litenn_hip_llama_eval": [_vp, _vp, _sz, _vp, _vp, _u],
     "litenn_hip_llama_generate": [_vp, _vp, _sz, _sz, _vp, _u, C.POINTER(_d), C.POINTER(_d)],
     "litenn_hip_llama_get_kv": [_vp, _i, _vp, _vp],
+    "litenn_hip_llama_model": [_vp],
+    "litenn_hip_model_load": [_i, C.c_char_p, _i, C.c_int32, C.POINTER(_vp)],
+    "litenn_hip_model_create": [_i, C.c_char_p, C.POINTER(ModelTensor), _sz, _i, C.c_int32, C.POINTER(_vp)],
+    "litenn_hip_model_free": [_vp],
+    "litenn_hip_model_reset": [_vp],
+    "litenn_hip_model_past": [_vp],
+    "litenn_hip_model_get_info": [_vp, C.POINTER(ModelInfo)],
+    "litenn_hip_model_eval": [_vp, _vp, _sz, _vp, _sz, _vp, _u],
+    "litenn_hip_model_generate": [_vp, _vp, _sz, _sz, _vp, _u, C.POINTER(_d), C.POINTER(_d)],
     "litenn_gguf_open": [C.c_char_p, C.POINTER(_vp)],
     "litenn_gguf_close": [_vp],
     "litenn_gguf_version": [_vp],
@@ -109,7 +129,7 @@ SIGNATURES = {
     "litenn_hip_llama_load_gguf": [_i, C.c_char_p, _i, C.c_int32, C.POINTER(_vp)],
 }
 _RESTYPES = {
-    "litenn_hip_last_error": C.c_char_p, "litenn_hip_mul_mat_q_workspace_bytes": C.c_size_t,
+    "litenn_hip_last_error": C.c_char_p, "litenn_hip_llama_model": C.c_void_p, "litenn_hip_mul_mat_q_workspace_bytes": C.c_size_t,
     "litenn_gguf_close": None, "litenn_gguf_version": C.c_uint, "litenn_gguf_tensor_count": C.c_size_t,
     "litenn_gguf_metadata_count": C.c_size_t, "litenn_gguf_metadata_key": C.c_char_p,
 }

@@ -14,7 +14,8 @@ LIB_PATH = os.path.join(LIB_DIR, "liblitenn_hip.so")
 # kernels of csrc/microbench.hip; only bench.py --microbench loads it
 TRACE_LIB_PATH = os.path.join(LIB_DIR, "liblitenn_hip_trace.so")
 
-SOURCES = ["api.hip", "gemv.hip", "gemm.hip", "glue.hip", "attn_tile.hip", "primitives.hip", "llama.hip", "gguf.hip"]
+SOURCES = ["api.hip", "gemv.hip", "gemm.hip", "glue.hip", "attn_tile.hip", "primitives.hip", "decoder.hip", "llama.hip", "gguf.hip",
+           "checkpoint.hip", "dense.hip", "layers.hip", "layered.hip", "registry.hip"]
 # gemv.hip: the dispatcher hands the first six kernel arguments over in registers (the streaming
 # kernel's activation pointer, K and first-row addressing), see gemv_stream_kernel
 # glue.hip: the attention step's pointers, among them the device-resident position it loads first
@@ -36,14 +37,15 @@ def hipcc() -> str:
     return exe
 
 
-def build(verbose: bool = True, jobs: int = 6) -> str:
-    """Compile every source (always, even if a library is already present) and link."""
+def build(verbose: bool = True, jobs: int = 6, measurement: bool = True) -> str:
+    """Compile every source (always, even if a library is already present) and link.  Without
+    `measurement` the timeline build of the library is left out."""
     os.makedirs(LIB_DIR, exist_ok=True)
     obj_dir = os.path.join(HERE, "build")
     os.makedirs(obj_dir, exist_ok=True)
     procs, objs = [], []
     trace_units = [("gemv.hip", "gemv_trace.o", ["-DLITENN_GEMV_TRACE"]), ("microbench.hip", "microbench.o", [])]
-    for src, obj_name, extra in [(s, s.replace(".hip", ".o"), []) for s in SOURCES] + trace_units:
+    for src, obj_name, extra in [(s, s.replace(".hip", ".o"), []) for s in SOURCES] + (trace_units if measurement else []):
         obj = os.path.join(obj_dir, obj_name)
         if not extra and src in SOURCES:
             objs.append(obj)
@@ -65,10 +67,13 @@ def build(verbose: bool = True, jobs: int = 6) -> str:
     if failed:
         raise RuntimeError("hipcc failed")
     cmd = [hipcc(), "--offload-arch=gfx950", "-shared", "-fPIC", "-fno-gpu-rdc",
-           "-Wl,--version-script=" + os.path.join(CSRC, "exports.map"), *objs, "-o", LIB_PATH]
+           "-Wl,--version-script=" + os.path.join(CSRC, "exports.map"), *objs, "-o", LIB_PATH + ".part"]
     if verbose:
         print(" ".join(cmd), flush=True)
     subprocess.check_call(cmd)
+    os.replace(LIB_PATH + ".part", LIB_PATH)  # a library that is there is whole
+    if not measurement:
+        return LIB_PATH
     trace_objs = [os.path.join(obj_dir, "gemv_trace.o") if o.endswith(os.sep + "gemv.o") else o for o in objs]
     trace_objs.append(os.path.join(obj_dir, "microbench.o"))
     cmd = [hipcc(), "--offload-arch=gfx950", "-shared", "-fPIC", "-fno-gpu-rdc",
@@ -76,6 +81,14 @@ def build(verbose: bool = True, jobs: int = 6) -> str:
     if verbose:
         print(" ".join(cmd), flush=True)
     subprocess.check_call(cmd)
+    return LIB_PATH
+
+
+def ensure_library() -> str:
+    """Build the library if there is none yet, and only it: what a program that runs a model needs in a
+    fresh checkout.  Compiler output goes to standard error."""
+    if not os.path.exists(LIB_PATH):
+        build(verbose=False, jobs=int(os.environ.get("MAX_JOBS") or 8), measurement=False)
     return LIB_PATH
 
 

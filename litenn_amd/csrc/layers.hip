@@ -1,0 +1,1433 @@
+// Mechanisms of the layered decoder for gfx950: token embedding with sinusoidal positions, the
+// residual-with-two-norms step, sliding-window attention with a sink over a latent cache (absorbed
+// form for few rows, expanded form on the matrix cores for a prompt), and gated linear attention
+// (recurrent step, and a chunked form whose contractions run on the Float32 matrix instructions).
+// Norms, positions, scores, softmax and everything inside a recurrence are Float32.  The reference
+// has no counterpart of these layers.
+#include "layers.hpp"
+
+#include <algorithm>
+#include <cmath>
+
+namespace litenn_hip
+{
+	namespace
+	{
+		typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+		typedef float floatx4 __attribute__((ext_vector_type(4)));
+		typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+
+		__device__ __forceinline__ int row_position(const Position& p, int row)
+		{
+			return (p.dev ? *p.dev : 0) + p.add + row;
+		}
+
+		// sum over a workgroup of 256
+		__device__ __forceinline__ float block_sum256(float v, float* red)
+		{
+			v = wave_sum(v);
+			__syncthreads();
+			if ((threadIdx.x & 63) == 0)
+			{
+				red[threadIdx.x >> 6] = v;
+			}
+			__syncthreads();
+			return (red[0] + red[1]) + (red[2] + red[3]);
+		}
+
+		// ---------------- embedding ----------------------------------------------------------
+		__global__ __launch_bounds__(256) void embed_rows_kernel(DenseMatrix table, const int32_t* __restrict__ ids,
+		                                                         const double* __restrict__ turns, Position pos,
+		                                                         float* __restrict__ x, int* __restrict__ err)
+		{
+			const int row = blockIdx.x;
+			const int id = ids[row];
+			if (id < 0 || id >= table.n)
+			{
+				if (threadIdx.x == 0)
+				{
+					*err = 1;
+				}
+				return;
+			}
+			const uint16_t* t = table.w + static_cast<size_t>(id) * table.pitch;
+			float* xr = x + static_cast<size_t>(row) * table.k;
+			const double p = static_cast<double>(row_position(pos, row));
+			for (int i = threadIdx.x; 2 * i < table.k; i += 256)
+			{
+				float sn = 0.0f, cs = 0.0f;
+				if (turns)
+				{
+					// the angle in turns, reduced in double: what reaches the Float32 sine is below half a turn
+					const double t0 = p * turns[i];
+					sincosf(static_cast<float>((t0 - rint(t0)) * 6.283185307179586476925), &sn, &cs);
+				}
+				xr[2 * i] = bf16_to_f32(t[2 * i]) + sn;
+				if (2 * i + 1 < table.k)
+				{
+					xr[2 * i + 1] = bf16_to_f32(t[2 * i + 1]) + cs;
+				}
+			}
+		}
+
+		// ---------------- residual and norms -------------------------------------------------
+		template <typename T>
+		__global__ __launch_bounds__(256) void add_norm_kernel(const AddNorm a)
+		{
+			__shared__ float red[4];
+			constexpr int kKept = 16; // values a thread keeps in registers (wider rows are read again)
+			const int row = blockIdx.x;
+			const float* x = a.x + static_cast<size_t>(row) * a.ldx;
+			float kept[kKept];
+			float scale_sub = 0.0f;
+			const float* sub = a.sub ? a.sub + static_cast<size_t>(row) * a.ldsub : nullptr;
+			if (sub)
+			{
+				float ss = 0.0f;
+				for (int i = threadIdx.x; i < a.width; i += 256)
+				{
+					ss = fmaf(sub[i], sub[i], ss);
+				}
+				scale_sub = 1.0f / sqrtf(block_sum256(ss, red) / static_cast<float>(a.width) + a.eps);
+			}
+			const auto value = [&](int i) { return sub ? x[i] + sub[i] * scale_sub * a.sub_w[i] : x[i]; };
+			float ss = 0.0f;
+#pragma unroll
+			for (int e = 0; e < kKept; ++e)
+			{
+				const int i = threadIdx.x + 256 * e;
+				kept[e] = i < a.width ? value(i) : 0.0f;
+				ss = fmaf(kept[e], kept[e], ss);
+			}
+			for (int i = threadIdx.x + 256 * kKept; i < a.width; i += 256)
+			{
+				const float v = value(i);
+				ss = fmaf(v, v, ss);
+			}
+			const float scale = 1.0f / sqrtf(block_sum256(ss, red) / static_cast<float>(a.width) + a.eps);
+			float* x_out = a.x_out ? a.x_out + static_cast<size_t>(row) * a.ldx : nullptr;
+			T* out = static_cast<T*>(a.out) + static_cast<size_t>(row) * a.ldo;
+			const auto put = [&](int i, float v) {
+				if (x_out)
+				{
+					x_out[i] = v;
+				}
+				operand_store(out + i, v * scale * a.norm_w[i]);
+			};
+#pragma unroll
+			for (int e = 0; e < kKept; ++e)
+			{
+				const int i = threadIdx.x + 256 * e;
+				if (i < a.width)
+				{
+					put(i, kept[e]);
+				}
+			}
+			for (int i = threadIdx.x + 256 * kKept; i < a.width; i += 256)
+			{
+				put(i, value(i));
+			}
+		}
+
+		// ---------------- latent cache -------------------------------------------------------
+		// norm(src) w -> one cache row, by 256 threads
+		template <typename T>
+		__device__ __forceinline__ void append_latent(const float* src, const float* w, float eps, const LatentCache& c,
+		                                              int position, float* red)
+		{
+			float ss = 0.0f;
+			for (int i = threadIdx.x; i < c.rank; i += 256)
+			{
+				ss = fmaf(src[i], src[i], ss);
+			}
+			const float scale = 1.0f / sqrtf(block_sum256(ss, red) / static_cast<float>(c.rank) + eps);
+			T* dst = static_cast<T*>(c.rows) + static_cast<size_t>(position % c.ring) * c.pitch;
+			for (int i = threadIdx.x; i < c.rank; i += 256)
+			{
+				operand_store(dst + i, src[i] * scale * w[i]);
+			}
+		}
+
+		template <typename T>
+		__global__ __launch_bounds__(256) void latent_append_kernel(const float* __restrict__ src, int ld,
+		                                                            const float* __restrict__ w, float eps, Position pos,
+		                                                            LatentCache cache)
+		{
+			__shared__ float red[4];
+			append_latent<T>(src + static_cast<size_t>(blockIdx.x) * ld, w, eps, cache,
+			                 row_position(pos, static_cast<int>(blockIdx.x)), red);
+		}
+
+		// ---------------- attention in the latent space (few rows) -----------------------------
+		constexpr int kAbsorbSlice = 128; // latent columns of a workgroup
+
+		// absorbed[row, h, :] = scale W_uk[h]^T q[row, h]; the last workgroup of a row appends its latent
+		template <typename T>
+		__global__ __launch_bounds__(256) void latent_absorb_kernel(const LatentStep a)
+		{
+			__shared__ float qs[256];
+			__shared__ float sums[16][kAbsorbSlice + 4];
+			__shared__ float red[4];
+			const int row = blockIdx.y;
+			const int slices = (a.cache.pitch + kAbsorbSlice - 1) / kAbsorbSlice;
+			const int h = static_cast<int>(blockIdx.x) / slices;
+			if (h == a.shape.heads)
+			{
+				if (a.latent)
+				{
+					append_latent<T>(a.latent + static_cast<size_t>(row) * a.ldl, a.latent_w, a.eps, a.cache,
+					                 row_position(a.pos, row), red);
+				}
+				return;
+			}
+			const int slice = static_cast<int>(blockIdx.x) % slices;
+			const int piece = threadIdx.x & 15, group = threadIdx.x >> 4;
+			const int r0 = slice * kAbsorbSlice + piece * 8;
+			const bool inside = r0 < a.cache.pitch;
+			const float* q = a.q + static_cast<size_t>(row) * a.ldq + static_cast<size_t>(h) * a.shape.dim;
+			float acc[8];
+#pragma unroll
+			for (int e = 0; e < 8; ++e)
+			{
+				acc[e] = 0.0f;
+			}
+			for (int first = 0; first < a.shape.dim; first += 256)
+			{
+				const int count = min(256, a.shape.dim - first);
+				__syncthreads();
+				if (static_cast<int>(threadIdx.x) < count)
+				{
+					qs[threadIdx.x] = q[first + threadIdx.x];
+				}
+				__syncthreads();
+				if (inside)
+				{
+					const uint16_t* w = a.uk.w + static_cast<size_t>(h * a.shape.dim + first) * a.uk.pitch + r0;
+#pragma unroll 4
+					for (int d = group; d < count; d += 16)
+					{
+						const u32x4 v = *reinterpret_cast<const u32x4*>(w + static_cast<size_t>(d) * a.uk.pitch);
+						const float qd = qs[d];
+#pragma unroll
+						for (int e = 0; e < 4; ++e)
+						{
+							acc[2 * e] = fmaf(qd, __uint_as_float(v[e] << 16), acc[2 * e]);
+							acc[2 * e + 1] = fmaf(qd, __uint_as_float(v[e] & 0xffff0000u), acc[2 * e + 1]);
+						}
+					}
+				}
+			}
+#pragma unroll
+			for (int e = 0; e < 8; ++e)
+			{
+				sums[group][piece * 8 + e] = acc[e];
+			}
+			__syncthreads();
+			const int r = slice * kAbsorbSlice + static_cast<int>(threadIdx.x);
+			if (threadIdx.x < kAbsorbSlice && r < a.cache.pitch)
+			{
+				float t = 0.0f;
+#pragma unroll
+				for (int g = 0; g < 16; ++g)
+				{
+					t += sums[g][threadIdx.x];
+				}
+				a.absorbed[(static_cast<size_t>(row) * a.shape.heads + h) * a.cache.pitch + r] = t * a.shape.scale;
+			}
+		}
+
+		// A workgroup takes four heads (one per wavefront) over one split of the visible positions, in tiles
+		// of kLatentTile cached rows staged in LDS as Float32; per split and head it leaves the running
+		// maximum, the sum of weights and the weighted sum of latents.
+		constexpr int kLatentTile = 32, kLatentHeads = 4, kLatentMaxRank = 1024;
+
+		template <typename T>
+		__global__ __launch_bounds__(256) void latent_step_kernel(const LatentStep a)
+		{
+			extern __shared__ __attribute__((aligned(16))) float latent_lds[];
+			const int pitch = a.cache.pitch, stride = pitch + 4;
+			float* const tile = latent_lds;                       // [kLatentTile][stride]
+			float* const qa = tile + kLatentTile * stride;        // [kLatentHeads][pitch]
+			float* const weights = qa + kLatentHeads * pitch;     // [kLatentHeads][kLatentTile]
+			const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+			const int row = blockIdx.z, split = blockIdx.y;
+			const int h = static_cast<int>(blockIdx.x) * kLatentHeads + wave;
+			const int hc = min(h, a.shape.heads - 1);
+			const float* src = a.absorbed + (static_cast<size_t>(row) * a.shape.heads + hc) * pitch;
+			for (int i = lane; i < pitch; i += 64)
+			{
+				qa[wave * pitch + i] = i < a.cache.rank ? src[i] : 0.0f;
+			}
+			const int last = row_position(a.pos, row);
+			const int first = max(0, last - a.shape.window + 1);
+			const int tiles = (last - first) / kLatentTile + 1;
+			const int per = (tiles + a.splits - 1) / a.splits;
+			const int t0 = split * per, t1 = min(tiles, t0 + per);
+			const T* const cache = static_cast<const T*>(a.cache.rows);
+
+			constexpr int kCols = kLatentMaxRank / 256;
+			floatx4 o[kCols];
+#pragma unroll
+			for (int c = 0; c < kCols; ++c)
+			{
+				o[c] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+			}
+			float run_m = -INFINITY, run_l = 0.0f;
+			for (int t = t0; t < t1; ++t)
+			{
+				const int base = first + t * kLatentTile;
+				const int count = min(kLatentTile, last - base + 1);
+				__syncthreads();
+				// rows past the last one are never stored: their weight is zero and they are skipped below
+				for (int i = threadIdx.x; i < kLatentTile * (pitch >> 2); i += 256)
+				{
+					const int key = i / (pitch >> 2), c = (i % (pitch >> 2)) * 4;
+					const T* p = cache + static_cast<size_t>((base + min(key, count - 1)) % a.cache.ring) * pitch + c;
+					floatx4 v;
+					if constexpr (sizeof(T) == 2)
+					{
+						const uint2 w = *reinterpret_cast<const uint2*>(p);
+						v = floatx4{ __uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u), __uint_as_float(w.y << 16),
+							         __uint_as_float(w.y & 0xffff0000u) };
+					}
+					else
+					{
+						v = *reinterpret_cast<const floatx4*>(p);
+					}
+					*reinterpret_cast<floatx4*>(&tile[key * stride + c]) = v;
+				}
+				__syncthreads();
+				// scores: two lanes per key, each half of the latent
+				const int key = lane & 31, part = lane >> 5;
+				float acc = 0.0f;
+				{
+					const float* kr = &tile[key * stride];
+					const float* qr = &qa[wave * pitch];
+					const int half = pitch >> 1;
+					for (int c = part * half; c < (part + 1) * half; c += 4)
+					{
+						const floatx4 kv = *reinterpret_cast<const floatx4*>(kr + c);
+						const floatx4 qv = *reinterpret_cast<const floatx4*>(qr + c);
+						acc = fmaf(kv.x, qv.x, acc);
+						acc = fmaf(kv.y, qv.y, acc);
+						acc = fmaf(kv.z, qv.z, acc);
+						acc = fmaf(kv.w, qv.w, acc);
+					}
+				}
+				acc += __shfl_xor(acc, 32, 64);
+				const float score = key < count ? acc : -INFINITY;
+				const float new_m = fmaxf(run_m, wave_max(score));
+				const float corr = run_m == -INFINITY ? 0.0f : expf(run_m - new_m);
+				const float p = expf(score - new_m);
+				run_l = run_l * corr + 0.5f * wave_sum(p); // every key is held by two lanes
+				run_m = new_m;
+				if (part == 0)
+				{
+					weights[wave * kLatentTile + key] = p;
+				}
+				// written and read by this wavefront only, in order
+				__builtin_amdgcn_wave_barrier();
+#pragma unroll
+				for (int c = 0; c < kCols; ++c)
+				{
+					o[c] *= corr;
+				}
+				for (int kk = 0; kk < count; ++kk)
+				{
+					const float w = weights[wave * kLatentTile + kk];
+#pragma unroll
+					for (int c = 0; c < kCols; ++c)
+					{
+						const int col = c * 256 + lane * 4;
+						if (col < pitch)
+						{
+							o[c] += w * *reinterpret_cast<const floatx4*>(&tile[kk * stride + col]);
+						}
+					}
+				}
+			}
+			if (h >= a.shape.heads)
+			{
+				return;
+			}
+			const size_t slot = (static_cast<size_t>(row) * a.splits + split) * a.shape.heads + h;
+			float* dst = a.partial + slot * (pitch + 4);
+#pragma unroll
+			for (int c = 0; c < kCols; ++c)
+			{
+				const int col = c * 256 + lane * 4;
+				if (col < pitch)
+				{
+					*reinterpret_cast<floatx4*>(dst + col) = o[c];
+				}
+			}
+			if (lane == 0)
+			{
+				dst[pitch] = run_m;
+				dst[pitch + 1] = run_l;
+			}
+		}
+
+		// Merges the splits (and the sink), takes the result through W_uv, applies the gate.  A workgroup
+		// makes kValueSlice outputs of one head.
+		constexpr int kValueSlice = 32;
+
+		template <typename T>
+		__global__ __launch_bounds__(256) void latent_value_kernel(const LatentStep a)
+		{
+			__shared__ __attribute__((aligned(16))) float o[kLatentMaxRank];
+			const int pitch = a.cache.pitch;
+			const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+			const int slices = (a.shape.vdim + kValueSlice - 1) / kValueSlice;
+			const int h = static_cast<int>(blockIdx.x) / slices, slice = static_cast<int>(blockIdx.x) % slices;
+			const int row = blockIdx.y;
+			const size_t step = static_cast<size_t>(a.shape.heads) * (pitch + 4);
+			const float* part = a.partial + (static_cast<size_t>(row) * a.splits * a.shape.heads + h) * (pitch + 4);
+			float top = a.shape.sink ? a.shape.sink[h] : -INFINITY;
+			for (int s = 0; s < a.splits; ++s)
+			{
+				top = fmaxf(top, part[s * step + pitch]);
+			}
+			float total = a.shape.sink ? expf(a.shape.sink[h] - top) : 0.0f;
+			float v[kLatentMaxRank / 256];
+#pragma unroll
+			for (int c = 0; c < kLatentMaxRank / 256; ++c)
+			{
+				v[c] = 0.0f;
+			}
+			for (int s = 0; s < a.splits; ++s)
+			{
+				const float m = part[s * step + pitch];
+				if (m == -INFINITY)
+				{
+					continue; // a split without a visible position
+				}
+				const float w = expf(m - top);
+				total = fmaf(w, part[s * step + pitch + 1], total);
+#pragma unroll
+				for (int c = 0; c < kLatentMaxRank / 256; ++c)
+				{
+					const int col = c * 256 + static_cast<int>(threadIdx.x);
+					if (col < a.cache.rank)
+					{
+						v[c] = fmaf(w, part[s * step + col], v[c]);
+					}
+				}
+			}
+			const float inv = 1.0f / total;
+#pragma unroll
+			for (int c = 0; c < kLatentMaxRank / 256; ++c)
+			{
+				o[c * 256 + threadIdx.x] = v[c] * inv;
+			}
+			__syncthreads();
+			for (int i = wave; i < kValueSlice; i += 4)
+			{
+				const int e = slice * kValueSlice + i;
+				if (e >= a.shape.vdim)
+				{
+					break;
+				}
+				const uint16_t* w = a.uv.w + static_cast<size_t>(h * a.shape.vdim + e) * a.uv.pitch;
+				float acc = 0.0f;
+				for (int r = lane * 8; r < pitch; r += 512)
+				{
+					const u32x4 x = *reinterpret_cast<const u32x4*>(w + r);
+					const floatx4 o0 = *reinterpret_cast<const floatx4*>(o + r);
+					const floatx4 o1 = *reinterpret_cast<const floatx4*>(o + r + 4);
+					acc = fmaf(__uint_as_float(x.x << 16), o0.x, acc);
+					acc = fmaf(__uint_as_float(x.x & 0xffff0000u), o0.y, acc);
+					acc = fmaf(__uint_as_float(x.y << 16), o0.z, acc);
+					acc = fmaf(__uint_as_float(x.y & 0xffff0000u), o0.w, acc);
+					acc = fmaf(__uint_as_float(x.z << 16), o1.x, acc);
+					acc = fmaf(__uint_as_float(x.z & 0xffff0000u), o1.y, acc);
+					acc = fmaf(__uint_as_float(x.w << 16), o1.z, acc);
+					acc = fmaf(__uint_as_float(x.w & 0xffff0000u), o1.w, acc);
+				}
+				acc = wave_sum(acc);
+				if (lane == 0)
+				{
+					const int col = h * a.shape.vdim + e;
+					if (a.gate)
+					{
+						acc *= sigmoid_f32(a.gate[static_cast<size_t>(row) * a.ldg + col]);
+					}
+					operand_store(static_cast<T*>(a.out) + static_cast<size_t>(row) * a.ldo + col, acc);
+				}
+			}
+		}
+
+		// ---------------- windowed attention over expanded keys and values -----------------------
+		// One wavefront per (query row, head), any head size up to 1024; Float32 arithmetic.
+		constexpr int kRowAttnMaxDim = 1024;
+
+		template <typename T>
+		__global__ __launch_bounds__(64) void window_attn_row_kernel(const WindowAttn a)
+		{
+			__shared__ float qs[kRowAttnMaxDim];
+			__shared__ float ws[64];
+			const int row = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+			const int dim = a.shape.dim, vdim = a.shape.vdim;
+			for (int d = lane; d < dim; d += 64)
+			{
+				qs[d] = a.q[static_cast<size_t>(row) * a.ldq + h * dim + d];
+			}
+			__syncthreads();
+			const int pos = a.q_base + row;
+			const int first = max(a.key_base, pos - a.shape.window + 1), last = min(pos, a.key_base + a.keys - 1);
+			const T* kv = static_cast<const T*>(a.kv);
+			constexpr int kCols = kRowAttnMaxDim / 64;
+			float o[kCols];
+#pragma unroll
+			for (int c = 0; c < kCols; ++c)
+			{
+				o[c] = 0.0f;
+			}
+			float run_m = -INFINITY, run_l = 0.0f;
+			for (int base = first; base <= last; base += 64)
+			{
+				const int key = base + lane;
+				float score = -INFINITY;
+				if (key <= last)
+				{
+					const T* k = kv + static_cast<size_t>(key - a.key_base) * a.ldkv + h * dim;
+					float acc = 0.0f;
+					for (int d = 0; d < dim; ++d)
+					{
+						acc = fmaf(qs[d], operand_load(k + d), acc);
+					}
+					score = acc * a.shape.scale;
+				}
+				const float new_m = fmaxf(run_m, wave_max(score));
+				const float corr = run_m == -INFINITY ? 0.0f : expf(run_m - new_m);
+				const float p = key <= last ? expf(score - new_m) : 0.0f;
+				run_l = run_l * corr + wave_sum(p);
+				run_m = new_m;
+				__syncthreads();
+				ws[lane] = p;
+				__syncthreads();
+				const int count = min(64, last - base + 1);
+#pragma unroll
+				for (int c = 0; c < kCols; ++c)
+				{
+					const int e = c * 64 + lane;
+					if (e < vdim)
+					{
+						float t = o[c] * corr;
+						const T* v = kv + static_cast<size_t>(base - a.key_base) * a.ldkv + a.v_first + h * vdim + e;
+						for (int i = 0; i < count; ++i)
+						{
+							t = fmaf(ws[i], operand_load(v + static_cast<size_t>(i) * a.ldkv), t);
+						}
+						o[c] = t;
+					}
+				}
+			}
+			float top = run_m, total = run_l, weight = 1.0f;
+			if (a.shape.sink)
+			{
+				const float sink = a.shape.sink[h];
+				top = fmaxf(run_m, sink);
+				weight = expf(run_m - top);
+				total = run_l * weight + expf(sink - top);
+			}
+#pragma unroll
+			for (int c = 0; c < kCols; ++c)
+			{
+				const int e = c * 64 + lane;
+				if (e < vdim)
+				{
+					float v = o[c] * weight / total;
+					if (a.gate)
+					{
+						v *= sigmoid_f32(a.gate[static_cast<size_t>(row) * a.ldg + h * vdim + e]);
+					}
+					operand_store(static_cast<T*>(a.out) + static_cast<size_t>(row) * a.ldo + h * vdim + e, v);
+				}
+			}
+		}
+
+		// Matrix-core form: a workgroup takes 64 query rows of one head (16 per wavefront) and walks the
+		// keys any of them sees in tiles of 64, staged in LDS (keys row-major, values transposed).  Both
+		// products are formed transposed (keys x queries, value dimensions x queries), so that a query
+		// stays in one lane column: the softmax weights leave the first product in the register layout
+		// the second one takes, and the running maximum and sum live beside the outputs.  DK and DV are the
+		// head sizes rounded up; what lies beyond the true sizes is zero in LDS and in the queries.
+		constexpr int kWinQ = 64, kWinKeys = 64, kWinVStride = 72;
+
+		template <int DK, int DV>
+		__global__ __launch_bounds__(256) void window_attn_tile_kernel(const WindowAttn a)
+		{
+			constexpr int KS = DK + 8;
+			extern __shared__ __attribute__((aligned(16))) uint16_t win_lds[];
+			uint16_t* const k_lds = win_lds;                 // [kWinKeys][KS]
+			uint16_t* const v_lds = win_lds + kWinKeys * KS; // [DV][kWinVStride]
+			const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+			const int j = lane & 15, g = lane >> 4;
+			const int h = blockIdx.x;
+			const int tile = static_cast<int>(gridDim.y) - 1 - static_cast<int>(blockIdx.y);
+			const int dim = a.shape.dim, vdim = a.shape.vdim;
+			const int q_first = tile * kWinQ;
+			const int my_q = q_first + 16 * wave + j;
+			const int my_row = min(my_q, a.rows - 1);
+			const int my_pos = a.q_base + my_row;
+			// key rows (relative to key_base) any query of the tile sees
+			const int lo = max(0, a.q_base + q_first - a.shape.window + 1 - a.key_base);
+			const int hi = min(a.keys, a.q_base + min(q_first + kWinQ, a.rows) - a.key_base);
+			const uint16_t* const kv = static_cast<const uint16_t*>(a.kv);
+
+			bf16x8 q_frag[DK / 32];
+			{
+				const float* q = a.q + static_cast<size_t>(my_row) * a.ldq + static_cast<size_t>(h) * dim;
+#pragma unroll
+				for (int st = 0; st < DK / 32; ++st)
+				{
+					uint32_t w[4];
+#pragma unroll
+					for (int e = 0; e < 4; ++e)
+					{
+						const int d = 32 * st + 8 * g + 2 * e; // dim is a multiple of 8
+						w[e] = d < dim ? pack_bf16(q[d], q[d + 1]) : 0u;
+					}
+					q_frag[st] = __builtin_bit_cast(bf16x8, u32x4{ w[0], w[1], w[2], w[3] });
+				}
+			}
+			floatx4 o[DV / 16];
+#pragma unroll
+			for (int b = 0; b < DV / 16; ++b)
+			{
+				o[b] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+			}
+			float run_m = -INFINITY, run_l = 0.0f;
+			constexpr int KP = DK / 8, VP = DV / 8;              // 16-byte pieces of a row
+			constexpr int KN = kWinKeys * KP / 256, VN = VP / 4; // pieces a thread stages
+			u32x4 kr[KN], vr[VN];
+			const int v_key = tid & 63, v_piece = (tid >> 6) * VN;
+			const auto request = [&](int base) {
+#pragma unroll
+				for (int i = 0; i < KN; ++i)
+				{
+					const int c = tid + 256 * i, key = min(base + c / KP, hi - 1), d = (c % KP) * 8;
+					kr[i] = d < dim ? *reinterpret_cast<const u32x4*>(kv + static_cast<size_t>(key) * a.ldkv + h * dim + d)
+					                : u32x4{ 0u, 0u, 0u, 0u };
+				}
+				const uint16_t* v = kv + static_cast<size_t>(min(base + v_key, hi - 1)) * a.ldkv + a.v_first + h * vdim;
+#pragma unroll
+				for (int i = 0; i < VN; ++i)
+				{
+					const int e = (v_piece + i) * 8;
+					vr[i] = e < vdim ? *reinterpret_cast<const u32x4*>(v + e) : u32x4{ 0u, 0u, 0u, 0u };
+				}
+			};
+			request(lo);
+			for (int base = lo; base < hi; base += kWinKeys)
+			{
+				__syncthreads(); // the previous tile has been consumed
+#pragma unroll
+				for (int i = 0; i < KN; ++i)
+				{
+					const int c = tid + 256 * i;
+					*reinterpret_cast<u32x4*>(&k_lds[(c / KP) * KS + (c % KP) * 8]) = kr[i];
+				}
+#pragma unroll
+				for (int i = 0; i < VN; ++i)
+				{
+#pragma unroll
+					for (int e = 0; e < 4; ++e)
+					{
+						const int d = (v_piece + i) * 8 + 2 * e;
+						v_lds[d * kWinVStride + v_key] = static_cast<uint16_t>(vr[i][e] & 0xffffu);
+						v_lds[(d + 1) * kWinVStride + v_key] = static_cast<uint16_t>(vr[i][e] >> 16);
+					}
+				}
+				if (base + kWinKeys < hi)
+				{
+					request(base + kWinKeys);
+				}
+				__syncthreads();
+				// lane (j, g) gets keys base + 16 b + 4 g + 0..3 of query j
+				floatx4 s[4];
+#pragma unroll
+				for (int b = 0; b < 4; ++b)
+				{
+					s[b] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+#pragma unroll
+					for (int st = 0; st < DK / 32; ++st)
+					{
+						const bf16x8 kf = *reinterpret_cast<const bf16x8*>(&k_lds[(16 * b + j) * KS + 32 * st + 8 * g]);
+						s[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, q_frag[st], s[b], 0, 0, 0);
+					}
+				}
+				const int pos0 = a.key_base + base + 4 * g;
+				float sv[4][4];
+				float top = -INFINITY;
+#pragma unroll
+				for (int b = 0; b < 4; ++b)
+				{
+#pragma unroll
+					for (int r = 0; r < 4; ++r)
+					{
+						const int back = my_pos - (pos0 + 16 * b + r);
+						sv[b][r] = back >= 0 && back < a.shape.window ? s[b][r] * a.shape.scale : -INFINITY;
+						top = fmaxf(top, sv[b][r]);
+					}
+				}
+				top = fmaxf(top, __shfl_xor(top, 16, 64));
+				top = fmaxf(top, __shfl_xor(top, 32, 64));
+				// a tile may hold no visible key of this query: exponents then take 0 as the maximum
+				const float new_m = fmaxf(run_m, top);
+				const float ref_m = new_m == -INFINITY ? 0.0f : new_m;
+				const float corr = expf(run_m - ref_m);
+				run_m = new_m;
+				float sum = 0.0f;
+				bf16x8 p_frag[2];
+#pragma unroll
+				for (int ks = 0; ks < 2; ++ks)
+				{
+					float p[8];
+#pragma unroll
+					for (int r = 0; r < 4; ++r)
+					{
+						p[r] = expf(sv[2 * ks][r] - ref_m);
+						p[4 + r] = expf(sv[2 * ks + 1][r] - ref_m);
+					}
+#pragma unroll
+					for (int e = 0; e < 8; ++e)
+					{
+						sum += p[e];
+					}
+					p_frag[ks] = __builtin_bit_cast(bf16x8, u32x4{ pack_bf16(p[0], p[1]), pack_bf16(p[2], p[3]),
+					                                               pack_bf16(p[4], p[5]), pack_bf16(p[6], p[7]) });
+				}
+				run_l = fmaf(run_l, corr, sum);
+				// contraction index 8 g + e of step ks stands for key 16 (2 ks) + 4 g + e (e < 4) and key
+				// 16 (2 ks + 1) + 4 g + e - 4 (e >= 4)
+#pragma unroll
+				for (int b = 0; b < DV / 16; ++b)
+				{
+					o[b] *= corr;
+#pragma unroll
+					for (int ks = 0; ks < 2; ++ks)
+					{
+						const uint16_t* col = &v_lds[(16 * b + j) * kWinVStride + 32 * ks + 4 * g];
+						const uint2 x = *reinterpret_cast<const uint2*>(col), y = *reinterpret_cast<const uint2*>(col + 16);
+						const bf16x8 vf = __builtin_bit_cast(bf16x8, u32x4{ x.x, x.y, y.x, y.y });
+						o[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, p_frag[ks], o[b], 0, 0, 0);
+					}
+				}
+			}
+			run_l += __shfl_xor(run_l, 16, 64);
+			run_l += __shfl_xor(run_l, 32, 64);
+			if (my_q >= a.rows)
+			{
+				return;
+			}
+			float weight = 1.0f, total = run_l;
+			if (a.shape.sink)
+			{
+				const float sink = a.shape.sink[h];
+				const float all_m = fmaxf(run_m, sink);
+				weight = expf(run_m - all_m);
+				total = run_l * weight + expf(sink - all_m);
+			}
+			const float inv = weight / total;
+			uint16_t* out = static_cast<uint16_t*>(a.out) + static_cast<size_t>(my_q) * a.ldo + static_cast<size_t>(h) * vdim;
+			const float* gate = a.gate ? a.gate + static_cast<size_t>(my_q) * a.ldg + static_cast<size_t>(h) * vdim : nullptr;
+#pragma unroll
+			for (int b = 0; b < DV / 16; ++b)
+			{
+				const int e = 16 * b + 4 * g; // vdim is a multiple of 8
+				if (e < vdim)
+				{
+					floatx4 v = o[b] * inv;
+					if (gate)
+					{
+#pragma unroll
+						for (int r = 0; r < 4; ++r)
+						{
+							v[r] *= sigmoid_f32(gate[e + r]);
+						}
+					}
+					*reinterpret_cast<uint2*>(out + e) = make_uint2(pack_bf16(v.x, v.y), pack_bf16(v.z, v.w));
+				}
+			}
+		}
+
+		// ---------------- gated linear attention ---------------------------------------------------
+		__device__ __forceinline__ float log_sigmoid_f32(float z)
+		{
+			return fminf(z, 0.0f) - log1pf(expf(-fabsf(z)));
+		}
+
+		// one row of W_a2 times the rank-wide vector `a1`
+		__device__ __forceinline__ float low_rank_dot(const DenseMatrix& a2, int channel, const float* a1)
+		{
+			const uint16_t* w = a2.w + static_cast<size_t>(channel) * a2.pitch;
+			float z = 0.0f;
+			for (int r = 0; r < a2.k; ++r)
+			{
+				z = fmaf(bf16_to_f32(w[r]), a1[r], z);
+			}
+			return z;
+		}
+
+		// log_decay[t, c] = log sigmoid(W_a2 a1[t] + bias)[c] / tau
+		constexpr int kDecayRows = 16, kDecayMaxRank = 512;
+
+		__global__ __launch_bounds__(256) void gla_decay_kernel(const Gla a)
+		{
+			__shared__ float a1[kDecayRows][kDecayMaxRank];
+			const int channels = a.shape.heads * a.shape.dim, rank = a.a2.k;
+			const int row0 = blockIdx.y * kDecayRows;
+			const int count = min(kDecayRows, a.rows - row0);
+			for (int i = threadIdx.x; i < count * rank; i += 256)
+			{
+				a1[i / rank][i % rank] = a.a1[static_cast<size_t>(row0 + i / rank) * a.ld + i % rank];
+			}
+			__syncthreads();
+			const int c = blockIdx.x * 256 + threadIdx.x;
+			if (c >= channels)
+			{
+				return;
+			}
+			const uint16_t* w = a.a2.w + static_cast<size_t>(c) * a.a2.pitch;
+			float z[kDecayRows];
+			const float bias = a.a2_bias[c];
+#pragma unroll
+			for (int t = 0; t < kDecayRows; ++t)
+			{
+				z[t] = bias;
+			}
+			for (int r = 0; r < rank; ++r)
+			{
+				const float wr = bf16_to_f32(w[r]);
+#pragma unroll
+				for (int t = 0; t < kDecayRows; ++t)
+				{
+					z[t] = fmaf(wr, a1[t][r], z[t]);
+				}
+			}
+#pragma unroll
+			for (int t = 0; t < kDecayRows; ++t)
+			{
+				if (t < count)
+				{
+					a.log_decay[static_cast<size_t>(row0 + t) * channels + c] = log_sigmoid_f32(z[t]) * a.shape.inv_tau;
+				}
+			}
+		}
+
+		// One token: S <- diag(alpha) S + k v^T, o = S^T q.  A workgroup takes kStepCols value columns of one
+		// head; a thread holds RPT rows (32 apart) of four columns.
+		constexpr int kStepCols = 32, kGlaMaxDim = 512;
+
+		template <int RPT>
+		__global__ __launch_bounds__(256) void gla_step_kernel(const Gla a)
+		{
+			__shared__ float alpha[32 * RPT], ks[32 * RPT], qs[32 * RPT];
+			__shared__ __attribute__((aligned(16))) float sums[32][kStepCols + 4];
+			const int dim = a.shape.dim, vdim = a.shape.vdim, pitch = gla_state_pitch(vdim);
+			const int h = blockIdx.x, tid = threadIdx.x;
+			const int e = static_cast<int>(blockIdx.y) * kStepCols + (tid & 7) * 4;
+			const int d0 = tid >> 3;
+			const bool inside = e < pitch;
+			float* const state = a.state + static_cast<size_t>(h) * dim * pitch + e;
+			floatx4 st[RPT];
+#pragma unroll
+			for (int i = 0; i < RPT; ++i)
+			{
+				const int d = d0 + 32 * i;
+				st[i] = inside && d < dim ? *reinterpret_cast<const floatx4*>(state + static_cast<size_t>(d) * pitch)
+				                          : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+			}
+			floatx4 v = { 0.0f, 0.0f, 0.0f, 0.0f };
+#pragma unroll
+			for (int i = 0; i < 4; ++i)
+			{
+				v[i] = e + i < vdim ? a.v[h * vdim + e + i] : 0.0f;
+			}
+			for (int d = tid; d < dim; d += 256)
+			{
+				const int c = h * dim + d;
+				alpha[d] = expf(log_sigmoid_f32(low_rank_dot(a.a2, c, a.a1) + a.a2_bias[c]) * a.shape.inv_tau);
+				ks[d] = a.k[c];
+				qs[d] = a.q[c] * a.shape.q_scale;
+			}
+			__syncthreads();
+			floatx4 acc = { 0.0f, 0.0f, 0.0f, 0.0f };
+#pragma unroll
+			for (int i = 0; i < RPT; ++i)
+			{
+				const int d = d0 + 32 * i;
+				if (d < dim)
+				{
+					st[i] = st[i] * alpha[d] + v * ks[d];
+					acc += st[i] * qs[d];
+					if (inside)
+					{
+						*reinterpret_cast<floatx4*>(state + static_cast<size_t>(d) * pitch) = st[i];
+					}
+				}
+			}
+			*reinterpret_cast<floatx4*>(&sums[d0][(tid & 7) * 4]) = acc;
+			__syncthreads();
+			const int col = static_cast<int>(blockIdx.y) * kStepCols + tid;
+			if (tid < kStepCols && col < vdim)
+			{
+				float t = 0.0f;
+#pragma unroll
+				for (int i = 0; i < 32; ++i)
+				{
+					t += sums[i][tid];
+				}
+				a.o[h * vdim + col] = t;
+			}
+		}
+
+		// ---- chunked form -------------------------------------------------------------------------
+		// Tokens in chunks of 64, a chunk in four blocks of 16.  With L_t the sum of a channel's log decays
+		// up to and including token t, every factor below is exp of a sum of log decays over some run of
+		// tokens, so none exceeds one whatever the decays are:
+		//   contribution of a chunk to the state:  sum_s (k_s exp(L_end - L_s)) v_s^T
+		//   o_t = (q_t exp(L_t - L_begin)) S_begin
+		//         + sum over earlier blocks of ((q_t exp(L_t - L_block)) . (k_s exp(L_block - L_s))) v_s
+		//         + inside t's own block  sum_s (sum_d q_td k_sd exp(L_td - L_sd)) v_s,
+		// L_block being L before the first token of t's block.  The contractions run on
+		// v_mfma_f32_16x16x4_f32; the own-block term is formed pair by pair.
+		constexpr int kChunk = 64, kSlab = 64, kSlabStride = 68;
+
+		// chunk_states: [chunk][head][dim][pitch] floats, then [chunk][head][dim] decays over the chunk
+		__device__ __forceinline__ float* chunk_decays(const Gla& a, int chunks)
+		{
+			return a.chunk_states +
+			       static_cast<size_t>(chunks) * a.shape.heads * a.shape.dim * gla_state_pitch(a.shape.vdim);
+		}
+
+		template <int NE>
+		__global__ __launch_bounds__(256) void gla_state_kernel(const Gla a)
+		{
+			__shared__ float ks[kChunk][kSlabStride];
+			__shared__ float totals[4][kSlab];
+			const int dim = a.shape.dim, vdim = a.shape.vdim, pitch = gla_state_pitch(vdim), heads = a.shape.heads;
+			const int slabs = (dim + kSlab - 1) / kSlab;
+			const int h = static_cast<int>(blockIdx.x) / slabs, d0 = static_cast<int>(blockIdx.x) % slabs * kSlab;
+			const int chunk = blockIdx.y, row0 = chunk * kChunk, count = min(kChunk, a.rows - row0);
+			const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+			{
+				// thread: one channel, 16 tokens
+				const int c = lane, part = wave;
+				const bool live = d0 + c < dim;
+				const size_t channel = static_cast<size_t>(h) * dim + d0 + (live ? c : 0);
+				float la[16], total = 0.0f;
+#pragma unroll
+				for (int t = 0; t < 16; ++t)
+				{
+					const int row = 16 * part + t;
+					la[t] = live && row < count ? a.log_decay[static_cast<size_t>(row0 + row) * heads * dim + channel] : 0.0f;
+					total += la[t];
+				}
+				totals[part][c] = total;
+				__syncthreads();
+				float after = 0.0f;
+				for (int p = part + 1; p < 4; ++p)
+				{
+					after += totals[p][c];
+				}
+#pragma unroll
+				for (int t = 15; t >= 0; --t)
+				{
+					const int row = 16 * part + t;
+					const float k = live && row < count ? a.k[static_cast<size_t>(row0 + row) * a.ld + channel] : 0.0f;
+					ks[row][c] = k * expf(after);
+					after += la[t];
+				}
+				if (part == 0 && live)
+				{
+					chunk_decays(a, gridDim.y)[(static_cast<size_t>(chunk) * heads + h) * dim + d0 + c] = expf(after);
+				}
+			}
+			__syncthreads();
+			const int j = lane & 15, g = lane >> 4;
+			floatx4 acc[NE];
+#pragma unroll
+			for (int n = 0; n < NE; ++n)
+			{
+				acc[n] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+			}
+#pragma unroll 4
+			for (int step = 0; step < kChunk / 4; ++step)
+			{
+				const int t = 4 * step + g;
+				const float kf = ks[t][16 * wave + j];
+				const float* v = a.v + static_cast<size_t>(row0 + min(t, count - 1)) * a.ld + h * vdim;
+#pragma unroll
+				for (int n = 0; n < NE; ++n)
+				{
+					const int e = 16 * n + j;
+					acc[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf, e < vdim ? v[e] : 0.0f, acc[n], 0, 0, 0);
+				}
+			}
+			float* dst = a.chunk_states + (static_cast<size_t>(chunk) * heads + h) * dim * pitch;
+#pragma unroll
+			for (int n = 0; n < NE; ++n)
+			{
+#pragma unroll
+				for (int r = 0; r < 4; ++r)
+				{
+					const int d = d0 + 16 * wave + 4 * g + r, e = 16 * n + j;
+					if (d < dim && e < pitch)
+					{
+						dst[static_cast<size_t>(d) * pitch + e] = acc[n][r];
+					}
+				}
+			}
+		}
+
+		// replaces every chunk's contribution by the state the chunk begins with; ends with the new state
+		__global__ __launch_bounds__(256) void gla_scan_kernel(const Gla a, int chunks)
+		{
+			const int pitch = gla_state_pitch(a.shape.vdim), quads = pitch >> 2;
+			const int rows = a.shape.heads * a.shape.dim;
+			const int i = static_cast<int>(blockIdx.x) * 256 + static_cast<int>(threadIdx.x);
+			if (i >= rows * quads)
+			{
+				return;
+			}
+			const int row = i / quads;
+			const size_t at = static_cast<size_t>(row) * pitch + static_cast<size_t>(i % quads) * 4;
+			const size_t step = static_cast<size_t>(rows) * pitch;
+			const float* decay = chunk_decays(a, chunks) + row;
+			floatx4 s = *reinterpret_cast<floatx4*>(a.state + at);
+			constexpr int kAhead = 4;
+			for (int c0 = 0; c0 < chunks; c0 += kAhead)
+			{
+				floatx4 in[kAhead];
+				float dec[kAhead];
+#pragma unroll
+				for (int u = 0; u < kAhead; ++u)
+				{
+					const int c = min(c0 + u, chunks - 1);
+					in[u] = *reinterpret_cast<floatx4*>(a.chunk_states + c * step + at);
+					dec[u] = decay[static_cast<size_t>(c) * rows];
+				}
+#pragma unroll
+				for (int u = 0; u < kAhead; ++u)
+				{
+					if (c0 + u < chunks)
+					{
+						*reinterpret_cast<floatx4*>(a.chunk_states + (c0 + u) * step + at) = s;
+						s = s * dec[u] + in[u];
+					}
+				}
+			}
+			*reinterpret_cast<floatx4*>(a.state + at) = s;
+		}
+
+		template <int NE, typename T>
+		__global__ __launch_bounds__(256) void gla_out_kernel(const Gla a)
+		{
+			__shared__ __attribute__((aligned(16))) float qs[kChunk][kSlabStride];
+			__shared__ __attribute__((aligned(16))) float ks[kChunk][kSlabStride];
+			__shared__ __attribute__((aligned(16))) float ls[kChunk][kSlabStride]; // log decays summed from the block's first token
+			__shared__ __attribute__((aligned(16))) float totals[4][kSlab];        // a block's whole sum
+			const int dim = a.shape.dim, vdim = a.shape.vdim, pitch = gla_state_pitch(vdim), heads = a.shape.heads;
+			const int h = blockIdx.x, chunk = blockIdx.y;
+			const int row0 = chunk * kChunk, count = min(kChunk, a.rows - row0);
+			const int tid = threadIdx.x, lane = tid & 63;
+			const int wave = __builtin_amdgcn_readfirstlane(tid >> 6); // = the block of 16 tokens it makes
+			const int j = lane & 15, g = lane >> 4;
+			const float* state = a.chunk_states + (static_cast<size_t>(chunk) * heads + h) * dim * pitch;
+
+			floatx4 o[NE];      // o[n][r]: value column 16 n + 4 g + r of token j of the block
+			floatx4 scores[4];  // scores[b][r]: token 4 g + r of block b against token j
+#pragma unroll
+			for (int n = 0; n < NE; ++n)
+			{
+				o[n] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+			}
+#pragma unroll
+			for (int b = 0; b < 4; ++b)
+			{
+				scores[b] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+			}
+			for (int d0 = 0; d0 < dim; d0 += kSlab)
+			{
+				__syncthreads();
+				{
+					const int c = lane;
+					const bool live = d0 + c < dim;
+					const size_t channel = static_cast<size_t>(h) * dim + d0 + (live ? c : 0);
+					float sum = 0.0f;
+#pragma unroll
+					for (int t = 0; t < 16; ++t)
+					{
+						const int row = 16 * wave + t;
+						const bool in = live && row < count;
+						const size_t at = static_cast<size_t>(row0 + row) * a.ld + channel;
+						sum += in ? a.log_decay[static_cast<size_t>(row0 + row) * heads * dim + channel] : 0.0f;
+						ls[row][c] = sum;
+						qs[row][c] = in ? a.q[at] * a.shape.q_scale : 0.0f;
+						ks[row][c] = in ? a.k[at] : 0.0f;
+					}
+					totals[wave][c] = sum;
+				}
+				__syncthreads();
+#pragma unroll
+				for (int quad = 0; quad < kSlab / 16; ++quad)
+				{
+					const int c = 16 * quad + 4 * g; // this lane's four channels of the slab
+					floatx4 qv = *reinterpret_cast<const floatx4*>(&qs[16 * wave + j][c]);
+					const floatx4 lq = *reinterpret_cast<const floatx4*>(&ls[16 * wave + j][c]);
+#pragma unroll
+					for (int r = 0; r < 4; ++r)
+					{
+						qv[r] *= expf(lq[r]);
+					}
+					// earlier blocks, the nearest first: `between` is the decay over the blocks in between
+					floatx4 between = { 0.0f, 0.0f, 0.0f, 0.0f };
+#pragma unroll
+					for (int back = 1; back < 4; ++back)
+					{
+						const int b = wave - back; // uniform
+						if (b >= 0)
+						{
+							const floatx4 kv = *reinterpret_cast<const floatx4*>(&ks[16 * b + j][c]);
+							const floatx4 lk = *reinterpret_cast<const floatx4*>(&ls[16 * b + j][c]);
+							const floatx4 tot = *reinterpret_cast<const floatx4*>(&totals[b][c]);
+							floatx4 sc = scores[back];
+#pragma unroll
+							for (int r = 0; r < 4; ++r)
+							{
+								sc = __builtin_amdgcn_mfma_f32_16x16x4f32(kv[r] * expf(tot[r] - lk[r] + between[r]), qv[r], sc, 0, 0, 0);
+							}
+							scores[back] = sc;
+							between += tot;
+						}
+					}
+					// the state the chunk begins with (`between` now spans all earlier blocks of the chunk)
+#pragma unroll
+					for (int r = 0; r < 4; ++r)
+					{
+						const float qi = qv[r] * expf(between[r]);
+						const int d = min(d0 + c + r, dim - 1); // qi is zero beyond
+						const float* sr = state + static_cast<size_t>(d) * pitch;
+#pragma unroll
+						for (int n = 0; n < NE; ++n)
+						{
+							const int e = 16 * n + j;
+							o[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(e < pitch ? sr[e] : 0.0f, qi, o[n], 0, 0, 0);
+						}
+					}
+				}
+				// own block, pair by pair: token j against tokens 4 g + r
+				for (int c = 0; c < kSlab; c += 4)
+				{
+					const floatx4 qv = *reinterpret_cast<const floatx4*>(&qs[16 * wave + j][c]);
+					const floatx4 lq = *reinterpret_cast<const floatx4*>(&ls[16 * wave + j][c]);
+#pragma unroll
+					for (int r = 0; r < 4; ++r)
+					{
+						const floatx4 kv = *reinterpret_cast<const floatx4*>(&ks[16 * wave + 4 * g + r][c]);
+						const floatx4 lk = *reinterpret_cast<const floatx4*>(&ls[16 * wave + 4 * g + r][c]);
+						float sc = scores[0][r];
+#pragma unroll
+						for (int x = 0; x < 4; ++x)
+						{
+							sc = fmaf(qv[x] * kv[x], expf(fminf(lq[x] - lk[x], 0.0f)), sc);
+						}
+						scores[0][r] = sc;
+					}
+				}
+			}
+#pragma unroll
+			for (int r = 0; r < 4; ++r)
+			{
+				scores[0][r] = 4 * g + r <= j ? scores[0][r] : 0.0f;
+			}
+			// o += scores . v; scores[back] belongs to block wave - back
+#pragma unroll
+			for (int back = 0; back < 4; ++back)
+			{
+				const int b = wave - back;
+				if (b >= 0)
+				{
+#pragma unroll
+					for (int r = 0; r < 4; ++r)
+					{
+						const int s = min(16 * b + 4 * g + r, count - 1); // scores are zero beyond
+						const float* v = a.v + static_cast<size_t>(row0 + s) * a.ld + h * vdim;
+#pragma unroll
+						for (int n = 0; n < NE; ++n)
+						{
+							const int e = 16 * n + j;
+							o[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(e < vdim ? v[e] : 0.0f, scores[back][r], o[n], 0, 0, 0);
+						}
+					}
+				}
+			}
+			// head norm and gate
+			float ss = 0.0f;
+#pragma unroll
+			for (int n = 0; n < NE; ++n)
+			{
+#pragma unroll
+				for (int r = 0; r < 4; ++r)
+				{
+					o[n][r] = 16 * n + 4 * g + r < vdim ? o[n][r] : 0.0f;
+					ss = fmaf(o[n][r], o[n][r], ss);
+				}
+			}
+			ss += __shfl_xor(ss, 16, 64);
+			ss += __shfl_xor(ss, 32, 64);
+			const int row = 16 * wave + j;
+			if (row >= count)
+			{
+				return;
+			}
+			const float scale = 1.0f / sqrtf(ss / static_cast<float>(vdim) + a.eps);
+			const float* gate = a.gate + static_cast<size_t>(row0 + row) * a.ld + h * vdim;
+			T* out = static_cast<T*>(a.out) + static_cast<size_t>(row0 + row) * a.ldo + h * vdim;
+#pragma unroll
+			for (int n = 0; n < NE; ++n)
+			{
+#pragma unroll
+				for (int r = 0; r < 4; ++r)
+				{
+					const int e = 16 * n + 4 * g + r;
+					if (e < vdim)
+					{
+						const float z = gate[e];
+						operand_store(out + e, o[n][r] * scale * a.norm_w[e] * (z * sigmoid_f32(z)));
+					}
+				}
+			}
+		}
+
+		template <int DK, int DV>
+		void launch_window_tile(const WindowAttn& a, hipStream_t s)
+		{
+			constexpr size_t lds = sizeof(uint16_t) * (kWinKeys * (DK + 8) + DV * kWinVStride);
+			allow_dynamic_lds(reinterpret_cast<const void*>(&window_attn_tile_kernel<DK, DV>), lds);
+			window_attn_tile_kernel<DK, DV>
+			    <<<dim3(a.shape.heads, (a.rows + kWinQ - 1) / kWinQ), dim3(256), lds, s>>>(a);
+		}
+
+		template <int DK>
+		void launch_window_tile(const WindowAttn& a, hipStream_t s)
+		{
+			if (a.shape.vdim <= 64)
+			{
+				launch_window_tile<DK, 64>(a, s);
+			}
+			else if (a.shape.vdim <= 128)
+			{
+				launch_window_tile<DK, 128>(a, s);
+			}
+			else
+			{
+				launch_window_tile<DK, 256>(a, s);
+			}
+		}
+
+		template <int NE>
+		void launch_gla_chunks(const Gla& a, int chunks, hipStream_t s)
+		{
+			const int slabs = (a.shape.dim + kSlab - 1) / kSlab;
+			gla_state_kernel<NE><<<dim3(a.shape.heads * slabs, chunks), dim3(256), 0, s>>>(a);
+			const int quads = a.shape.heads * a.shape.dim * (gla_state_pitch(a.shape.vdim) >> 2);
+			gla_scan_kernel<<<dim3((quads + 255) / 256), dim3(256), 0, s>>>(a, chunks);
+			if (a.f32)
+			{
+				gla_out_kernel<NE, float><<<dim3(a.shape.heads, chunks), dim3(256), 0, s>>>(a);
+			}
+			else
+			{
+				gla_out_kernel<NE, uint16_t><<<dim3(a.shape.heads, chunks), dim3(256), 0, s>>>(a);
+			}
+		}
+
+		size_t latent_step_lds(int pitch)
+		{
+			return sizeof(float) * (static_cast<size_t>(kLatentTile) * (pitch + 4) + static_cast<size_t>(kLatentHeads) * pitch +
+			                        kLatentHeads * kLatentTile);
+		}
+	} // namespace
+
+	void launch_embed_rows(const DenseMatrix& table, const int32_t* ids, int rows, const double* turns, Position pos,
+	                       float* x, int* err, hipStream_t s)
+	{
+		if (rows > 0)
+		{
+			embed_rows_kernel<<<dim3(rows), dim3(256), 0, s>>>(table, ids, turns, pos, x, err);
+		}
+	}
+
+	void launch_add_norm(const AddNorm& a, hipStream_t s)
+	{
+		if (a.rows <= 0)
+		{
+			return;
+		}
+		if (a.f32)
+		{
+			add_norm_kernel<float><<<dim3(a.rows), dim3(256), 0, s>>>(a);
+		}
+		else
+		{
+			add_norm_kernel<uint16_t><<<dim3(a.rows), dim3(256), 0, s>>>(a);
+		}
+	}
+
+	void launch_latent_append(const float* src, int ld, const float* norm_w, float eps, int rows, Position pos,
+	                          const LatentCache& cache, hipStream_t s)
+	{
+		if (rows <= 0)
+		{
+			return;
+		}
+		if (cache.f32)
+		{
+			latent_append_kernel<float><<<dim3(rows), dim3(256), 0, s>>>(src, ld, norm_w, eps, pos, cache);
+		}
+		else
+		{
+			latent_append_kernel<uint16_t><<<dim3(rows), dim3(256), 0, s>>>(src, ld, norm_w, eps, pos, cache);
+		}
+	}
+
+	int latent_step_max_rank() { return kLatentMaxRank; }
+
+	// about two workgroups per CU, and no split shorter than a tile
+	int latent_step_splits(int heads, int rows, int window)
+	{
+		const int groups = (heads + kLatentHeads - 1) / kLatentHeads * rows;
+		const int tiles = (window + kLatentTile - 1) / kLatentTile;
+		return std::max(1, std::min({ tiles, 512 / std::max(1, groups), 64 }));
+	}
+
+	size_t latent_step_partial_floats(int heads, int rows, int pitch, int splits)
+	{
+		return static_cast<size_t>(heads) * rows * splits * (pitch + 4);
+	}
+
+	void launch_latent_step(const LatentStep& a, hipStream_t s)
+	{
+		const int slices = (a.cache.pitch + kAbsorbSlice - 1) / kAbsorbSlice;
+		const dim3 absorb(a.shape.heads * slices + 1, a.rows);
+		const dim3 attend((a.shape.heads + kLatentHeads - 1) / kLatentHeads, a.splits, a.rows);
+		const size_t lds = latent_step_lds(a.cache.pitch);
+		if (a.cache.f32)
+		{
+			latent_absorb_kernel<float><<<absorb, dim3(256), 0, s>>>(a);
+			allow_dynamic_lds(reinterpret_cast<const void*>(&latent_step_kernel<float>), latent_step_lds(kLatentMaxRank));
+			latent_step_kernel<float><<<attend, dim3(256), lds, s>>>(a);
+		}
+		else
+		{
+			latent_absorb_kernel<uint16_t><<<absorb, dim3(256), 0, s>>>(a);
+			allow_dynamic_lds(reinterpret_cast<const void*>(&latent_step_kernel<uint16_t>), latent_step_lds(kLatentMaxRank));
+			latent_step_kernel<uint16_t><<<attend, dim3(256), lds, s>>>(a);
+		}
+		const dim3 value(a.shape.heads * ((a.shape.vdim + kValueSlice - 1) / kValueSlice), a.rows);
+		if (a.out_f32)
+		{
+			latent_value_kernel<float><<<value, dim3(256), 0, s>>>(a);
+		}
+		else
+		{
+			latent_value_kernel<uint16_t><<<value, dim3(256), 0, s>>>(a);
+		}
+	}
+
+	void launch_window_attn(const WindowAttn& a, hipStream_t s)
+	{
+		if (a.rows <= 0)
+		{
+			return;
+		}
+		const dim3 rows(a.rows, a.shape.heads);
+		if (a.f32)
+		{
+			window_attn_row_kernel<float><<<rows, dim3(64), 0, s>>>(a);
+			return;
+		}
+		// whole 16-byte pieces of a head's keys and values
+		const bool pieces = a.shape.dim % 8 == 0 && a.shape.vdim % 8 == 0 && a.ldkv % 8 == 0 && a.v_first % 8 == 0 &&
+		                    a.ldo % 4 == 0 && a.shape.dim <= 256 && a.shape.vdim <= 256;
+		if (!pieces)
+		{
+			window_attn_row_kernel<uint16_t><<<rows, dim3(64), 0, s>>>(a);
+		}
+		else if (a.shape.dim <= 64)
+		{
+			launch_window_tile<64>(a, s);
+		}
+		else if (a.shape.dim <= 128)
+		{
+			launch_window_tile<128>(a, s);
+		}
+		else
+		{
+			launch_window_tile<256>(a, s);
+		}
+	}
+
+	int gla_max_dim() { return kGlaMaxDim; }
+	int gla_max_vdim() { return 256; }
+
+	size_t gla_chunk_floats(int rows, int heads, int dim, int vdim)
+	{
+		const size_t chunks = (static_cast<size_t>(rows) + kChunk - 1) / kChunk;
+		return chunks * heads * dim * (static_cast<size_t>(gla_state_pitch(vdim)) + 1);
+	}
+
+	void launch_gla_step(const Gla& a, hipStream_t s)
+	{
+		const dim3 grid(a.shape.heads, (a.shape.vdim + kStepCols - 1) / kStepCols);
+		const int rpt = (a.shape.dim + 31) / 32;
+		if (rpt <= 2)
+		{
+			gla_step_kernel<2><<<grid, dim3(256), 0, s>>>(a);
+		}
+		else if (rpt <= 4)
+		{
+			gla_step_kernel<4><<<grid, dim3(256), 0, s>>>(a);
+		}
+		else if (rpt <= 8)
+		{
+			gla_step_kernel<8><<<grid, dim3(256), 0, s>>>(a);
+		}
+		else
+		{
+			gla_step_kernel<16><<<grid, dim3(256), 0, s>>>(a);
+		}
+	}
+
+	void launch_gla_rows(const Gla& a, hipStream_t s)
+	{
+		if (a.rows <= 0)
+		{
+			return;
+		}
+		const int channels = a.shape.heads * a.shape.dim;
+		gla_decay_kernel<<<dim3((channels + 255) / 256, (a.rows + kDecayRows - 1) / kDecayRows), dim3(256), 0, s>>>(a);
+		const int chunks = (a.rows + kChunk - 1) / kChunk;
+		const int ne = (a.shape.vdim + 15) / 16;
+		if (ne <= 2)
+		{
+			launch_gla_chunks<2>(a, chunks, s);
+		}
+		else if (ne <= 4)
+		{
+			launch_gla_chunks<4>(a, chunks, s);
+		}
+		else if (ne <= 8)
+		{
+			launch_gla_chunks<8>(a, chunks, s);
+		}
+		else
+		{
+			launch_gla_chunks<16>(a, chunks, s);
+		}
+	}
+} // namespace litenn_hip

@@ -5,9 +5,9 @@
 // (tools/gguf/LLaMABuilder.cpp:826-872, src/LiteNN/Runtime/Interpreter.h:89-104,325-329).
 // Here the same operator sequence (LLaMABuilder.cpp:568-668,774-800) runs as a fixed list of
 // kernel launches over weights that stay in their .gguf block layout in HBM, with a
-// preallocated KV cache, the current length kept in device memory, and the single-token
-// step captured once into a HIP graph so that a greedy loop never returns to the host.
-#include "common.hpp"
+// preallocated KV cache and the current length kept in device memory.  The token loops around
+// it (evaluation, and the greedy loop over a captured single-token step) are decoder.hip's.
+#include "decoder.hpp"
 
 #include <algorithm>
 #include <cmath>
@@ -70,22 +70,10 @@ namespace litenn_hip
 	                        float* out, size_t splits, float* partial, int* counters, hipStream_t s);
 	void launch_silu_mul(const float* gate, const float* up, float* y, size_t n, hipStream_t s);
 	void launch_argmax(const float* x, size_t rows, size_t n, int32_t* out, hipStream_t s);
-	size_t argmax_step_scratch_bytes(size_t n);
-	void launch_argmax_step(const float* x, size_t n, void* scratch, int32_t* next, int* counters, int past_inc,
-	                        int32_t* out, hipStream_t s);
 	bool launch_convert(int src_dtype, const void* src, size_t n, int dst_dtype, void* dst, hipStream_t s);
 
 	namespace
 	{
-		// counters[0] = past length, counters[1] = tokens emitted so far, counters[2] = steps this model
-		// has run (never reset: it names a step in the values its workgroups hand to each other)
-		__global__ void set_counters_kernel(int* counters, int past, int emitted)
-		{
-			counters[0] = past;
-			counters[1] = emitted;
-			counters[2] += 1;
-		}
-
 		struct Weight
 		{
 			int fmt = 0;
@@ -106,32 +94,22 @@ namespace litenn_hip
 
 using namespace litenn_hip;
 
-struct litenn_hip_llama
+struct litenn_hip_llama : litenn_hip_model
 {
-	int dev = 0;
 	litenn_hip_llama_params p{};
 	int head_dim = 0;
 	Weight tok_embd, output;
 	const float* output_norm = nullptr;
 	std::vector<Layer> layers;
-	hipStream_t stream = nullptr;
 	float* cos_t = nullptr; // [context_length, rope_dims/2]
 	float* sin_t = nullptr;
 	// activations for `cap_rows` rows
-	size_t cap_rows = 0, cap_logit_rows = 0;
+	size_t cap_rows = 0;
 	float *x = nullptr, *xn = nullptr, *q = nullptr, *k = nullptr, *v = nullptr, *attn = nullptr, *gate = nullptr,
-	      *gate2 = nullptr, *up = nullptr, *logits = nullptr;
+	      *gate2 = nullptr, *up = nullptr;
 	size_t xn_floats = 0; // what xn holds (rows x embedding_length, three times that for short prompts)
 	void* xh = nullptr; // fp16 copy of a matmul's activations (multi-row path), 16-row padded
 	size_t xh_halves = 0; // its size: room for the widest matmul, and for two copies of the embedding width
-	void* argmax_scratch = nullptr; // per-chunk (value, index) pairs of the vocabulary arg-max
-	std::vector<void*> owned; // device buffers freed with the model (tensors uploaded by the GGUF loader)
-	int32_t* d_tokens = nullptr;
-	int32_t* d_next = nullptr; // token produced by the last arg-max
-	int32_t* d_out = nullptr;  // generated tokens
-	size_t cap_out = 0;
-	int* d_counters = nullptr; // {past, emitted, steps run}
-	int* d_err = nullptr;
 	// single-row attention: key chunks per head, their meeting place and arrival counters
 	size_t attn_splits = 1;
 	float* attn_partial = nullptr;
@@ -143,9 +121,13 @@ struct litenn_hip_llama
 	unsigned* blk_flags = nullptr; // [2][256] tags of the launch's two meetings
 	float* blk_partial = nullptr; // [8][embedding_length] the launch's result, one vector per team
 	int blk_spins = 8192;         // polls a wait inside the launch may take before it gives up
-	int past = 0;
-	hipGraphExec_t step_exec = nullptr;
-	hipGraph_t step_graph = nullptr;
+
+	~litenn_hip_llama() override;
+	int check_complete() override;
+	int ensure_rows(size_t rows) override;
+	void prepare() override;
+	void forward(const int32_t* ids, size_t rows, size_t logit_rows, unsigned flags, int past) override;
+	bool give_up_waiting() override;
 };
 
 namespace
@@ -163,11 +145,6 @@ namespace
 				*b = nullptr;
 			}
 		}
-		if (m->d_tokens)
-		{
-			(void)hipFree(m->d_tokens);
-			m->d_tokens = nullptr;
-		}
 		if (m->xh)
 		{
 			(void)hipFree(m->xh);
@@ -176,21 +153,7 @@ namespace
 		m->cap_rows = 0;
 	}
 
-	void drop_graph(litenn_hip_llama* m)
-	{
-		if (m->step_exec)
-		{
-			(void)hipGraphExecDestroy(m->step_exec);
-			m->step_exec = nullptr;
-		}
-		if (m->step_graph)
-		{
-			(void)hipGraphDestroy(m->step_graph);
-			m->step_graph = nullptr;
-		}
-	}
-
-	int ensure_rows(litenn_hip_llama* m, size_t rows, size_t logit_rows)
+	int ensure_scratch(litenn_hip_llama* m, size_t rows)
 	{
 		const size_t d = m->p.embedding_length;
 		const size_t qw = static_cast<size_t>(m->p.head_count) * m->head_dim;
@@ -198,7 +161,7 @@ namespace
 		const size_t ff = m->p.feed_forward_length;
 		if (rows > m->cap_rows)
 		{
-			drop_graph(m); // the captured step references the old buffers
+			decoder_drop_graph(m); // the captured step references the old buffers
 			free_scratch(m);
 			// xn also takes the products of K's later ranges when a GEMM on few weight rows walks K in up to
 			// four ranges at once: room for three, for prompts where that is used
@@ -211,28 +174,15 @@ namespace
 			{
 				LITENN_HIP_TRY(kAction, hipMalloc(reinterpret_cast<void**>(b.p), sizeof(float) * rows * b.n));
 			}
-			LITENN_HIP_TRY(kAction, hipMalloc(reinterpret_cast<void**>(&m->d_tokens), sizeof(int32_t) * rows));
 			// (q/k/v projections in two formats share a launch that wants the rows in both fragment orders)
 			m->xh_halves = std::max(gemm_scratch_halves(rows, std::max({ d, qw, ff })), 2 * gemm_scratch_halves(rows, d));
 			LITENN_HIP_TRY(kAction, hipMalloc(&m->xh, 2 * m->xh_halves));
 			m->cap_rows = rows;
 		}
-		if (logit_rows > m->cap_logit_rows)
-		{
-			drop_graph(m);
-			if (m->logits)
-			{
-				(void)hipFree(m->logits);
-				m->logits = nullptr;
-			}
-			LITENN_HIP_TRY(kAction, hipMalloc(reinterpret_cast<void**>(&m->logits),
-			                                  sizeof(float) * logit_rows * static_cast<size_t>(m->p.vocab_size)));
-			m->cap_logit_rows = logit_rows;
-		}
 		return 0;
 	}
 
-	int check_complete(const litenn_hip_llama* m)
+	int check_tensors(const litenn_hip_llama* m)
 	{
 		if (!m->tok_embd.data || !m->output_norm)
 		{
@@ -500,7 +450,7 @@ namespace
 
 	// Enqueues the decoder over `rows` tokens whose ids are at `ids` (device); positions start at
 	// counters[0].  Logits are produced for the last `logit_rows` rows into m->logits.
-	void forward(litenn_hip_llama* m, const int32_t* ids, size_t rows, size_t logit_rows, unsigned flags)
+	void forward_rows(litenn_hip_llama* m, const int32_t* ids, size_t rows, size_t logit_rows, unsigned flags)
 	{
 		static const bool fuse_token = !(getenv("LITENN_HIP_FUSE") && getenv("LITENN_HIP_FUSE")[0] == '0');
 		if (rows == 1 && logit_rows == 1 && fuse_token)
@@ -572,26 +522,6 @@ namespace
 		matmul(m, head, m->xn, logit_rows, m->logits, nullptr, nullptr, flags, s);
 	}
 
-	constexpr int kBlockWaitRanOut = -2;
-
-	int check_error_flag(litenn_hip_llama* m)
-	{
-		int flag = 0;
-		LITENN_HIP_TRY(kAction, hipMemcpyAsync(&flag, m->d_err, sizeof(int), hipMemcpyDeviceToHost, m->stream));
-		LITENN_HIP_TRY(kAction, hipStreamSynchronize(m->stream));
-		if (flag)
-		{
-			const int zero = 0;
-			(void)hipMemcpy(m->d_err, &zero, sizeof(int), hipMemcpyHostToDevice);
-			if (flag & 2)
-			{
-				return kBlockWaitRanOut;
-			}
-			return fail(kAction, "GetRows index out of range");
-		}
-		return 0;
-	}
-
 	// A wait inside the one-launch attention half ran out (its workgroups were not all running at
 	// once: the card was shared, or is not the one the launch is shaped for).  What that step
 	// computed is void; the model takes the separate launches from now on and the caller repeats
@@ -599,9 +529,30 @@ namespace
 	void give_up_block_launch(litenn_hip_llama* m)
 	{
 		m->block_fused = -1;
-		drop_graph(m);
+		decoder_drop_graph(m);
 	}
 } // namespace
+
+int litenn_hip_llama::check_complete() { return check_tensors(this); }
+
+int litenn_hip_llama::ensure_rows(size_t rows) { return ensure_scratch(this, rows); }
+
+void litenn_hip_llama::prepare() { (void)block_fused_ready(this); }
+
+void litenn_hip_llama::forward(const int32_t* ids, size_t rows, size_t logit_rows, unsigned flags, int)
+{
+	forward_rows(this, ids, rows, logit_rows, flags);
+}
+
+bool litenn_hip_llama::give_up_waiting()
+{
+	if (block_fused <= 0)
+	{
+		return false;
+	}
+	give_up_block_launch(this);
+	return true;
+}
 
 namespace
 {
@@ -683,6 +634,11 @@ int llama_create_impl(int dev, const litenn_hip_llama_params* params, litenn_hip
 	}
 	m = new litenn_hip_llama();
 	m->dev = dev;
+	m->action = kAction;
+	m->architecture = "llama";
+	m->vocab = p.vocab_size;
+	m->context_length = p.context_length;
+	m->dtype = p.kv_dtype;
 	m->p = p;
 	m->p.rope_dimension_count = rope_dims;
 	m->head_dim = head_dim;
@@ -692,13 +648,9 @@ int llama_create_impl(int dev, const litenn_hip_llama_params* params, litenn_hip
 		m = nullptr;
 		return fail_hip(kAction, e);
 	};
-	// Non-blocking: a stream that synchronises with the legacy default stream would, while its
-	// decode step is being captured, make every default-stream call of another host thread fail
-	// ("would make the legacy stream depend on a capturing blocking stream").
-	hipError_t e = hipStreamCreateWithFlags(&m->stream, hipStreamNonBlocking);
+	hipError_t e = decoder_init(m);
 	if (e != hipSuccess)
 	{
-		m->stream = nullptr;
 		return bail(e);
 	}
 	const size_t kv_bytes = static_cast<size_t>(p.context_length) * p.head_count_kv * head_dim * dtype_size(p.kv_dtype);
@@ -738,19 +690,6 @@ int llama_create_impl(int dev, const litenn_hip_llama_params* params, litenn_hip
 			return bail(e);
 		}
 	}
-	if ((e = hipMalloc(reinterpret_cast<void**>(&m->d_counters), 4 * sizeof(int))) != hipSuccess ||
-	    (e = hipMalloc(reinterpret_cast<void**>(&m->d_err), sizeof(int))) != hipSuccess ||
-	    (e = hipMalloc(reinterpret_cast<void**>(&m->d_next), sizeof(int32_t))) != hipSuccess ||
-	    (e = hipMemsetAsync(m->d_counters, 0, 4 * sizeof(int), m->stream)) != hipSuccess ||
-	    (e = hipMemsetAsync(m->d_err, 0, sizeof(int), m->stream)) != hipSuccess ||
-	    (e = hipMemsetAsync(m->d_next, 0, sizeof(int32_t), m->stream)) != hipSuccess)
-	{
-		return bail(e);
-	}
-	if ((e = hipMalloc(&m->argmax_scratch, argmax_step_scratch_bytes(static_cast<size_t>(p.vocab_size)))) != hipSuccess)
-	{
-		return bail(e);
-	}
 	m->attn_splits = attn_splits(1, static_cast<size_t>(p.context_length), static_cast<size_t>(p.head_count));
 	if (m->attn_splits > 1)
 	{
@@ -783,27 +722,10 @@ namespace litenn_hip
 	}
 } // namespace litenn_hip
 
-extern "C" int litenn_hip_llama_free(litenn_hip_llama* m)
+litenn_hip_llama::~litenn_hip_llama()
 {
-	if (!m)
-	{
-		return 0;
-	}
-	DeviceGuard guard(m->dev);
-	if (m->stream)
-	{
-		(void)hipStreamSynchronize(m->stream);
-	}
-	drop_graph(m);
-	free_scratch(m);
-	for (void* p : { static_cast<void*>(m->blk_triples), static_cast<void*>(m->blk_flags), static_cast<void*>(m->blk_partial) })
-	{
-		if (p)
-		{
-			(void)hipFree(p);
-		}
-	}
-	for (Layer& L : m->layers)
+	free_scratch(this);
+	for (Layer& L : layers)
 	{
 		if (L.kcache)
 		{
@@ -814,13 +736,7 @@ extern "C" int litenn_hip_llama_free(litenn_hip_llama* m)
 			(void)hipFree(L.vcache);
 		}
 	}
-	for (void* ptr : m->owned)
-	{
-		(void)hipFree(ptr);
-	}
-	void* singles[] = { m->cos_t, m->sin_t,      m->logits,       m->d_next,       m->d_out,
-	                    m->d_counters, m->d_err, m->attn_partial, m->attn_counters,
-	                    m->argmax_scratch };
+	void* singles[] = { blk_triples, blk_flags, blk_partial, cos_t, sin_t, attn_partial, attn_counters };
 	for (void* ptr : singles)
 	{
 		if (ptr)
@@ -828,11 +744,16 @@ extern "C" int litenn_hip_llama_free(litenn_hip_llama* m)
 			(void)hipFree(ptr);
 		}
 	}
-	if (m->stream)
+}
+
+extern "C" litenn_hip_model* litenn_hip_llama_model(litenn_hip_llama* m) { return m; }
+
+extern "C" int litenn_hip_llama_free(litenn_hip_llama* m)
+{
+	if (m)
 	{
-		(void)hipStreamDestroy(m->stream);
+		decoder_free(m);
 	}
-	delete m;
 	return 0;
 }
 
@@ -884,7 +805,7 @@ extern "C" int litenn_hip_llama_set_tensor(litenn_hip_llama* m, int which, int l
 		{
 			L->ffn_norm = static_cast<const float*>(data);
 		}
-		drop_graph(m);
+		decoder_drop_graph(m);
 		return 0;
 	default:
 		return fail(kAction, "unknown tensor id");
@@ -901,19 +822,14 @@ extern "C" int litenn_hip_llama_set_tensor(litenn_hip_llama* m, int which, int l
 	target->data = data;
 	target->n = n;
 	target->k = k;
-	drop_graph(m);
+	decoder_drop_graph(m);
 	m->block_fused = 0; // decided again with the new tensor
 	return 0;
 }
 
 extern "C" int litenn_hip_llama_reset(litenn_hip_llama* m)
 {
-	if (!m)
-	{
-		return fail(kAction, "null argument");
-	}
-	m->past = 0;
-	return 0;
+	return m ? decoder_reset(m) : fail(kAction, "null argument");
 }
 
 extern "C" int litenn_hip_llama_past(const litenn_hip_llama* m)
@@ -933,67 +849,7 @@ extern "C" int litenn_hip_llama_eval(litenn_hip_llama* m, const int32_t* tokens,
 	{
 		return fail(kAction, "null argument");
 	}
-	if (rows == 0)
-	{
-		return fail(kAction, "sequence length must be positive");
-	}
-	if (static_cast<size_t>(m->past) + rows > static_cast<size_t>(m->p.context_length))
-	{
-		return fail(kAction, "context length exceeded");
-	}
-	if (check_complete(m) != 0)
-	{
-		return 1;
-	}
-	for (size_t i = 0; i < rows; ++i)
-	{
-		if (tokens[i] < 0 || tokens[i] >= m->p.vocab_size)
-		{
-			return fail(kAction, "GetRows index out of range"); // Device.h:868-871
-		}
-	}
-	DeviceGuard guard(m->dev);
-	if (!guard.ok())
-	{
-		return fail_hip(kAction, guard.error());
-	}
-	const size_t logit_rows = logits ? rows : 1;
-	if (ensure_rows(m, rows, logit_rows) != 0)
-	{
-		return 1;
-	}
-	(void)block_fused_ready(m);
-	hipStream_t s = m->stream;
-	for (int attempt = 0;; ++attempt)
-	{
-		LITENN_HIP_TRY(kAction, hipMemcpyAsync(m->d_tokens, tokens, sizeof(int32_t) * rows, hipMemcpyHostToDevice, s));
-		set_counters_kernel<<<1, 1, 0, s>>>(m->d_counters, m->past, 0);
-		forward(m, m->d_tokens, rows, logit_rows, flags);
-		LITENN_HIP_TRY(kAction, hipGetLastError());
-		const size_t vocab = m->p.vocab_size;
-		if (logits)
-		{
-			LITENN_HIP_TRY(kAction, hipMemcpyAsync(logits, m->logits, sizeof(float) * rows * vocab, hipMemcpyDeviceToHost, s));
-		}
-		if (last_logits)
-		{
-			LITENN_HIP_TRY(kAction, hipMemcpyAsync(last_logits, m->logits + (logit_rows - 1) * vocab, sizeof(float) * vocab,
-			                                       hipMemcpyDeviceToHost, s));
-		}
-		const int rc = check_error_flag(m);
-		if (rc == kBlockWaitRanOut && attempt == 0)
-		{
-			give_up_block_launch(m); // and once more through the separate launches
-			continue;
-		}
-		if (rc != 0)
-		{
-			return rc == kBlockWaitRanOut ? fail(kAction, "a wait inside the decoder step ran out") : 1;
-		}
-		break;
-	}
-	m->past += static_cast<int>(rows);
-	return 0;
+	return decoder_eval(m, tokens, rows, nullptr, 0, logits, last_logits, flags);
 }
 
 extern "C" int litenn_hip_llama_generate(litenn_hip_llama* m, const int32_t* prompt, size_t n_prompt, size_t n_new,
@@ -1003,167 +859,7 @@ extern "C" int litenn_hip_llama_generate(litenn_hip_llama* m, const int32_t* pro
 	{
 		return fail(kAction, "null argument");
 	}
-	if (n_prompt == 0 || n_new == 0)
-	{
-		return fail(kAction, "prompt and generation lengths must be positive");
-	}
-	if (static_cast<size_t>(m->past) + n_prompt + n_new - 1 > static_cast<size_t>(m->p.context_length))
-	{
-		return fail(kAction, "context length exceeded");
-	}
-	if (check_complete(m) != 0)
-	{
-		return 1;
-	}
-	for (size_t i = 0; i < n_prompt; ++i)
-	{
-		if (prompt[i] < 0 || prompt[i] >= m->p.vocab_size)
-		{
-			return fail(kAction, "GetRows index out of range");
-		}
-	}
-	DeviceGuard guard(m->dev);
-	if (!guard.ok())
-	{
-		return fail_hip(kAction, guard.error());
-	}
-	if (ensure_rows(m, n_prompt, 1) != 0)
-	{
-		return 1;
-	}
-	(void)block_fused_ready(m);
-	if (n_new > m->cap_out)
-	{
-		drop_graph(m);
-		if (m->d_out)
-		{
-			(void)hipFree(m->d_out);
-			m->d_out = nullptr;
-		}
-		LITENN_HIP_TRY(kAction, hipMalloc(reinterpret_cast<void**>(&m->d_out), sizeof(int32_t) * n_new));
-		m->cap_out = n_new;
-	}
-	hipStream_t s = m->stream;
-	// the events exist before any work is queued and are destroyed on every way out
-	hipEvent_t ev[3] = { nullptr, nullptr, nullptr };
-	auto cleanup = [&]() {
-		for (hipEvent_t& e : ev)
-		{
-			if (e)
-			{
-				(void)hipEventDestroy(e);
-				e = nullptr;
-			}
-		}
-	};
-	for (hipEvent_t& e : ev)
-	{
-		const hipError_t ce = hipEventCreate(&e);
-		if (ce != hipSuccess)
-		{
-			e = nullptr;
-			cleanup();
-			return fail_hip(kAction, ce);
-		}
-	}
-	int rc = 0;
-	// A failure part-way leaves `past` as it was: the rows a failed run appended lie beyond it, are
-	// never read (every pass takes its position from `past`) and are overwritten by the next call.
-	// The stream is drained first so that nothing of the failed run is still in flight afterwards.
-#define GEN_TRY(expr)                                                                                                  \
-	do                                                                                                                 \
-	{                                                                                                                  \
-		const hipError_t e_ = (expr);                                                                                  \
-		if (e_ != hipSuccess)                                                                                          \
-		{                                                                                                              \
-			(void)hipStreamSynchronize(s);                                                                             \
-			cleanup();                                                                                                 \
-			return fail_hip(kAction, e_);                                                                              \
-		}                                                                                                              \
-	} while (0)
-
-	// prompt: one pass over n_prompt rows, logits of the last row only, first token from its arg-max
-	GEN_TRY(hipMemcpyAsync(m->d_tokens, prompt, sizeof(int32_t) * n_prompt, hipMemcpyHostToDevice, s));
-	set_counters_kernel<<<1, 1, 0, s>>>(m->d_counters, m->past, 0);
-	GEN_TRY(hipEventRecord(ev[0], s));
-	forward(m, m->d_tokens, n_prompt, 1, flags);
-	launch_argmax_step(m->logits, m->p.vocab_size, m->argmax_scratch, m->d_next, m->d_counters,
-	                   static_cast<int>(n_prompt), m->d_out, s);
-	GEN_TRY(hipEventRecord(ev[1], s));
-	GEN_TRY(hipGetLastError());
-
-	// single-token steps: embed d_next at position counters[0], arg-max, append.  The step is
-	// captured once; every replay reads its position from device memory.
-	const char* graph_env = getenv("LITENN_HIP_GRAPH");
-	const bool use_graph = !(graph_env && graph_env[0] == '0');
-	if (n_new > 1)
-	{
-		if (use_graph && !m->step_exec)
-		{
-			GEN_TRY(hipStreamSynchronize(s));
-			hipError_t ce = hipStreamBeginCapture(s, hipStreamCaptureModeThreadLocal);
-			if (ce == hipSuccess)
-			{
-				forward(m, m->d_next, 1, 1, flags);
-				launch_argmax_step(m->logits, m->p.vocab_size, m->argmax_scratch, m->d_next, m->d_counters, 1, m->d_out, s);
-				ce = hipStreamEndCapture(s, &m->step_graph);
-			}
-			if (ce == hipSuccess)
-			{
-				ce = hipGraphInstantiate(&m->step_exec, m->step_graph, nullptr, nullptr, 0);
-			}
-			if (ce != hipSuccess)
-			{
-				drop_graph(m);
-				cleanup();
-				return fail_hip(kAction, ce);
-			}
-		}
-		for (size_t i = 1; i < n_new; ++i)
-		{
-			if (use_graph)
-			{
-				GEN_TRY(hipGraphLaunch(m->step_exec, s));
-			}
-			else
-			{
-				forward(m, m->d_next, 1, 1, flags);
-				launch_argmax_step(m->logits, m->p.vocab_size, m->argmax_scratch, m->d_next, m->d_counters, 1, m->d_out, s);
-			}
-		}
-	}
-	GEN_TRY(hipEventRecord(ev[2], s));
-	GEN_TRY(hipGetLastError());
-	GEN_TRY(hipMemcpyAsync(out_tokens, m->d_out, sizeof(int32_t) * n_new, hipMemcpyDeviceToHost, s));
-	int step_flag = 0;
-	GEN_TRY(hipMemcpyAsync(&step_flag, m->d_err, sizeof(int), hipMemcpyDeviceToHost, s));
-	GEN_TRY(hipStreamSynchronize(s));
-	if ((step_flag & 2) && m->block_fused > 0)
-	{
-		// a wait inside the one-launch attention half ran out: the tokens are void; once more, from
-		// the prompt, through the separate launches (`past` has not moved)
-		const int zero = 0;
-		GEN_TRY(hipMemcpy(m->d_err, &zero, sizeof(int), hipMemcpyHostToDevice));
-		cleanup();
-		give_up_block_launch(m);
-		return litenn_hip_llama_generate(m, prompt, n_prompt, n_new, out_tokens, flags, prefill_ms, decode_ms);
-	}
-	float ms = 0.0f;
-	if (prefill_ms)
-	{
-		GEN_TRY(hipEventElapsedTime(&ms, ev[0], ev[1]));
-		*prefill_ms = ms;
-	}
-	if (decode_ms)
-	{
-		GEN_TRY(hipEventElapsedTime(&ms, ev[1], ev[2]));
-		*decode_ms = ms;
-	}
-	cleanup();
-#undef GEN_TRY
-	// the last emitted token has not been fed back: the cache holds prompt + (n_new - 1) rows
-	m->past += static_cast<int>(n_prompt + n_new - 1);
-	return rc;
+	return decoder_generate(m, prompt, n_prompt, n_new, out_tokens, flags, prefill_ms, decode_ms);
 }
 
 extern "C" int litenn_hip_llama_get_kv(litenn_hip_llama* m, int layer, float* k, float* v)
