@@ -282,6 +282,55 @@ int litenn_hip_silu_mul(int dev, const void* gate, const void* up, void* y, size
  * (cf. the stable sort at src/LiteNN/Runtime/Interpreter.h:134-163). */
 int litenn_hip_argmax(int dev, const void* x, size_t rows, size_t n, void* out_index, const litenn_hip_exec* opts);
 
+/* ---- group 2b: layer mechanisms of the layered decoder ----------------- */
+
+/* y[m, n] (f32) = x . W^T over BFloat16 weights whose rows are `pitch` elements apart, pitch being k
+ * rounded up to a multiple of 64 and the elements behind the k-th zero.  x is [m, pitch] Float32 or
+ * BFloat16 (what lies behind the k-th element of a row is not used).  One Float32 row streams the
+ * weights once; other Float32 calls use the Float32 matrix instructions, BFloat16 ones the bfloat16
+ * ones.  Accumulation is Float32 throughout. */
+int litenn_hip_linear_bf16(int dev, const void* w, size_t n, size_t k, size_t pitch, const void* x, int x_dtype, size_t m,
+                           void* y, const litenn_hip_exec* opts);
+
+typedef struct litenn_hip_window_attn_opts
+{
+	double scale;          /* multiplies q.k */
+	size_t window;         /* positions a query sees, its own included */
+	size_t key_position;   /* position of key row 0 */
+	size_t query_position; /* position of query row 0 */
+	const void* sinks;     /* F32 [heads] on the device or NULL: exp(sink) joins the denominator */
+	const void* gate;      /* F32 [m, heads vdim] on the device or NULL: the result is multiplied by sigmoid(gate) */
+} litenn_hip_window_attn_opts;
+/* Causal sliding-window attention of m query rows: q [m, heads dim] F32, kv [keys, heads dim + heads vdim]
+ * of `dtype` (F32 or BF16; keys head by head, then values head by head), out [m, heads vdim] of
+ * `dtype`.  The keys must hold every query's own position.  BF16 with dim and vdim multiples of 8 up to 256
+ * runs on the matrix cores (q and the softmax weights rounded to bfloat16 once, scores and softmax
+ * Float32), every other shape (up to 1024) in Float32. */
+int litenn_hip_window_attn(int dev, const void* q, const void* kv, int dtype, size_t m, size_t keys, size_t heads,
+                           size_t dim, size_t vdim, const litenn_hip_window_attn_opts* o, void* out,
+                           const litenn_hip_exec* opts);
+
+/* Gated linear attention: per head S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = S_t^T (q_scale q_t), with
+ * a_t = sigmoid(decay_w low_t + decay_bias)^(1 / tau) per key channel. */
+typedef struct litenn_hip_gla_args
+{
+	size_t heads, dim, vdim, rank; /* dim <= 512, vdim <= 256, rank <= 512 */
+	double q_scale, tau, eps;
+	size_t ld;              /* floats between rows of the five below */
+	const void *q, *k;      /* F32 [m, heads dim] */
+	const void *v, *gate;   /* F32 [m, heads vdim] */
+	const void* low;        /* F32 [m, rank] */
+	const void* decay_w;    /* BF16 [heads dim, rank rounded up to a multiple of 64], zeros behind the rank */
+	const void* decay_bias; /* F32 [heads dim] */
+	const void* head_norm;  /* F32 [vdim] or NULL */
+} litenn_hip_gla_args;
+/* Advances state (F32 [heads, dim, vdim rounded up to a multiple of 4]) over m rows.  With head_norm every
+ * head of o is RMS-normalised, scaled by it and multiplied by silu(gate) (out [m, heads vdim], F32 or BF16; the
+ * chunked form, which needs a workspace); without it m must be 1 and out receives o itself (F32). */
+int litenn_hip_gla(int dev, const litenn_hip_gla_args* p, size_t m, void* state, void* out, int out_dtype,
+                   void* workspace, size_t workspace_bytes, const litenn_hip_exec* opts);
+size_t litenn_hip_gla_workspace_bytes(size_t m, size_t heads, size_t dim, size_t vdim);
+
 /* ---- group 3: LLaMA decoder runtime ----------------------------------- */
 
 typedef struct litenn_hip_llama litenn_hip_llama;

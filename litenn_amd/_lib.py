@@ -44,6 +44,18 @@ class GgufTensor(C.Structure):
     ]
 
 
+class WindowAttnOpts(C.Structure):
+    _fields_ = [("scale", C.c_double), ("window", C.c_size_t), ("key_position", C.c_size_t),
+                ("query_position", C.c_size_t), ("sinks", C.c_void_p), ("gate", C.c_void_p)]
+
+
+class GlaArgs(C.Structure):
+    _fields_ = [("heads", C.c_size_t), ("dim", C.c_size_t), ("vdim", C.c_size_t), ("rank", C.c_size_t),
+                ("q_scale", C.c_double), ("tau", C.c_double), ("eps", C.c_double), ("ld", C.c_size_t),
+                ("q", C.c_void_p), ("k", C.c_void_p), ("v", C.c_void_p), ("gate", C.c_void_p), ("low", C.c_void_p),
+                ("decay_w", C.c_void_p), ("decay_bias", C.c_void_p), ("head_norm", C.c_void_p)]
+
+
 class ModelTensor(C.Structure):
     """litenn_hip_model_tensor: a host tensor of a model under construction."""
     _fields_ = [("name", C.c_char_p), ("dtype", C.c_int), ("rank", C.c_size_t), ("shape", C.c_size_t * 4),
@@ -92,6 +104,10 @@ SIGNATURES = {
     "litenn_hip_attn_decode_noalloc": [_i, _vp, _vp, _vp, _i, _sz, _sz, _sz, _sz, _sz, _vp, _ex],
     "litenn_hip_attn_rows": [_i, _vp, _vp, _vp, _i, _sz, _sz, _sz, _sz, _sz, _vp, _u, _ex],
     "litenn_hip_flash_attn_ext": [_i, _vp, _vp, _vp, _i, _sz, _sz, _sz, _sz, _sz, C.POINTER(AttnExtOpts), _vp, _ex],
+    "litenn_hip_linear_bf16": [_i, _vp, _sz, _sz, _sz, _vp, _i, _sz, _vp, _ex],
+    "litenn_hip_window_attn": [_i, _vp, _vp, _i, _sz, _sz, _sz, _sz, _sz, C.POINTER(WindowAttnOpts), _vp, _ex],
+    "litenn_hip_gla": [_i, C.POINTER(GlaArgs), _sz, _vp, _vp, _i, _vp, _sz, _ex],
+    "litenn_hip_gla_workspace_bytes": [_sz, _sz, _sz, _sz],
     "litenn_hip_silu_mul": [_i, _vp, _vp, _vp, _sz, _ex],
     "litenn_hip_argmax": [_i, _vp, _sz, _sz, _vp, _ex],
     "litenn_hip_llama_create": [_i, C.POINTER(LlamaParams), C.POINTER(_vp)],
@@ -129,6 +145,7 @@ SIGNATURES = {
     "litenn_hip_llama_load_gguf": [_i, C.c_char_p, _i, C.c_int32, C.POINTER(_vp)],
 }
 _RESTYPES = {
+    "litenn_hip_gla_workspace_bytes": C.c_size_t,
     "litenn_hip_last_error": C.c_char_p, "litenn_hip_llama_model": C.c_void_p, "litenn_hip_mul_mat_q_workspace_bytes": C.c_size_t,
     "litenn_gguf_close": None, "litenn_gguf_version": C.c_uint, "litenn_gguf_tensor_count": C.c_size_t,
     "litenn_gguf_metadata_count": C.c_size_t, "litenn_gguf_metadata_key": C.c_char_p,

@@ -300,6 +300,43 @@ def flash_attn_ext(q: Tensor, k: Tensor, v: Tensor, m: int, keys: int, n_head: i
     return out
 
 
+def linear_bf16(w: Tensor, n: int, k: int, x: Tensor, m: int) -> Tensor:
+    """y [m, n] Float32 = x . W^T: w [n, pitch] bfloat16 bits (UInt8 or BFloat16 buffer), x [m, pitch] Float32 or
+    BFloat16, pitch = k rounded up to a multiple of 64."""
+    y = Tensor((m, n), DT_F32, x.device)
+    check(_lib.load().litenn_hip_linear_bf16(x.device.deviceIndex, w.ptr, n, k, -(-k // 64) * 64, x.ptr, x.dtype, m, y.ptr,
+                                             None))
+    return y
+
+
+def window_attn(q: Tensor, kv: Tensor, m: int, keys: int, heads: int, dim: int, vdim: int, window: int,
+                scale: float = 1.0, key_position: int = 0, query_position: int = 0, sinks: Tensor | None = None,
+                gate: Tensor | None = None) -> Tensor:
+    """Causal sliding-window attention with an optional sink per head and an optional sigmoid gate; q [m, heads dim]
+    Float32, kv [keys, heads (dim + vdim)] Float32 or BFloat16, the result has kv's type."""
+    out = Tensor((m, heads * vdim), kv.dtype, q.device)
+    o = _lib.WindowAttnOpts(scale, window, key_position, query_position, sinks.ptr if sinks is not None else None,
+                            gate.ptr if gate is not None else None)
+    check(_lib.load().litenn_hip_window_attn(q.device.deviceIndex, q.ptr, kv.ptr, kv.dtype, m, keys, heads, dim, vdim, o,
+                                             out.ptr, None))
+    return out
+
+
+def gla(q: Tensor, k: Tensor, v: Tensor, gate: Tensor | None, low: Tensor, decay_w: Tensor, decay_bias: Tensor,
+        head_norm: Tensor | None, state: Tensor, m: int, heads: int, dim: int, vdim: int, rank: int, ld: int,
+        q_scale: float, tau: float, eps: float = 1e-5, out_dtype: int = DT_F32) -> Tensor:
+    """Gated linear attention over m rows that advances `state` in place; q, k, v, gate and low are rows `ld` floats
+    apart.  With head_norm the normalised and gated heads come back, without it (m == 1) o itself."""
+    out = Tensor((m, heads * vdim), out_dtype, state.device)
+    a = _lib.GlaArgs(heads, dim, vdim, rank, q_scale, tau, eps, ld, q.ptr, k.ptr, v.ptr, gate.ptr if gate is not None else None,
+                     low.ptr, decay_w.ptr, decay_bias.ptr, head_norm.ptr if head_norm is not None else None)
+    ws_bytes = _lib.load().litenn_hip_gla_workspace_bytes(m, heads, dim, vdim)
+    ws = Tensor((ws_bytes,), DT_U8, state.device)
+    check(_lib.load().litenn_hip_gla(state.device.deviceIndex, a, m, state.ptr, out.ptr, out_dtype, ws.ptr, ws_bytes, None))
+    ws.free()
+    return out
+
+
 def silu_mul(gate: Tensor, up: Tensor) -> Tensor:
     y = Tensor(gate.shape, DT_F32, gate.device)
     check(_lib.load().litenn_hip_silu_mul(gate.device.deviceIndex, gate.ptr, up.ptr, y.ptr, gate.size, None))
