@@ -749,6 +749,78 @@ def bench_gemv_configs(ln, hiprt, steps=1600, warmup=64):
     return out
 
 
+KULURAX_SHAPES = {
+    # width, ff, heads, kv_rank, q_rank, gla heads; the LLaMA model beside it has the same width, ff, heads of 128
+    # (a quarter of them KV heads), layers and vocabulary
+    "2048": dict(width=2048, ff=5632, heads=16, kv_rank=256, q_rank=768, gla_heads=8, layers=8),
+    "4096": dict(width=4096, ff=14336, heads=32, kv_rank=512, q_rank=1536, gla_heads=16, layers=8),
+}
+
+
+def bench_kulurax(ln, names, prompts, n_new=128, window=1024, vocab=32000, repeats=3, llama=True):
+    """Prefill and decode of a layered decoder (linear and latent attention alternating, bfloat16 weights) beside
+    a LLaMA decoder of the same width, feed-forward, depth and vocabulary in Q8_0, the block format nearest to
+    16 bits.  Random weights; the best of `repeats` runs after one warm-up, model sides in turn."""
+    from litenn_amd import synth
+    from litenn_amd.formats import DT_F16, Q8_0
+    out = []
+    for name in names:
+        shape = KULURAX_SHAPES[name]
+        cfg = synth.kulurax_config(vocab=vocab, window=window, **shape)
+        context = max(prompts) + n_new + 8
+        t0 = time.perf_counter()
+        k_model = ln.create_model(cfg, synth.kulurax_large_tensors(cfg, 7), context_length=context)
+        sides = {"kulurax": k_model}
+        if llama:
+            lcfg = synth.LLaMAConfig(f"llama-{name}-q8_0", shape["layers"], shape["width"], shape["heads"],
+                                     shape["heads"] // 4, shape["ff"], vocab, context, formats={"default": Q8_0})
+            l_model = ln.LLaMA.from_config(lcfg, kv_dtype=DT_F16)
+            for item in synth.llama_tensors(lcfg, 3):
+                l_model.set_tensor(*item)
+            sides["llama"] = l_model
+        log(f"[bench] models of width {name} resident after {time.perf_counter() - t0:.1f} s")
+        entry = {"width": shape["width"], "ff": shape["ff"], "layers": shape["layers"], "vocab": vocab, "window": window,
+                 "shape": shape, "runs": []}
+        for n_prompt in prompts:
+            prompt = np.random.default_rng(5).integers(0, vocab, n_prompt).astype(np.int32)
+            best = {}
+            for model in sides.values():
+                model.reset()
+                model.generate(prompt, 8, precise=False)
+            for _ in range(repeats):
+                for side, model in sides.items():
+                    model.reset()
+                    _, pre, dec = model.generate(prompt, n_new, precise=False)
+                    b = best.setdefault(side, [pre, dec])
+                    b[0], b[1] = min(b[0], pre), min(b[1], dec)
+            run = {"prompt": n_prompt, "new_tokens": n_new}
+            for side, (pre, dec) in best.items():
+                if side == "kulurax":
+                    w_bytes = synth.kulurax_decode_weight_bytes(cfg)
+                    flops = synth.kulurax_prefill_flops(cfg, n_prompt)
+                else:
+                    w_bytes = lcfg.matmul_weight_bytes_per_token()
+                    per_token = sum(2.0 * s[0] * s[1] for kind, s in lcfg.tensor_shapes().items()
+                                    if kind not in ("token_embd", "output")) * lcfg.block_count
+                    flops = per_token * n_prompt + 2.0 * vocab * lcfg.embedding_length + \
+                        4.0 * lcfg.block_count * lcfg.embedding_length * n_prompt * (n_prompt + 1) / 2
+                step_us = dec / (n_new - 1) * 1e3
+                run[side] = {"prefill_ms": round(pre, 3), "prefill_tokens_per_s": round(n_prompt / pre * 1e3, 1),
+                             "prefill_tflops": round(flops / pre / 1e9, 1),
+                             "prefill_frac_of_matrix_peak": round(flops / pre / 1e9 / 2500.0, 4),
+                             "decode_us_per_token": round(step_us, 2), "decode_tokens_per_s": round(1e6 / step_us, 1),
+                             "decode_weight_bytes": w_bytes,
+                             "decode_frac_of_hbm_peak": round(w_bytes / step_us / 1e3 / HBM_PEAK_GBPS, 4)}
+                log(f"[bench] width {name}, prompt {n_prompt}, {side}: prefill {pre:.3f} ms = "
+                    f"{run[side]['prefill_tflops']} TFLOP/s, decode {step_us:.1f} us/token = "
+                    f"{100 * run[side]['decode_frac_of_hbm_peak']:.1f}% of HBM peak by weight bytes")
+            entry["runs"].append(run)
+        for model in sides.values():
+            model.close()
+        out.append(entry)
+    return out
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -774,6 +846,12 @@ def main() -> int:
                     help="also measure an empty kernel, a read-only kernel and the GEMV's in-kernel timeline")
     ap.add_argument("--block-timeline", action="store_true",
                     help="print the decoder-block kernel's in-kernel timeline (timeline build of the library) and exit")
+    ap.add_argument("--kulurax", action="store_true",
+                    help="measure the layered decoder (Kulurax) beside a LLaMA model of equal size, print that and exit")
+    ap.add_argument("--kulurax-widths", default="2048,4096", help="model widths of --kulurax")
+    ap.add_argument("--kulurax-prompts", default="128,512,2048", help="prompt lengths of --kulurax")
+    ap.add_argument("--kulurax-new", type=int, default=128, help="generated tokens of --kulurax")
+    ap.add_argument("--kulurax-alone", action="store_true", help="--kulurax without the LLaMA side (profiler runs)")
     ap.add_argument("--traffic-probe", action="store_true",
                     help="also launch a known-size streaming kernel (profiler counter calibration)")
     args = ap.parse_args()
@@ -794,6 +872,12 @@ def main() -> int:
         print("bench.py needs a HIP device", file=sys.stderr)
         return 1
     log("[bench]", ln.DeviceTraits.Info(ln.HIP(0)))
+
+    if args.kulurax:
+        result = bench_kulurax(ln, args.kulurax_widths.split(","), [int(p) for p in args.kulurax_prompts.split(",")],
+                               n_new=args.kulurax_new, repeats=1 if args.kulurax_alone else 3, llama=not args.kulurax_alone)
+        print(json.dumps({"kulurax": result, "dtype": "bf16 weights, f32 residual", "data": "synthetic"}), flush=True)
+        return 0
 
     if args.traffic_probe:
         traffic_probe(ln)

@@ -197,3 +197,79 @@ def llama_tensors(cfg: LLaMAConfig, seed: int):
 
 def prompt_tokens(cfg: LLaMAConfig, n: int, seed: int) -> np.ndarray:
     return _rng(seed, 777).integers(0, cfg.vocab, size=n, dtype=np.int32)
+
+
+# ---- layered decoders --------------------------------------------------------------------------------
+
+def kulurax_config(width: int, ff: int, layers: int, heads: int, vocab: int, window: int, kv_rank: int, q_rank: int,
+                   dim: int = 128, gla_heads: int = 16, gla_dim: int = 128, gla_vdim: int = 256) -> dict:
+    """A Kulurax decoder in which linear and latent attention alternate, every layer with a feed-forward."""
+    mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
+    linear = {"type": "gla", "mlp": mlp, "mixer": {"heads": gla_heads, "dim": gla_dim, "vdim": gla_vdim, "tau": 16.0}}
+    latent = {"type": "latent_attention", "mlp": mlp,
+              "mixer": {"heads": heads, "dim": dim, "vdim": dim, "kv_rank": kv_rank, "q_rank": q_rank,
+                        "scale": dim ** -0.5, "mask": {"size": window}}}
+    return {"architecture": "Kulurax", "vocab": vocab, "width": width, "norm": {"eps": 1e-5},
+            "layers": [linear if i % 2 == 0 else latent for i in range(layers)]}
+
+
+def kulurax_tensor_shapes(cfg: dict, decay_rank: int = 16) -> dict:
+    w = cfg["width"]
+    out = {"embed": (cfg["vocab"], w), "final.norm": (w,)}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        keys, values = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+        out[p + "norm1"] = out[p + "norm1b"] = (w,)
+        if layer["type"] == "gla":
+            parts = {"q": (keys, w), "k": (keys, w), "v": (values, w), "g": (values, w), "o": (w, values),
+                     "norm": (m["vdim"],), "a1": (decay_rank, w), "a2": (keys, decay_rank), "a2.b": (keys,)}
+        else:
+            parts = {"dq": (m["q_rank"], w), "dq.norm": (m["q_rank"],), "uq": (keys, m["q_rank"]),
+                     "dkv": (m["kv_rank"], w), "dkv.norm": (m["kv_rank"],), "uk": (keys, m["kv_rank"]),
+                     "uv": (values, m["kv_rank"]), "sink": (m["heads"],), "g": (values, w), "o": (w, values)}
+        out.update({p + "mix." + k: s for k, s in parts.items()})
+        if layer["mlp"]:
+            ff = layer["mlp"]["ff"]
+            out[p + "norm2"] = out[p + "norm2b"] = (w,)
+            out.update({p + "mlp.gate": (ff, w), p + "mlp.up": (ff, w), p + "mlp.down": (w, ff)})
+    return out
+
+
+def kulurax_large_tensors(cfg: dict, seed) -> dict:
+    """bfloat16 bits for a large model: every matrix is a window into one pool of N(0, 1/64) values, so that
+    gigabytes of weights take a second to make and little host memory."""
+    rng = _rng(seed)
+    shapes = kulurax_tensor_shapes(cfg)
+    size = max(int(np.prod(s)) for s in shapes.values()) + 65536
+    pool = (rng.standard_normal(size, dtype=np.float32) * np.float32(1.0 / 64.0)).view(np.uint32)
+    pool = ((pool + 0x8000) >> 16).astype(np.uint16)
+    out = {}
+    for name, s in shapes.items():
+        n = int(np.prod(s))
+        if len(s) == 1:
+            out[name] = rng.uniform(0.5, 1.5, s).astype(np.float32)
+        else:
+            at = int(rng.integers(0, 65536))
+            out[name] = pool[at:at + n].reshape(s)
+    return out
+
+
+def kulurax_decode_weight_bytes(cfg: dict) -> int:
+    """Weight bytes a single-token step reads: every matrix once (the tied table as the head)."""
+    return 2 * sum(int(np.prod(s)) for s in kulurax_tensor_shapes(cfg).values() if len(s) == 2)
+
+
+def kulurax_prefill_flops(cfg: dict, rows: int) -> float:
+    """Matrix-product operations of a prompt pass of `rows` tokens from an empty sequence: linears, window attention's
+    visible scores and values, the recurrence (state update and read)."""
+    shapes = kulurax_tensor_shapes(cfg)
+    total = sum(2.0 * rows * np.prod(s) for n, s in shapes.items() if len(s) == 2 and n != "embed")
+    for layer in cfg["layers"]:
+        m = layer["mixer"]
+        if layer["type"] == "gla":
+            total += 4.0 * rows * m["heads"] * m["dim"] * m["vdim"]
+        else:
+            w = m["mask"]["size"]
+            seen = rows * (rows + 1) / 2 if rows <= w else w * (w + 1) / 2 + (rows - w) * w
+            total += 2.0 * seen * m["heads"] * (m["dim"] + m["vdim"])
+    return float(total + 2.0 * cfg["vocab"] * cfg["width"])

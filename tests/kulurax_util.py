@@ -7,6 +7,7 @@ import struct
 
 import numpy as np
 
+from litenn_amd.synth import kulurax_tensor_shapes
 from litenn_amd.model import from_bfloat16, to_bfloat16
 
 
@@ -28,34 +29,12 @@ def config(layers, vocab=131, width=88, eps=3e-5):
     return {"architecture": "Kulurax", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers}
 
 
-def tensor_shapes(cfg, decay_rank=7):
-    w = cfg["width"]
-    out = {"embed": (cfg["vocab"], w), "final.norm": (w,)}
-    for i, layer in enumerate(cfg["layers"]):
-        p, m = f"l{i}.", layer["mixer"]
-        keys, values = m["heads"] * m["dim"], m["heads"] * m["vdim"]
-        out[p + "norm1"] = out[p + "norm1b"] = (w,)
-        if layer["type"] == "gla":
-            parts = {"q": (keys, w), "k": (keys, w), "v": (values, w), "g": (values, w), "o": (w, values),
-                     "norm": (m["vdim"],), "a1": (decay_rank, w), "a2": (keys, decay_rank), "a2.b": (keys,)}
-        else:
-            parts = {"dq": (m["q_rank"], w), "dq.norm": (m["q_rank"],), "uq": (keys, m["q_rank"]),
-                     "dkv": (m["kv_rank"], w), "dkv.norm": (m["kv_rank"],), "uk": (keys, m["kv_rank"]),
-                     "uv": (values, m["kv_rank"]), "sink": (m["heads"],), "g": (values, w), "o": (w, values)}
-        out.update({p + "mix." + k: s for k, s in parts.items()})
-        if layer["mlp"]:
-            ff = layer["mlp"]["ff"]
-            out[p + "norm2"] = out[p + "norm2b"] = (w,)
-            out.update({p + "mlp.gate": (ff, w), p + "mlp.up": (ff, w), p + "mlp.down": (w, ff)})
-    return out
-
-
 def random_weights(cfg, seed, decay_rank=7, decay_bias=(-1.0, 4.0), gain=1.0, edit=None):
     """{name: bfloat16 bits}.  Linears have entries of root mean square gain / sqrt(inputs); norms lie around
     one; decay biases are spread over `decay_bias`; edit(weights) may change the Float32 values first."""
     rng = np.random.default_rng(seed)
     w = {}
-    for name, shape in tensor_shapes(cfg, decay_rank).items():
+    for name, shape in kulurax_tensor_shapes(cfg, decay_rank).items():
         if name.endswith("a2.b"):
             v = rng.uniform(*decay_bias, shape)
         elif name.endswith("sink"):
