@@ -38,6 +38,34 @@ namespace litenn_hip
 			return ((k >> 2) & 1) * half + (k >> 3) * 4 + (k & 3);
 		}
 
+		// elements i .. i + 3 of a vector of k, zero beyond (global loads take any 4-byte address)
+		__device__ __forceinline__ floatx4 load_piece(const float* x, int i, int k)
+		{
+			typedef floatx4 floatx4_a4 __attribute__((aligned(4)));
+			floatx4 v = { 0.0f, 0.0f, 0.0f, 0.0f };
+			if (i + 3 < k)
+			{
+				v = *reinterpret_cast<const floatx4_a4*>(x + i);
+			}
+			else
+			{
+#pragma unroll
+				for (int e = 0; e < 3; ++e)
+				{
+					v[e] = i + e < k ? x[i + e] : 0.0f;
+				}
+			}
+			return v;
+		}
+
+		__device__ __forceinline__ float square_sum(const floatx4& v, float acc)
+		{
+			acc = fmaf(v.x, v.x, acc);
+			acc = fmaf(v.y, v.y, acc);
+			acc = fmaf(v.z, v.z, acc);
+			return fmaf(v.w, v.w, acc);
+		}
+
 		// sum over the workgroup; `red` holds one float per wavefront
 		__device__ __forceinline__ float block_sum(float v, float* red)
 		{
@@ -91,43 +119,83 @@ namespace litenn_hip
 				request(cur, rg, 0);
 			}
 
-			// activations
+			// activations, four at a time where k allows; a thread's first kKept pieces stay in registers
+			const int pieces = half >> 1; // of four floats, zeros behind the k-th
+			const auto put = [&](int piece, floatx4 v) {
+				*reinterpret_cast<floatx4*>(row_lds + (piece & 1) * half + (piece >> 1) * 4) = v;
+			};
 			if (d.prologue == kRowAddNorm)
 			{
+				constexpr int kKept = 2;
+				floatx4 x[kKept], sub[kKept], subw[kKept], nw[kKept];
+#pragma unroll
+				for (int e = 0; e < kKept; ++e)
+				{
+					const int i = 4 * (static_cast<int>(threadIdx.x) + kRowThreads * e);
+					x[e] = load_piece(d.x, i, k);
+					sub[e] = d.sub ? load_piece(d.sub, i, k) : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+					subw[e] = d.sub ? load_piece(d.sub_w, i, k) : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+					nw[e] = load_piece(d.norm_w, i, k);
+				}
 				float scale_sub = 0.0f;
 				if (d.sub)
 				{
 					float ss = 0.0f;
-					for (int i = threadIdx.x; i < k; i += kRowThreads)
+#pragma unroll
+					for (int e = 0; e < kKept; ++e)
 					{
-						ss = fmaf(d.sub[i], d.sub[i], ss);
+						ss = square_sum(sub[e], ss);
+					}
+					for (int p = threadIdx.x + kRowThreads * kKept; p < pieces; p += kRowThreads)
+					{
+						ss = square_sum(load_piece(d.sub, 4 * p, k), ss);
 					}
 					scale_sub = 1.0f / sqrtf(block_sum(ss, red) / static_cast<float>(k) + d.eps);
 				}
 				float ss = 0.0f;
-				for (int i = threadIdx.x; i < 2 * half; i += kRowThreads)
-				{
-					float v = 0.0f;
-					if (i < k)
+				const auto enter = [&](int p, floatx4 v, floatx4 s, floatx4 sw, floatx4 w) {
+					if (d.sub)
 					{
-						v = d.x[i];
-						if (d.sub)
-						{
-							v += d.sub[i] * scale_sub * d.sub_w[i];
-						}
-						if (d.x_out && blockIdx.x == 0)
-						{
-							d.x_out[i] = v;
-						}
-						ss = fmaf(v, v, ss);
-						v *= d.norm_w[i];
+						v += s * scale_sub * sw;
 					}
-					row_lds[row_slot(i, half)] = v;
+					if (d.x_out && blockIdx.x == 0)
+					{
+#pragma unroll
+						for (int i = 0; i < 4; ++i)
+						{
+							if (4 * p + i < k)
+							{
+								d.x_out[4 * p + i] = v[i];
+							}
+						}
+					}
+					ss = square_sum(v, ss);
+					return v * w;
+				};
+#pragma unroll
+				for (int e = 0; e < kKept; ++e)
+				{
+					x[e] = enter(static_cast<int>(threadIdx.x) + kRowThreads * e, x[e], sub[e], subw[e], nw[e]);
+				}
+				for (int p = threadIdx.x + kRowThreads * kKept; p < pieces; p += kRowThreads)
+				{
+					put(p, enter(p, load_piece(d.x, 4 * p, k), d.sub ? load_piece(d.sub, 4 * p, k) : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f },
+					             d.sub ? load_piece(d.sub_w, 4 * p, k) : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f }, load_piece(d.norm_w, 4 * p, k)));
 				}
 				const float scale = 1.0f / sqrtf(block_sum(ss, red) / static_cast<float>(k) + d.eps);
-				for (int i = threadIdx.x; i < k; i += kRowThreads)
+#pragma unroll
+				for (int e = 0; e < kKept; ++e)
 				{
-					row_lds[row_slot(i, half)] *= scale;
+					const int p = static_cast<int>(threadIdx.x) + kRowThreads * e;
+					if (p < pieces)
+					{
+						put(p, x[e] * scale);
+					}
+				}
+				for (int p = threadIdx.x + kRowThreads * kKept; p < pieces; p += kRowThreads)
+				{
+					floatx4* slot = reinterpret_cast<floatx4*>(row_lds + (p & 1) * half + (p >> 1) * 4);
+					*slot = *slot * scale; // this thread's own
 				}
 			}
 			else if (d.prologue == kRowHeadGate)
@@ -155,9 +223,10 @@ namespace litenn_hip
 			}
 			else
 			{
-				for (int i = threadIdx.x; i < 2 * half; i += kRowThreads)
+#pragma unroll 4
+				for (int p = threadIdx.x; p < pieces; p += kRowThreads)
 				{
-					row_lds[row_slot(i, half)] = i < k ? d.x[i] : 0.0f;
+					put(p, load_piece(d.x, 4 * p, k));
 				}
 			}
 			__syncthreads();

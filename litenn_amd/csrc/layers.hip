@@ -16,6 +16,7 @@ namespace litenn_hip
 		typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 		typedef float floatx4 __attribute__((ext_vector_type(4)));
 		typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+		typedef floatx4 floatx4_a4 __attribute__((aligned(4))); // global loads and stores take any 4-byte address
 
 		__device__ __forceinline__ int row_position(const Position& p, int row)
 		{
@@ -53,7 +54,8 @@ namespace litenn_hip
 			const uint16_t* t = table.w + static_cast<size_t>(id) * table.pitch;
 			float* xr = x + static_cast<size_t>(row) * table.k;
 			const double p = static_cast<double>(row_position(pos, row));
-			for (int i = threadIdx.x; 2 * i < table.k; i += 256)
+			const int i = static_cast<int>(blockIdx.y) * 256 + static_cast<int>(threadIdx.x);
+			if (2 * i < table.k)
 			{
 				float sn = 0.0f, cs = 0.0f;
 				if (turns)
@@ -78,13 +80,26 @@ namespace litenn_hip
 			constexpr int kKept = 16; // values a thread keeps in registers (wider rows are read again)
 			const int row = blockIdx.x;
 			const float* x = a.x + static_cast<size_t>(row) * a.ldx;
-			float kept[kKept];
+			float kept[kKept], added[kKept];
 			float scale_sub = 0.0f;
 			const float* sub = a.sub ? a.sub + static_cast<size_t>(row) * a.ldsub : nullptr;
+			// every load of the kept part is on its way before the first one is needed
+#pragma unroll
+			for (int e = 0; e < kKept; ++e)
+			{
+				const int i = threadIdx.x + 256 * e;
+				kept[e] = i < a.width ? x[i] : 0.0f;
+				added[e] = sub && i < a.width ? sub[i] : 0.0f;
+			}
 			if (sub)
 			{
 				float ss = 0.0f;
-				for (int i = threadIdx.x; i < a.width; i += 256)
+#pragma unroll
+				for (int e = 0; e < kKept; ++e)
+				{
+					ss = fmaf(added[e], added[e], ss);
+				}
+				for (int i = threadIdx.x + 256 * kKept; i < a.width; i += 256)
 				{
 					ss = fmaf(sub[i], sub[i], ss);
 				}
@@ -96,7 +111,10 @@ namespace litenn_hip
 			for (int e = 0; e < kKept; ++e)
 			{
 				const int i = threadIdx.x + 256 * e;
-				kept[e] = i < a.width ? value(i) : 0.0f;
+				if (sub && i < a.width)
+				{
+					kept[e] += added[e] * scale_sub * a.sub_w[i];
+				}
 				ss = fmaf(kept[e], kept[e], ss);
 			}
 			for (int i = threadIdx.x + 256 * kKept; i < a.width; i += 256)
@@ -278,23 +296,28 @@ namespace litenn_hip
 				const int base = first + t * kLatentTile;
 				const int count = min(kLatentTile, last - base + 1);
 				__syncthreads();
-				// rows past the last one are never stored: their weight is zero and they are skipped below
-				for (int i = threadIdx.x; i < kLatentTile * (pitch >> 2); i += 256)
 				{
-					const int key = i / (pitch >> 2), c = (i % (pitch >> 2)) * 4;
-					const T* p = cache + static_cast<size_t>((base + min(key, count - 1)) % a.cache.ring) * pitch + c;
-					floatx4 v;
-					if constexpr (sizeof(T) == 2)
+					// eight threads per row, 16 bytes each at a time (the pitch is a multiple of 64)
+					constexpr int E = 16 / sizeof(T);
+					const int key = threadIdx.x >> 3, c0 = (threadIdx.x & 7) * E;
+					const T* p = cache + static_cast<size_t>((base + min(key, count - 1)) % a.cache.ring) * pitch + c0;
+					float* dst = &tile[key * stride + c0];
+#pragma unroll 8
+					for (int c = 0; c < pitch; c += 8 * E)
 					{
-						const uint2 w = *reinterpret_cast<const uint2*>(p);
-						v = floatx4{ __uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u), __uint_as_float(w.y << 16),
-							         __uint_as_float(w.y & 0xffff0000u) };
+						const u32x4 w = *reinterpret_cast<const u32x4*>(p + c);
+						if constexpr (sizeof(T) == 2)
+						{
+							*reinterpret_cast<floatx4*>(dst + c) = floatx4{ __uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u),
+								                                            __uint_as_float(w.y << 16), __uint_as_float(w.y & 0xffff0000u) };
+							*reinterpret_cast<floatx4*>(dst + c + 4) = floatx4{ __uint_as_float(w.z << 16), __uint_as_float(w.z & 0xffff0000u),
+								                                                __uint_as_float(w.w << 16), __uint_as_float(w.w & 0xffff0000u) };
+						}
+						else
+						{
+							*reinterpret_cast<u32x4*>(dst + c) = w;
+						}
 					}
-					else
-					{
-						v = *reinterpret_cast<const floatx4*>(p);
-					}
-					*reinterpret_cast<floatx4*>(&tile[key * stride + c]) = v;
 				}
 				__syncthreads();
 				// scores: two lanes per key, each half of the latent
@@ -304,6 +327,7 @@ namespace litenn_hip
 					const float* kr = &tile[key * stride];
 					const float* qr = &qa[wave * pitch];
 					const int half = pitch >> 1;
+#pragma unroll 8
 					for (int c = part * half; c < (part + 1) * half; c += 4)
 					{
 						const floatx4 kv = *reinterpret_cast<const floatx4*>(kr + c);
@@ -332,7 +356,8 @@ namespace litenn_hip
 				{
 					o[c] *= corr;
 				}
-				for (int kk = 0; kk < count; ++kk)
+#pragma unroll 4
+				for (int kk = 0; kk < kLatentTile; ++kk) // the tile's unused rows repeat its last one, with weight zero
 				{
 					const float w = weights[wave * kLatentTile + kk];
 #pragma unroll
@@ -376,6 +401,7 @@ namespace litenn_hip
 		__global__ __launch_bounds__(256) void latent_value_kernel(const LatentStep a)
 		{
 			__shared__ __attribute__((aligned(16))) float o[kLatentMaxRank];
+			__shared__ float weight[64], sum;
 			const int pitch = a.cache.pitch;
 			const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
 			const int slices = (a.shape.vdim + kValueSlice - 1) / kValueSlice;
@@ -383,34 +409,35 @@ namespace litenn_hip
 			const int row = blockIdx.y;
 			const size_t step = static_cast<size_t>(a.shape.heads) * (pitch + 4);
 			const float* part = a.partial + (static_cast<size_t>(row) * a.splits * a.shape.heads + h) * (pitch + 4);
-			float top = a.shape.sink ? a.shape.sink[h] : -INFINITY;
-			for (int s = 0; s < a.splits; ++s)
+			// weights of the splits (at most 64; one without a visible position has maximum -inf and weight 0)
+			if (wave == 0)
 			{
-				top = fmaxf(top, part[s * step + pitch]);
+				const float sink = a.shape.sink ? a.shape.sink[h] : -INFINITY;
+				const float m = lane < a.splits ? part[lane * step + pitch] : -INFINITY;
+				const float l = lane < a.splits ? part[lane * step + pitch + 1] : 0.0f;
+				const float top = fmaxf(wave_max(m), sink);
+				const float w = expf(m - top);
+				const float all = wave_sum(w * l);
+				weight[lane] = w;
+				if (lane == 0)
+				{
+					sum = all + expf(sink - top);
+				}
 			}
-			float total = a.shape.sink ? expf(a.shape.sink[h] - top) : 0.0f;
+			__syncthreads();
+			const float total = sum;
 			float v[kLatentMaxRank / 256];
 #pragma unroll
 			for (int c = 0; c < kLatentMaxRank / 256; ++c)
 			{
 				v[c] = 0.0f;
-			}
-			for (int s = 0; s < a.splits; ++s)
-			{
-				const float m = part[s * step + pitch];
-				if (m == -INFINITY)
+				const int col = c * 256 + static_cast<int>(threadIdx.x);
+				if (col < a.cache.rank)
 				{
-					continue; // a split without a visible position
-				}
-				const float w = expf(m - top);
-				total = fmaf(w, part[s * step + pitch + 1], total);
-#pragma unroll
-				for (int c = 0; c < kLatentMaxRank / 256; ++c)
-				{
-					const int col = c * 256 + static_cast<int>(threadIdx.x);
-					if (col < a.cache.rank)
+#pragma unroll 8
+					for (int s = 0; s < a.splits; ++s)
 					{
-						v[c] = fmaf(w, part[s * step + col], v[c]);
+						v[c] = fmaf(weight[s], part[s * step + col], v[c]);
 					}
 				}
 			}
@@ -771,7 +798,7 @@ namespace litenn_hip
 			return z;
 		}
 
-		// log_decay[t, c] = log sigmoid(W_a2 a1[t] + bias)[c] / tau
+		// log_decay[t, c] = log2 sigmoid(W_a2 a1[t] + bias)[c] / tau
 		constexpr int kDecayRows = 16, kDecayMaxRank = 512;
 
 		__global__ __launch_bounds__(256) void gla_decay_kernel(const Gla a)
@@ -812,7 +839,7 @@ namespace litenn_hip
 			{
 				if (t < count)
 				{
-					a.log_decay[static_cast<size_t>(row0 + t) * channels + c] = log_sigmoid_f32(z[t]) * a.shape.inv_tau;
+					a.log_decay[static_cast<size_t>(row0 + t) * channels + c] = log_sigmoid_f32(z[t]) * (a.shape.inv_tau * 1.44269504f);
 				}
 			}
 		}
@@ -887,13 +914,15 @@ namespace litenn_hip
 		// ---- chunked form -------------------------------------------------------------------------
 		// Tokens in chunks of 64, a chunk in four blocks of 16.  With L_t the sum of a channel's log decays
 		// up to and including token t, every factor below is exp of a sum of log decays over some run of
-		// tokens, so none exceeds one whatever the decays are:
+		// tokens, so none exceeds one whatever the decays are (they are kept in units of log 2):
 		//   contribution of a chunk to the state:  sum_s (k_s exp(L_end - L_s)) v_s^T
 		//   o_t = (q_t exp(L_t - L_begin)) S_begin
 		//         + sum over earlier blocks of ((q_t exp(L_t - L_block)) . (k_s exp(L_block - L_s))) v_s
 		//         + inside t's own block  sum_s (sum_d q_td k_sd exp(L_td - L_sd)) v_s,
-		// L_block being L before the first token of t's block.  The contractions run on
-		// v_mfma_f32_16x16x4_f32; the own-block term is formed pair by pair.
+		// L_block being L before the first token of t's block.  The own-block term is split once more the same
+		// way into quarters of four tokens; only the pairs inside a quarter are formed one by one.  The
+		// contractions run on v_mfma_f32_16x16x4_f32.  Value columns are dealt out to the 16-wide tiles so that
+		// a lane's four consecutive columns (one 16-byte access) belong to four tiles.
 		constexpr int kChunk = 64, kSlab = 64, kSlabStride = 68;
 
 		// chunk_states: [chunk][head][dim][pitch] floats, then [chunk][head][dim] decays over the chunk
@@ -903,7 +932,29 @@ namespace litenn_hip
 			       static_cast<size_t>(chunks) * a.shape.heads * a.shape.dim * gla_state_pitch(a.shape.vdim);
 		}
 
-		template <int NE>
+		__device__ __forceinline__ float exp2_f32(float x) { return __builtin_amdgcn_exp2f(x); }
+
+		// four columns from column e of a row of `n`, zero beyond
+		__device__ __forceinline__ floatx4 load_columns(const float* row, int e, int n)
+		{
+			floatx4 v = { 0.0f, 0.0f, 0.0f, 0.0f };
+			if (e + 3 < n)
+			{
+				v = *reinterpret_cast<const floatx4_a4*>(row + e);
+			}
+			else
+			{
+#pragma unroll
+				for (int i = 0; i < 3; ++i)
+				{
+					v[i] = e + i < n ? row[e + i] : 0.0f;
+				}
+			}
+			return v;
+		}
+
+		// NC: groups of 64 value columns; tile b of group c holds columns 64 c + 4 i + b, i = 0 .. 15
+		template <int NC>
 		__global__ __launch_bounds__(256) void gla_state_kernel(const Gla a)
 		{
 			__shared__ float ks[kChunk][kSlabStride];
@@ -918,12 +969,18 @@ namespace litenn_hip
 				const int c = lane, part = wave;
 				const bool live = d0 + c < dim;
 				const size_t channel = static_cast<size_t>(h) * dim + d0 + (live ? c : 0);
-				float la[16], total = 0.0f;
+				float la[16], kv[16], total = 0.0f;
 #pragma unroll
 				for (int t = 0; t < 16; ++t)
 				{
 					const int row = 16 * part + t;
-					la[t] = live && row < count ? a.log_decay[static_cast<size_t>(row0 + row) * heads * dim + channel] : 0.0f;
+					const bool in = live && row < count;
+					la[t] = in ? a.log_decay[static_cast<size_t>(row0 + row) * heads * dim + channel] : 0.0f;
+					kv[t] = in ? a.k[static_cast<size_t>(row0 + row) * a.ld + channel] : 0.0f;
+				}
+#pragma unroll
+				for (int t = 0; t < 16; ++t)
+				{
 					total += la[t];
 				}
 				totals[part][c] = total;
@@ -936,23 +993,25 @@ namespace litenn_hip
 #pragma unroll
 				for (int t = 15; t >= 0; --t)
 				{
-					const int row = 16 * part + t;
-					const float k = live && row < count ? a.k[static_cast<size_t>(row0 + row) * a.ld + channel] : 0.0f;
-					ks[row][c] = k * expf(after);
+					ks[16 * part + t][c] = kv[t] * exp2_f32(after);
 					after += la[t];
 				}
 				if (part == 0 && live)
 				{
-					chunk_decays(a, gridDim.y)[(static_cast<size_t>(chunk) * heads + h) * dim + d0 + c] = expf(after);
+					chunk_decays(a, gridDim.y)[(static_cast<size_t>(chunk) * heads + h) * dim + d0 + c] = exp2_f32(after);
 				}
 			}
 			__syncthreads();
 			const int j = lane & 15, g = lane >> 4;
-			floatx4 acc[NE];
+			floatx4 acc[NC][4];
 #pragma unroll
-			for (int n = 0; n < NE; ++n)
+			for (int c = 0; c < NC; ++c)
 			{
-				acc[n] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+#pragma unroll
+				for (int b = 0; b < 4; ++b)
+				{
+					acc[c][b] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+				}
 			}
 #pragma unroll 4
 			for (int step = 0; step < kChunk / 4; ++step)
@@ -961,23 +1020,29 @@ namespace litenn_hip
 				const float kf = ks[t][16 * wave + j];
 				const float* v = a.v + static_cast<size_t>(row0 + min(t, count - 1)) * a.ld + h * vdim;
 #pragma unroll
-				for (int n = 0; n < NE; ++n)
+				for (int c = 0; c < NC; ++c)
 				{
-					const int e = 16 * n + j;
-					acc[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf, e < vdim ? v[e] : 0.0f, acc[n], 0, 0, 0);
+					const floatx4 vv = load_columns(v, 64 * c + 4 * j, vdim);
+#pragma unroll
+					for (int b = 0; b < 4; ++b)
+					{
+						acc[c][b] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf, vv[b], acc[c][b], 0, 0, 0);
+					}
 				}
 			}
 			float* dst = a.chunk_states + (static_cast<size_t>(chunk) * heads + h) * dim * pitch;
 #pragma unroll
-			for (int n = 0; n < NE; ++n)
+			for (int c = 0; c < NC; ++c)
 			{
+				const int e = 64 * c + 4 * j;
 #pragma unroll
 				for (int r = 0; r < 4; ++r)
 				{
-					const int d = d0 + 16 * wave + 4 * g + r, e = 16 * n + j;
+					const int d = d0 + 16 * wave + 4 * g + r;
 					if (d < dim && e < pitch)
 					{
-						dst[static_cast<size_t>(d) * pitch + e] = acc[n][r];
+						*reinterpret_cast<floatx4*>(dst + static_cast<size_t>(d) * pitch + e) =
+						    floatx4{ acc[c][0][r], acc[c][1][r], acc[c][2][r], acc[c][3][r] };
 					}
 				}
 			}
@@ -1023,7 +1088,7 @@ namespace litenn_hip
 			*reinterpret_cast<floatx4*>(a.state + at) = s;
 		}
 
-		template <int NE, typename T>
+		template <int NC, typename T>
 		__global__ __launch_bounds__(256) void gla_out_kernel(const Gla a)
 		{
 			__shared__ __attribute__((aligned(16))) float qs[kChunk][kSlabStride];
@@ -1036,14 +1101,20 @@ namespace litenn_hip
 			const int tid = threadIdx.x, lane = tid & 63;
 			const int wave = __builtin_amdgcn_readfirstlane(tid >> 6); // = the block of 16 tokens it makes
 			const int j = lane & 15, g = lane >> 4;
+			const int quarter = j >> 2; // of token j in its block
 			const float* state = a.chunk_states + (static_cast<size_t>(chunk) * heads + h) * dim * pitch;
 
-			floatx4 o[NE];      // o[n][r]: value column 16 n + 4 g + r of token j of the block
-			floatx4 scores[4];  // scores[b][r]: token 4 g + r of block b against token j
+			floatx4 o[NC][4];  // o[c][b][r]: value column 64 c + 16 g + 4 r + b of token j of the block
+			floatx4 scores[4]; // scores[back][r]: token 4 g + r of block wave - back against token j
+			float near[4] = { 0.0f, 0.0f, 0.0f, 0.0f }; // token j against the tokens of its quarter, a share of the channels
 #pragma unroll
-			for (int n = 0; n < NE; ++n)
+			for (int c = 0; c < NC; ++c)
 			{
-				o[n] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+#pragma unroll
+				for (int b = 0; b < 4; ++b)
+				{
+					o[c][b] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+				}
 			}
 #pragma unroll
 			for (int b = 0; b < 4; ++b)
@@ -1057,31 +1128,44 @@ namespace litenn_hip
 					const int c = lane;
 					const bool live = d0 + c < dim;
 					const size_t channel = static_cast<size_t>(h) * dim + d0 + (live ? c : 0);
-					float sum = 0.0f;
+					float la[16], qv[16], kv[16];
 #pragma unroll
 					for (int t = 0; t < 16; ++t)
 					{
 						const int row = 16 * wave + t;
 						const bool in = live && row < count;
 						const size_t at = static_cast<size_t>(row0 + row) * a.ld + channel;
-						sum += in ? a.log_decay[static_cast<size_t>(row0 + row) * heads * dim + channel] : 0.0f;
+						la[t] = in ? a.log_decay[static_cast<size_t>(row0 + row) * heads * dim + channel] : 0.0f;
+						qv[t] = in ? a.q[at] : 0.0f;
+						kv[t] = in ? a.k[at] : 0.0f;
+					}
+					float sum = 0.0f;
+#pragma unroll
+					for (int t = 0; t < 16; ++t)
+					{
+						const int row = 16 * wave + t;
+						sum += la[t];
 						ls[row][c] = sum;
-						qs[row][c] = in ? a.q[at] * a.shape.q_scale : 0.0f;
-						ks[row][c] = in ? a.k[at] : 0.0f;
+						qs[row][c] = qv[t] * a.shape.q_scale;
+						ks[row][c] = kv[t];
 					}
 					totals[wave][c] = sum;
 				}
 				__syncthreads();
-#pragma unroll
 				for (int quad = 0; quad < kSlab / 16; ++quad)
 				{
 					const int c = 16 * quad + 4 * g; // this lane's four channels of the slab
-					floatx4 qv = *reinterpret_cast<const floatx4*>(&qs[16 * wave + j][c]);
+					if (d0 + 16 * quad >= dim)
+					{
+						break; // uniform
+					}
+					const floatx4 qv = *reinterpret_cast<const floatx4*>(&qs[16 * wave + j][c]);
 					const floatx4 lq = *reinterpret_cast<const floatx4*>(&ls[16 * wave + j][c]);
+					floatx4 qb; // decayed from the block's first token
 #pragma unroll
 					for (int r = 0; r < 4; ++r)
 					{
-						qv[r] *= expf(lq[r]);
+						qb[r] = qv[r] * exp2_f32(lq[r]);
 					}
 					// earlier blocks, the nearest first: `between` is the decay over the blocks in between
 					floatx4 between = { 0.0f, 0.0f, 0.0f, 0.0f };
@@ -1098,7 +1182,7 @@ namespace litenn_hip
 #pragma unroll
 							for (int r = 0; r < 4; ++r)
 							{
-								sc = __builtin_amdgcn_mfma_f32_16x16x4f32(kv[r] * expf(tot[r] - lk[r] + between[r]), qv[r], sc, 0, 0, 0);
+								sc = __builtin_amdgcn_mfma_f32_16x16x4f32(kv[r] * exp2_f32(tot[r] - lk[r] + between[r]), qb[r], sc, 0, 0, 0);
 							}
 							scores[back] = sc;
 							between += tot;
@@ -1108,43 +1192,60 @@ namespace litenn_hip
 #pragma unroll
 					for (int r = 0; r < 4; ++r)
 					{
-						const float qi = qv[r] * expf(between[r]);
+						const float qi = qb[r] * exp2_f32(between[r]);
 						const int d = min(d0 + c + r, dim - 1); // qi is zero beyond
 						const float* sr = state + static_cast<size_t>(d) * pitch;
 #pragma unroll
-						for (int n = 0; n < NE; ++n)
+						for (int n = 0; n < NC; ++n)
 						{
-							const int e = 16 * n + j;
-							o[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(e < pitch ? sr[e] : 0.0f, qi, o[n], 0, 0, 0);
+							const int e = 64 * n + 4 * j;
+							const floatx4 sv = e < pitch ? *reinterpret_cast<const floatx4*>(sr + e) : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+#pragma unroll
+							for (int b = 0; b < 4; ++b)
+							{
+								o[n][b] = __builtin_amdgcn_mfma_f32_16x16x4f32(sv[b], qi, o[n][b], 0, 0, 0);
+							}
 						}
 					}
-				}
-				// own block, pair by pair: token j against tokens 4 g + r
-				for (int c = 0; c < kSlab; c += 4)
-				{
-					const floatx4 qv = *reinterpret_cast<const floatx4*>(&qs[16 * wave + j][c]);
-					const floatx4 lq = *reinterpret_cast<const floatx4*>(&ls[16 * wave + j][c]);
+					// own block, earlier quarters: pass u pairs the tokens of quarter u with all tokens before it
+					const floatx4 kv = *reinterpret_cast<const floatx4*>(&ks[16 * wave + j][c]);
+					const floatx4 lk = *reinterpret_cast<const floatx4*>(&ls[16 * wave + j][c]);
+					floatx4 sc = scores[0];
 #pragma unroll
-					for (int r = 0; r < 4; ++r)
+					for (int u = 1; u < 4; ++u)
 					{
-						const floatx4 kv = *reinterpret_cast<const floatx4*>(&ks[16 * wave + 4 * g + r][c]);
-						const floatx4 lk = *reinterpret_cast<const floatx4*>(&ls[16 * wave + 4 * g + r][c]);
-						float sc = scores[0][r];
+						const floatx4 lu = *reinterpret_cast<const floatx4*>(&ls[16 * wave + 4 * u - 1][c]);
 #pragma unroll
-						for (int x = 0; x < 4; ++x)
+						for (int r = 0; r < 4; ++r)
 						{
-							sc = fmaf(qv[x] * kv[x], expf(fminf(lq[x] - lk[x], 0.0f)), sc);
+							const float kf = quarter < u ? kv[r] * exp2_f32(lu[r] - lk[r]) : 0.0f;
+							const float qf = quarter == u ? qv[r] * exp2_f32(lq[r] - lu[r]) : 0.0f;
+							sc = __builtin_amdgcn_mfma_f32_16x16x4f32(kf, qf, sc, 0, 0, 0);
 						}
-						scores[0][r] = sc;
+					}
+					scores[0] = sc;
+					// inside the quarter, pair by pair
+#pragma unroll
+					for (int s = 0; s < 4; ++s)
+					{
+						const floatx4 kn = *reinterpret_cast<const floatx4*>(&ks[16 * wave + 4 * quarter + s][c]);
+						const floatx4 ln = *reinterpret_cast<const floatx4*>(&ls[16 * wave + 4 * quarter + s][c]);
+#pragma unroll
+						for (int r = 0; r < 4; ++r)
+						{
+							near[s] = fmaf(qv[r] * kn[r], exp2_f32(fminf(lq[r] - ln[r], 0.0f)), near[s]);
+						}
 					}
 				}
 			}
 #pragma unroll
-			for (int r = 0; r < 4; ++r)
+			for (int s = 0; s < 4; ++s)
 			{
-				scores[0][r] = 4 * g + r <= j ? scores[0][r] : 0.0f;
+				near[s] += __shfl_xor(near[s], 16, 64);
+				near[s] += __shfl_xor(near[s], 32, 64);
+				scores[0][s] += g == quarter && s <= (j & 3) ? near[s] : 0.0f;
 			}
-			// o += scores . v; scores[back] belongs to block wave - back
+			// o += scores . v
 #pragma unroll
 			for (int back = 0; back < 4; ++back)
 			{
@@ -1157,24 +1258,31 @@ namespace litenn_hip
 						const int s = min(16 * b + 4 * g + r, count - 1); // scores are zero beyond
 						const float* v = a.v + static_cast<size_t>(row0 + s) * a.ld + h * vdim;
 #pragma unroll
-						for (int n = 0; n < NE; ++n)
+						for (int n = 0; n < NC; ++n)
 						{
-							const int e = 16 * n + j;
-							o[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(e < vdim ? v[e] : 0.0f, scores[back][r], o[n], 0, 0, 0);
+							const floatx4 vv = load_columns(v, 64 * n + 4 * j, vdim);
+#pragma unroll
+							for (int x = 0; x < 4; ++x)
+							{
+								o[n][x] = __builtin_amdgcn_mfma_f32_16x16x4f32(vv[x], scores[back][r], o[n][x], 0, 0, 0);
+							}
 						}
 					}
 				}
 			}
-			// head norm and gate
+			// head norm and gate (columns past vdim are zero)
 			float ss = 0.0f;
 #pragma unroll
-			for (int n = 0; n < NE; ++n)
+			for (int n = 0; n < NC; ++n)
 			{
 #pragma unroll
-				for (int r = 0; r < 4; ++r)
+				for (int b = 0; b < 4; ++b)
 				{
-					o[n][r] = 16 * n + 4 * g + r < vdim ? o[n][r] : 0.0f;
-					ss = fmaf(o[n][r], o[n][r], ss);
+#pragma unroll
+					for (int r = 0; r < 4; ++r)
+					{
+						ss = fmaf(o[n][b][r], o[n][b][r], ss);
+					}
 				}
 			}
 			ss += __shfl_xor(ss, 16, 64);
@@ -1188,16 +1296,36 @@ namespace litenn_hip
 			const float* gate = a.gate + static_cast<size_t>(row0 + row) * a.ld + h * vdim;
 			T* out = static_cast<T*>(a.out) + static_cast<size_t>(row0 + row) * a.ldo + h * vdim;
 #pragma unroll
-			for (int n = 0; n < NE; ++n)
+			for (int n = 0; n < NC; ++n)
 			{
 #pragma unroll
 				for (int r = 0; r < 4; ++r)
 				{
-					const int e = 16 * n + 4 * g + r;
+					const int e = 64 * n + 16 * g + 4 * r;
 					if (e < vdim)
 					{
-						const float z = gate[e];
-						operand_store(out + e, o[n][r] * scale * a.norm_w[e] * (z * sigmoid_f32(z)));
+						const floatx4 z = load_columns(gate, e, vdim), w = load_columns(a.norm_w, e, vdim);
+						floatx4 y;
+#pragma unroll
+						for (int b = 0; b < 4; ++b)
+						{
+							y[b] = o[n][b][r] * scale * w[b] * (z[b] * sigmoid_f32(z[b]));
+						}
+						if (sizeof(T) == 2 && (vdim & 3) == 0 && (a.ldo & 3) == 0)
+						{
+							*reinterpret_cast<uint2*>(out + e) = make_uint2(pack_bf16(y[0], y[1]), pack_bf16(y[2], y[3]));
+						}
+						else
+						{
+#pragma unroll
+							for (int b = 0; b < 4; ++b)
+							{
+								if (e + b < vdim)
+								{
+									operand_store(out + e + b, y[b]);
+								}
+							}
+						}
 					}
 				}
 			}
@@ -1229,20 +1357,20 @@ namespace litenn_hip
 			}
 		}
 
-		template <int NE>
+		template <int NC>
 		void launch_gla_chunks(const Gla& a, int chunks, hipStream_t s)
 		{
 			const int slabs = (a.shape.dim + kSlab - 1) / kSlab;
-			gla_state_kernel<NE><<<dim3(a.shape.heads * slabs, chunks), dim3(256), 0, s>>>(a);
+			gla_state_kernel<NC><<<dim3(a.shape.heads * slabs, chunks), dim3(256), 0, s>>>(a);
 			const int quads = a.shape.heads * a.shape.dim * (gla_state_pitch(a.shape.vdim) >> 2);
 			gla_scan_kernel<<<dim3((quads + 255) / 256), dim3(256), 0, s>>>(a, chunks);
 			if (a.f32)
 			{
-				gla_out_kernel<NE, float><<<dim3(a.shape.heads, chunks), dim3(256), 0, s>>>(a);
+				gla_out_kernel<NC, float><<<dim3(a.shape.heads, chunks), dim3(256), 0, s>>>(a);
 			}
 			else
 			{
-				gla_out_kernel<NE, uint16_t><<<dim3(a.shape.heads, chunks), dim3(256), 0, s>>>(a);
+				gla_out_kernel<NC, uint16_t><<<dim3(a.shape.heads, chunks), dim3(256), 0, s>>>(a);
 			}
 		}
 
@@ -1258,7 +1386,7 @@ namespace litenn_hip
 	{
 		if (rows > 0)
 		{
-			embed_rows_kernel<<<dim3(rows), dim3(256), 0, s>>>(table, ids, turns, pos, x, err);
+			embed_rows_kernel<<<dim3(rows, (table.k + 511) / 512), dim3(256), 0, s>>>(table, ids, turns, pos, x, err);
 		}
 	}
 
@@ -1412,22 +1540,17 @@ namespace litenn_hip
 		const int channels = a.shape.heads * a.shape.dim;
 		gla_decay_kernel<<<dim3((channels + 255) / 256, (a.rows + kDecayRows - 1) / kDecayRows), dim3(256), 0, s>>>(a);
 		const int chunks = (a.rows + kChunk - 1) / kChunk;
-		const int ne = (a.shape.vdim + 15) / 16;
-		if (ne <= 2)
+		if (a.shape.vdim <= 64)
+		{
+			launch_gla_chunks<1>(a, chunks, s);
+		}
+		else if (a.shape.vdim <= 128)
 		{
 			launch_gla_chunks<2>(a, chunks, s);
 		}
-		else if (ne <= 4)
-		{
-			launch_gla_chunks<4>(a, chunks, s);
-		}
-		else if (ne <= 8)
-		{
-			launch_gla_chunks<8>(a, chunks, s);
-		}
 		else
 		{
-			launch_gla_chunks<16>(a, chunks, s);
+			launch_gla_chunks<4>(a, chunks, s);
 		}
 	}
 } // namespace litenn_hip
