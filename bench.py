@@ -757,7 +757,7 @@ KULURAX_SHAPES = {
 }
 
 
-def bench_kulurax(ln, names, prompts, n_new=128, window=1024, vocab=32000, repeats=3, llama=True):
+def bench_kulurax(ln, names, prompts, n_new=128, window=1024, vocab=32000, repeats=3, which=("kulurax", "llama")):
     """Prefill and decode of a layered decoder (linear and latent attention alternating, bfloat16 weights) beside
     a LLaMA decoder of the same width, feed-forward, depth and vocabulary in Q8_0, the block format nearest to
     16 bits.  Random weights; the best of `repeats` runs after one warm-up, model sides in turn."""
@@ -769,9 +769,10 @@ def bench_kulurax(ln, names, prompts, n_new=128, window=1024, vocab=32000, repea
         cfg = synth.kulurax_config(vocab=vocab, window=window, **shape)
         context = max(prompts) + n_new + 8
         t0 = time.perf_counter()
-        k_model = ln.create_model(cfg, synth.kulurax_large_tensors(cfg, 7), context_length=context)
-        sides = {"kulurax": k_model}
-        if llama:
+        sides = {}
+        if "kulurax" in which:
+            sides["kulurax"] = ln.create_model(cfg, synth.kulurax_large_tensors(cfg, 7), context_length=context)
+        if "llama" in which:
             lcfg = synth.LLaMAConfig(f"llama-{name}-q8_0", shape["layers"], shape["width"], shape["heads"],
                                      shape["heads"] // 4, shape["ff"], vocab, context, formats={"default": Q8_0})
             l_model = ln.LLaMA.from_config(lcfg, kv_dtype=DT_F16)
@@ -851,7 +852,7 @@ def main() -> int:
     ap.add_argument("--kulurax-widths", default="2048,4096", help="model widths of --kulurax")
     ap.add_argument("--kulurax-prompts", default="128,512,2048", help="prompt lengths of --kulurax")
     ap.add_argument("--kulurax-new", type=int, default=128, help="generated tokens of --kulurax")
-    ap.add_argument("--kulurax-alone", action="store_true", help="--kulurax without the LLaMA side (profiler runs)")
+    ap.add_argument("--kulurax-sides", default="kulurax,llama", help="which of the two models --kulurax runs (profiler runs take one)")
     ap.add_argument("--traffic-probe", action="store_true",
                     help="also launch a known-size streaming kernel (profiler counter calibration)")
     args = ap.parse_args()
@@ -875,7 +876,7 @@ def main() -> int:
 
     if args.kulurax:
         result = bench_kulurax(ln, args.kulurax_widths.split(","), [int(p) for p in args.kulurax_prompts.split(",")],
-                               n_new=args.kulurax_new, repeats=1 if args.kulurax_alone else 3, llama=not args.kulurax_alone)
+                               n_new=args.kulurax_new, repeats=3 if "," in args.kulurax_sides else 1, which=args.kulurax_sides.split(","))
         print(json.dumps({"kulurax": result, "dtype": "bf16 weights, f32 residual", "data": "synthetic"}), flush=True)
         return 0
 

@@ -18,6 +18,10 @@ namespace litenn_hip
 		typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 		typedef floatx4 floatx4_a4 __attribute__((aligned(4))); // global loads and stores take any 4-byte address
 
+		constexpr float kLog2e = 1.44269504088896340736f;
+
+		__device__ __forceinline__ float exp2_f32(float x) { return __builtin_amdgcn_exp2f(x); }
+
 		__device__ __forceinline__ int row_position(const Position& p, int row)
 		{
 			return (p.dev ? *p.dev : 0) + p.add + row;
@@ -80,7 +84,7 @@ namespace litenn_hip
 			constexpr int kKept = 16; // values a thread keeps in registers (wider rows are read again)
 			const int row = blockIdx.x;
 			const float* x = a.x + static_cast<size_t>(row) * a.ldx;
-			float kept[kKept], added[kKept];
+			float kept[kKept], added[kKept], sub_w[kKept], norm_w[kKept];
 			float scale_sub = 0.0f;
 			const float* sub = a.sub ? a.sub + static_cast<size_t>(row) * a.ldsub : nullptr;
 			// every load of the kept part is on its way before the first one is needed
@@ -90,6 +94,8 @@ namespace litenn_hip
 				const int i = threadIdx.x + 256 * e;
 				kept[e] = i < a.width ? x[i] : 0.0f;
 				added[e] = sub && i < a.width ? sub[i] : 0.0f;
+				sub_w[e] = sub && i < a.width ? a.sub_w[i] : 0.0f;
+				norm_w[e] = i < a.width ? a.norm_w[i] : 0.0f;
 			}
 			if (sub)
 			{
@@ -110,11 +116,7 @@ namespace litenn_hip
 #pragma unroll
 			for (int e = 0; e < kKept; ++e)
 			{
-				const int i = threadIdx.x + 256 * e;
-				if (sub && i < a.width)
-				{
-					kept[e] += added[e] * scale_sub * a.sub_w[i];
-				}
+				kept[e] += added[e] * scale_sub * sub_w[e];
 				ss = fmaf(kept[e], kept[e], ss);
 			}
 			for (int i = threadIdx.x + 256 * kKept; i < a.width; i += 256)
@@ -125,12 +127,12 @@ namespace litenn_hip
 			const float scale = 1.0f / sqrtf(block_sum256(ss, red) / static_cast<float>(a.width) + a.eps);
 			float* x_out = a.x_out ? a.x_out + static_cast<size_t>(row) * a.ldx : nullptr;
 			T* out = static_cast<T*>(a.out) + static_cast<size_t>(row) * a.ldo;
-			const auto put = [&](int i, float v) {
+			const auto put = [&](int i, float v, float w) {
 				if (x_out)
 				{
 					x_out[i] = v;
 				}
-				operand_store(out + i, v * scale * a.norm_w[i]);
+				operand_store(out + i, v * scale * w);
 			};
 #pragma unroll
 			for (int e = 0; e < kKept; ++e)
@@ -138,12 +140,12 @@ namespace litenn_hip
 				const int i = threadIdx.x + 256 * e;
 				if (i < a.width)
 				{
-					put(i, kept[e]);
+					put(i, kept[e], norm_w[e]);
 				}
 			}
 			for (int i = threadIdx.x + 256 * kKept; i < a.width; i += 256)
 			{
-				put(i, value(i));
+				put(i, value(i), a.norm_w[i]);
 			}
 		}
 
@@ -271,17 +273,39 @@ namespace litenn_hip
 			const int row = blockIdx.z, split = blockIdx.y;
 			const int h = static_cast<int>(blockIdx.x) * kLatentHeads + wave;
 			const int hc = min(h, a.shape.heads - 1);
-			const float* src = a.absorbed + (static_cast<size_t>(row) * a.shape.heads + hc) * pitch;
-			for (int i = lane; i < pitch; i += 64)
-			{
-				qa[wave * pitch + i] = i < a.cache.rank ? src[i] : 0.0f;
-			}
 			const int last = row_position(a.pos, row);
 			const int first = max(0, last - a.shape.window + 1);
 			const int tiles = (last - first) / kLatentTile + 1;
 			const int per = (tiles + a.splits - 1) / a.splits;
 			const int t0 = split * per, t1 = min(tiles, t0 + per);
 			const T* const cache = static_cast<const T*>(a.cache.rows);
+			// eight threads per row of a tile, 16 bytes each at a time (the pitch is a multiple of 64); a row's
+			// first kAhead pieces per thread are requested before anything waits
+			constexpr int E = 16 / sizeof(T), kAhead = 8;
+			const int my_key = threadIdx.x >> 3, c0 = (threadIdx.x & 7) * E;
+			const auto row_of = [&](int base) {
+				const int count = min(kLatentTile, last - base + 1);
+				return cache + static_cast<size_t>((base + min(my_key, count - 1)) % a.cache.ring) * pitch + c0;
+			};
+			u32x4 ahead[kAhead];
+			const auto request = [&](int base) {
+				const T* p = row_of(base);
+#pragma unroll
+				for (int i = 0; i < kAhead; ++i)
+				{
+					ahead[i] = *reinterpret_cast<const u32x4*>(p + (8 * E * i < pitch ? 8 * E * i : 0));
+				}
+			};
+			if (t0 < t1)
+			{
+				request(first + t0 * kLatentTile);
+			}
+			const float* src = a.absorbed + (static_cast<size_t>(row) * a.shape.heads + hc) * pitch;
+#pragma unroll 8
+			for (int i = lane; i < pitch; i += 64)
+			{
+				qa[wave * pitch + i] = i < a.cache.rank ? src[i] : 0.0f;
+			}
 
 			constexpr int kCols = kLatentMaxRank / 256;
 			floatx4 o[kCols];
@@ -297,15 +321,8 @@ namespace litenn_hip
 				const int count = min(kLatentTile, last - base + 1);
 				__syncthreads();
 				{
-					// eight threads per row, 16 bytes each at a time (the pitch is a multiple of 64)
-					constexpr int E = 16 / sizeof(T);
-					const int key = threadIdx.x >> 3, c0 = (threadIdx.x & 7) * E;
-					const T* p = cache + static_cast<size_t>((base + min(key, count - 1)) % a.cache.ring) * pitch + c0;
-					float* dst = &tile[key * stride + c0];
-#pragma unroll 8
-					for (int c = 0; c < pitch; c += 8 * E)
-					{
-						const u32x4 w = *reinterpret_cast<const u32x4*>(p + c);
+					float* dst = &tile[my_key * stride + c0];
+					const auto store = [&](int c, u32x4 w) {
 						if constexpr (sizeof(T) == 2)
 						{
 							*reinterpret_cast<floatx4*>(dst + c) = floatx4{ __uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u),
@@ -317,6 +334,23 @@ namespace litenn_hip
 						{
 							*reinterpret_cast<u32x4*>(dst + c) = w;
 						}
+					};
+#pragma unroll
+					for (int i = 0; i < kAhead; ++i)
+					{
+						if (8 * E * i < pitch)
+						{
+							store(8 * E * i, ahead[i]);
+						}
+					}
+					const T* p = row_of(base);
+					for (int c = 8 * E * kAhead; c < pitch; c += 8 * E)
+					{
+						store(c, *reinterpret_cast<const u32x4*>(p + c));
+					}
+					if (t + 1 < t1)
+					{
+						request(base + kLatentTile);
 					}
 				}
 				__syncthreads();
@@ -407,6 +441,16 @@ namespace litenn_hip
 			const int slices = (a.shape.vdim + kValueSlice - 1) / kValueSlice;
 			const int h = static_cast<int>(blockIdx.x) / slices, slice = static_cast<int>(blockIdx.x) % slices;
 			const int row = blockIdx.y;
+			// this wavefront's first rows of W_uv (a rank of up to 512 is one piece per lane), ahead of the merge
+			constexpr int kRows = kValueSlice / 4;
+			u32x4 first[kRows];
+#pragma unroll
+			for (int i = 0; i < kRows; ++i)
+			{
+				const int e = min(slice * kValueSlice + wave + 4 * i, a.shape.vdim - 1);
+				first[i] = *reinterpret_cast<const u32x4*>(a.uv.w + static_cast<size_t>(h * a.shape.vdim + e) * a.uv.pitch +
+				                                           (lane * 8 < pitch ? lane * 8 : 0));
+			}
 			const size_t step = static_cast<size_t>(a.shape.heads) * (pitch + 4);
 			const float* part = a.partial + (static_cast<size_t>(row) * a.splits * a.shape.heads + h) * (pitch + 4);
 			// weights of the splits (at most 64; one without a visible position has maximum -inf and weight 0)
@@ -448,9 +492,10 @@ namespace litenn_hip
 				o[c * 256 + threadIdx.x] = v[c] * inv;
 			}
 			__syncthreads();
-			for (int i = wave; i < kValueSlice; i += 4)
+#pragma unroll
+			for (int i = 0; i < kRows; ++i)
 			{
-				const int e = slice * kValueSlice + i;
+				const int e = slice * kValueSlice + wave + 4 * i;
 				if (e >= a.shape.vdim)
 				{
 					break;
@@ -459,7 +504,7 @@ namespace litenn_hip
 				float acc = 0.0f;
 				for (int r = lane * 8; r < pitch; r += 512)
 				{
-					const u32x4 x = *reinterpret_cast<const u32x4*>(w + r);
+					const u32x4 x = r < 512 ? first[i] : *reinterpret_cast<const u32x4*>(w + r);
 					const floatx4 o0 = *reinterpret_cast<const floatx4*>(o + r);
 					const floatx4 o1 = *reinterpret_cast<const floatx4*>(o + r + 4);
 					acc = fmaf(__uint_as_float(x.x << 16), o0.x, acc);
@@ -602,6 +647,7 @@ namespace litenn_hip
 			const int lo = max(0, a.q_base + q_first - a.shape.window + 1 - a.key_base);
 			const int hi = min(a.keys, a.q_base + min(q_first + kWinQ, a.rows) - a.key_base);
 			const uint16_t* const kv = static_cast<const uint16_t*>(a.kv);
+			const float scale2 = a.shape.scale * kLog2e; // scores in units of log 2
 
 			bf16x8 q_frag[DK / 32];
 			{
@@ -695,7 +741,7 @@ namespace litenn_hip
 					for (int r = 0; r < 4; ++r)
 					{
 						const int back = my_pos - (pos0 + 16 * b + r);
-						sv[b][r] = back >= 0 && back < a.shape.window ? s[b][r] * a.shape.scale : -INFINITY;
+						sv[b][r] = back >= 0 && back < a.shape.window ? s[b][r] * scale2 : -INFINITY;
 						top = fmaxf(top, sv[b][r]);
 					}
 				}
@@ -704,7 +750,7 @@ namespace litenn_hip
 				// a tile may hold no visible key of this query: exponents then take 0 as the maximum
 				const float new_m = fmaxf(run_m, top);
 				const float ref_m = new_m == -INFINITY ? 0.0f : new_m;
-				const float corr = expf(run_m - ref_m);
+				const float corr = exp2_f32(run_m - ref_m);
 				run_m = new_m;
 				float sum = 0.0f;
 				bf16x8 p_frag[2];
@@ -715,8 +761,8 @@ namespace litenn_hip
 #pragma unroll
 					for (int r = 0; r < 4; ++r)
 					{
-						p[r] = expf(sv[2 * ks][r] - ref_m);
-						p[4 + r] = expf(sv[2 * ks + 1][r] - ref_m);
+						p[r] = exp2_f32(sv[2 * ks][r] - ref_m);
+						p[4 + r] = exp2_f32(sv[2 * ks + 1][r] - ref_m);
 					}
 #pragma unroll
 					for (int e = 0; e < 8; ++e)
@@ -752,10 +798,10 @@ namespace litenn_hip
 			float weight = 1.0f, total = run_l;
 			if (a.shape.sink)
 			{
-				const float sink = a.shape.sink[h];
+				const float sink = a.shape.sink[h] * kLog2e;
 				const float all_m = fmaxf(run_m, sink);
-				weight = expf(run_m - all_m);
-				total = run_l * weight + expf(sink - all_m);
+				weight = exp2_f32(run_m - all_m);
+				total = run_l * weight + exp2_f32(sink - all_m);
 			}
 			const float inv = weight / total;
 			uint16_t* out = static_cast<uint16_t*>(a.out) + static_cast<size_t>(my_q) * a.ldo + static_cast<size_t>(h) * vdim;
@@ -839,7 +885,7 @@ namespace litenn_hip
 			{
 				if (t < count)
 				{
-					a.log_decay[static_cast<size_t>(row0 + t) * channels + c] = log_sigmoid_f32(z[t]) * (a.shape.inv_tau * 1.44269504f);
+					a.log_decay[static_cast<size_t>(row0 + t) * channels + c] = log_sigmoid_f32(z[t]) * (a.shape.inv_tau * kLog2e);
 				}
 			}
 		}
@@ -932,8 +978,6 @@ namespace litenn_hip
 			       static_cast<size_t>(chunks) * a.shape.heads * a.shape.dim * gla_state_pitch(a.shape.vdim);
 		}
 
-		__device__ __forceinline__ float exp2_f32(float x) { return __builtin_amdgcn_exp2f(x); }
-
 		// four columns from column e of a row of `n`, zero beyond
 		__device__ __forceinline__ floatx4 load_columns(const float* row, int e, int n)
 		{
@@ -953,9 +997,10 @@ namespace litenn_hip
 			return v;
 		}
 
-		// NC: groups of 64 value columns; tile b of group c holds columns 64 c + 4 i + b, i = 0 .. 15
+		// NC: groups of 64 value columns, each the work of four wavefronts (which share out the channels or the
+		// tokens); tile b of group c holds columns 64 c + 4 i + b, i = 0 .. 15
 		template <int NC>
-		__global__ __launch_bounds__(256) void gla_state_kernel(const Gla a)
+		__global__ __launch_bounds__(256 * NC) void gla_state_kernel(const Gla a)
 		{
 			__shared__ float ks[kChunk][kSlabStride];
 			__shared__ float totals[4][kSlab];
@@ -963,13 +1008,29 @@ namespace litenn_hip
 			const int slabs = (dim + kSlab - 1) / kSlab;
 			const int h = static_cast<int>(blockIdx.x) / slabs, d0 = static_cast<int>(blockIdx.x) % slabs * kSlab;
 			const int chunk = blockIdx.y, row0 = chunk * kChunk, count = min(kChunk, a.rows - row0);
-			const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+			const int lane = threadIdx.x & 63;
+			const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+			const int part = wave & 3, col = wave >> 2;
+			const int j = lane & 15, g = lane >> 4;
+			const int e = 64 * col + 4 * j;
+			// the values are requested first: half of them travel while the keys are decayed
+			constexpr int kSteps = kChunk / 4, kAhead = 8;
+			const auto value = [&](int step) {
+				return load_columns(a.v + static_cast<size_t>(row0 + min(4 * step + g, count - 1)) * a.ld + h * vdim, e, vdim);
+			};
+			floatx4 ahead[kAhead];
+#pragma unroll
+			for (int i = 0; i < kAhead; ++i)
+			{
+				ahead[i] = value(i);
+			}
+			float la[16], kv[16];
+			const bool live = d0 + lane < dim;
+			if (col == 0)
 			{
 				// thread: one channel, 16 tokens
-				const int c = lane, part = wave;
-				const bool live = d0 + c < dim;
-				const size_t channel = static_cast<size_t>(h) * dim + d0 + (live ? c : 0);
-				float la[16], kv[16], total = 0.0f;
+				const size_t channel = static_cast<size_t>(h) * dim + d0 + (live ? lane : 0);
+				float total = 0.0f;
 #pragma unroll
 				for (int t = 0; t < 16; ++t)
 				{
@@ -983,67 +1044,58 @@ namespace litenn_hip
 				{
 					total += la[t];
 				}
-				totals[part][c] = total;
-				__syncthreads();
+				totals[part][lane] = total;
+			}
+			__syncthreads();
+			if (col == 0)
+			{
 				float after = 0.0f;
 				for (int p = part + 1; p < 4; ++p)
 				{
-					after += totals[p][c];
+					after += totals[p][lane];
 				}
 #pragma unroll
 				for (int t = 15; t >= 0; --t)
 				{
-					ks[16 * part + t][c] = kv[t] * exp2_f32(after);
+					ks[16 * part + t][lane] = kv[t] * exp2_f32(after);
 					after += la[t];
 				}
 				if (part == 0 && live)
 				{
-					chunk_decays(a, gridDim.y)[(static_cast<size_t>(chunk) * heads + h) * dim + d0 + c] = exp2_f32(after);
+					chunk_decays(a, gridDim.y)[(static_cast<size_t>(chunk) * heads + h) * dim + d0 + lane] = exp2_f32(after);
 				}
 			}
 			__syncthreads();
-			const int j = lane & 15, g = lane >> 4;
-			floatx4 acc[NC][4];
+			floatx4 acc[4];
 #pragma unroll
-			for (int c = 0; c < NC; ++c)
+			for (int b = 0; b < 4; ++b)
 			{
+				acc[b] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+			}
+#pragma unroll
+			for (int step = 0; step < kSteps; ++step)
+			{
+				const float kf = ks[4 * step + g][16 * part + j];
+				const floatx4 vv = ahead[step % kAhead];
+				if (step + kAhead < kSteps)
+				{
+					ahead[step % kAhead] = value(step + kAhead);
+				}
 #pragma unroll
 				for (int b = 0; b < 4; ++b)
 				{
-					acc[c][b] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
-				}
-			}
-#pragma unroll 4
-			for (int step = 0; step < kChunk / 4; ++step)
-			{
-				const int t = 4 * step + g;
-				const float kf = ks[t][16 * wave + j];
-				const float* v = a.v + static_cast<size_t>(row0 + min(t, count - 1)) * a.ld + h * vdim;
-#pragma unroll
-				for (int c = 0; c < NC; ++c)
-				{
-					const floatx4 vv = load_columns(v, 64 * c + 4 * j, vdim);
-#pragma unroll
-					for (int b = 0; b < 4; ++b)
-					{
-						acc[c][b] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf, vv[b], acc[c][b], 0, 0, 0);
-					}
+					acc[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf, vv[b], acc[b], 0, 0, 0);
 				}
 			}
 			float* dst = a.chunk_states + (static_cast<size_t>(chunk) * heads + h) * dim * pitch;
 #pragma unroll
-			for (int c = 0; c < NC; ++c)
+			for (int r = 0; r < 4; ++r)
 			{
-				const int e = 64 * c + 4 * j;
-#pragma unroll
-				for (int r = 0; r < 4; ++r)
+				const int d = d0 + 16 * part + 4 * g + r;
+				if (d < dim && e < pitch)
 				{
-					const int d = d0 + 16 * wave + 4 * g + r;
-					if (d < dim && e < pitch)
-					{
-						*reinterpret_cast<floatx4*>(dst + static_cast<size_t>(d) * pitch + e) =
-						    floatx4{ acc[c][0][r], acc[c][1][r], acc[c][2][r], acc[c][3][r] };
-					}
+					*reinterpret_cast<floatx4*>(dst + static_cast<size_t>(d) * pitch + e) =
+					    floatx4{ acc[0][r], acc[1][r], acc[2][r], acc[3][r] };
 				}
 			}
 		}
@@ -1088,70 +1140,90 @@ namespace litenn_hip
 			*reinterpret_cast<floatx4*>(a.state + at) = s;
 		}
 
+		// A wavefront makes 64 value columns of a block of 16 tokens.  The NC wavefronts of a block share out the
+		// channels for the scores, whose shares meet in LDS, and each takes the state and the values of its
+		// own columns.
 		template <int NC, typename T>
-		__global__ __launch_bounds__(256) void gla_out_kernel(const Gla a)
+		__global__ __launch_bounds__(256 * NC) void gla_out_kernel(const Gla a)
 		{
-			__shared__ __attribute__((aligned(16))) float qs[kChunk][kSlabStride];
-			__shared__ __attribute__((aligned(16))) float ks[kChunk][kSlabStride];
-			__shared__ __attribute__((aligned(16))) float ls[kChunk][kSlabStride]; // log decays summed from the block's first token
-			__shared__ __attribute__((aligned(16))) float totals[4][kSlab];        // a block's whole sum
+			constexpr int kTiles = 10; // score tiles of a chunk: block b against blocks b, b - 1 .. 0
+			__shared__ __attribute__((aligned(16))) float lds[3 * kChunk * kSlabStride + 4 * kSlab];
+			static_assert(NC * kTiles * 256 <= 3 * kChunk * kSlabStride + 4 * kSlab, "the shares fit over the slab");
+			__shared__ float squares[4][NC][16];
+			float(*const qs)[kSlabStride] = reinterpret_cast<float(*)[kSlabStride]>(lds);
+			float(*const ks)[kSlabStride] = qs + kChunk;
+			float(*const ls)[kSlabStride] = ks + kChunk; // log decays summed from the block's first token
+			float(*const totals)[kSlab] = reinterpret_cast<float(*)[kSlab]>(lds + 3 * kChunk * kSlabStride); // a block's whole sum
 			const int dim = a.shape.dim, vdim = a.shape.vdim, pitch = gla_state_pitch(vdim), heads = a.shape.heads;
 			const int h = blockIdx.x, chunk = blockIdx.y;
 			const int row0 = chunk * kChunk, count = min(kChunk, a.rows - row0);
-			const int tid = threadIdx.x, lane = tid & 63;
-			const int wave = __builtin_amdgcn_readfirstlane(tid >> 6); // = the block of 16 tokens it makes
+			const int lane = threadIdx.x & 63;
+			const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+			const int block = wave & 3, col = wave >> 2;
 			const int j = lane & 15, g = lane >> 4;
 			const int quarter = j >> 2; // of token j in its block
+			const int e0 = 64 * col + 4 * j;
 			const float* state = a.chunk_states + (static_cast<size_t>(chunk) * heads + h) * dim * pitch;
 
-			floatx4 o[NC][4];  // o[c][b][r]: value column 64 c + 16 g + 4 r + b of token j of the block
-			floatx4 scores[4]; // scores[back][r]: token 4 g + r of block wave - back against token j
+			floatx4 o[4];      // o[b][r]: value column 64 col + 16 g + 4 r + b of token j of the block
+			floatx4 scores[4]; // scores[back][r]: token 4 g + r of `block - back` against token j
 			float near[4] = { 0.0f, 0.0f, 0.0f, 0.0f }; // token j against the tokens of its quarter, a share of the channels
-#pragma unroll
-			for (int c = 0; c < NC; ++c)
-			{
-#pragma unroll
-				for (int b = 0; b < 4; ++b)
-				{
-					o[c][b] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
-				}
-			}
 #pragma unroll
 			for (int b = 0; b < 4; ++b)
 			{
+				o[b] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
 				scores[b] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
 			}
 			for (int d0 = 0; d0 < dim; d0 += kSlab)
 			{
 				__syncthreads();
 				{
-					const int c = lane;
-					const bool live = d0 + c < dim;
-					const size_t channel = static_cast<size_t>(h) * dim + d0 + (live ? c : 0);
-					float la[16], qv[16], kv[16];
+					// thread: one channel, 16 tokens, of one or more of the three arrays
+					const bool live = d0 + lane < dim;
+					const size_t channel = static_cast<size_t>(h) * dim + d0 + (live ? lane : 0);
+					const auto fetch = [&](const float* src, size_t ld, float (&v)[16]) {
 #pragma unroll
-					for (int t = 0; t < 16; ++t)
+						for (int t = 0; t < 16; ++t)
+						{
+							const int row = 16 * block + t;
+							v[t] = live && row < count ? src[static_cast<size_t>(row0 + row) * ld + channel] : 0.0f;
+						}
+					};
+					if (col == 0)
 					{
-						const int row = 16 * wave + t;
-						const bool in = live && row < count;
-						const size_t at = static_cast<size_t>(row0 + row) * a.ld + channel;
-						la[t] = in ? a.log_decay[static_cast<size_t>(row0 + row) * heads * dim + channel] : 0.0f;
-						qv[t] = in ? a.q[at] : 0.0f;
-						kv[t] = in ? a.k[at] : 0.0f;
-					}
-					float sum = 0.0f;
+						float la[16], sum = 0.0f;
+						fetch(a.log_decay, static_cast<size_t>(heads) * dim, la);
 #pragma unroll
-					for (int t = 0; t < 16; ++t)
-					{
-						const int row = 16 * wave + t;
-						sum += la[t];
-						ls[row][c] = sum;
-						qs[row][c] = qv[t] * a.shape.q_scale;
-						ks[row][c] = kv[t];
+						for (int t = 0; t < 16; ++t)
+						{
+							sum += la[t];
+							ls[16 * block + t][lane] = sum;
+						}
+						totals[block][lane] = sum;
 					}
-					totals[wave][c] = sum;
+					if (col == (NC > 1 ? 1 : 0))
+					{
+						float v[16];
+						fetch(a.q, static_cast<size_t>(a.ld), v);
+#pragma unroll
+						for (int t = 0; t < 16; ++t)
+						{
+							qs[16 * block + t][lane] = v[t] * a.shape.q_scale;
+						}
+					}
+					if (col == (NC > 2 ? 2 : NC - 1))
+					{
+						float v[16];
+						fetch(a.k, static_cast<size_t>(a.ld), v);
+#pragma unroll
+						for (int t = 0; t < 16; ++t)
+						{
+							ks[16 * block + t][lane] = v[t];
+						}
+					}
 				}
 				__syncthreads();
+#pragma unroll
 				for (int quad = 0; quad < kSlab / 16; ++quad)
 				{
 					const int c = 16 * quad + 4 * g; // this lane's four channels of the slab
@@ -1159,33 +1231,77 @@ namespace litenn_hip
 					{
 						break; // uniform
 					}
-					const floatx4 qv = *reinterpret_cast<const floatx4*>(&qs[16 * wave + j][c]);
-					const floatx4 lq = *reinterpret_cast<const floatx4*>(&ls[16 * wave + j][c]);
+					floatx4 sv[4];
+#pragma unroll
+					for (int r = 0; r < 4; ++r)
+					{
+						const int d = min(d0 + c + r, dim - 1); // the query is zero beyond
+						sv[r] = e0 < pitch ? *reinterpret_cast<const floatx4*>(state + static_cast<size_t>(d) * pitch + e0)
+						                   : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
+					}
+					const floatx4 qv = *reinterpret_cast<const floatx4*>(&qs[16 * block + j][c]);
+					const floatx4 lq = *reinterpret_cast<const floatx4*>(&ls[16 * block + j][c]);
 					floatx4 qb; // decayed from the block's first token
 #pragma unroll
 					for (int r = 0; r < 4; ++r)
 					{
 						qb[r] = qv[r] * exp2_f32(lq[r]);
 					}
+					const bool mine = quad % NC == col; // this wavefront's share of the scores
 					// earlier blocks, the nearest first: `between` is the decay over the blocks in between
 					floatx4 between = { 0.0f, 0.0f, 0.0f, 0.0f };
 #pragma unroll
 					for (int back = 1; back < 4; ++back)
 					{
-						const int b = wave - back; // uniform
+						const int b = block - back; // uniform
 						if (b >= 0)
 						{
-							const floatx4 kv = *reinterpret_cast<const floatx4*>(&ks[16 * b + j][c]);
-							const floatx4 lk = *reinterpret_cast<const floatx4*>(&ls[16 * b + j][c]);
 							const floatx4 tot = *reinterpret_cast<const floatx4*>(&totals[b][c]);
-							floatx4 sc = scores[back];
+							if (mine)
+							{
+								const floatx4 kv = *reinterpret_cast<const floatx4*>(&ks[16 * b + j][c]);
+								const floatx4 lk = *reinterpret_cast<const floatx4*>(&ls[16 * b + j][c]);
+								floatx4 sc = scores[back];
+#pragma unroll
+								for (int r = 0; r < 4; ++r)
+								{
+									sc = __builtin_amdgcn_mfma_f32_16x16x4f32(kv[r] * exp2_f32(tot[r] - lk[r] + between[r]), qb[r], sc, 0, 0, 0);
+								}
+								scores[back] = sc;
+							}
+							between += tot;
+						}
+					}
+					if (mine)
+					{
+						// own block, earlier quarters: pass u pairs the tokens of quarter u with all tokens before it
+						const floatx4 kv = *reinterpret_cast<const floatx4*>(&ks[16 * block + j][c]);
+						const floatx4 lk = *reinterpret_cast<const floatx4*>(&ls[16 * block + j][c]);
+						floatx4 sc = scores[0];
+#pragma unroll
+						for (int u = 1; u < 4; ++u)
+						{
+							const floatx4 lu = *reinterpret_cast<const floatx4*>(&ls[16 * block + 4 * u - 1][c]);
 #pragma unroll
 							for (int r = 0; r < 4; ++r)
 							{
-								sc = __builtin_amdgcn_mfma_f32_16x16x4f32(kv[r] * exp2_f32(tot[r] - lk[r] + between[r]), qb[r], sc, 0, 0, 0);
+								const float kf = quarter < u ? kv[r] * exp2_f32(lu[r] - lk[r]) : 0.0f;
+								const float qf = quarter == u ? qv[r] * exp2_f32(lq[r] - lu[r]) : 0.0f;
+								sc = __builtin_amdgcn_mfma_f32_16x16x4f32(kf, qf, sc, 0, 0, 0);
 							}
-							scores[back] = sc;
-							between += tot;
+						}
+						scores[0] = sc;
+						// inside the quarter, pair by pair
+#pragma unroll
+						for (int s = 0; s < 4; ++s)
+						{
+							const floatx4 kn = *reinterpret_cast<const floatx4*>(&ks[16 * block + 4 * quarter + s][c]);
+							const floatx4 ln = *reinterpret_cast<const floatx4*>(&ls[16 * block + 4 * quarter + s][c]);
+#pragma unroll
+							for (int r = 0; r < 4; ++r)
+							{
+								near[s] = fmaf(qv[r] * kn[r], exp2_f32(fminf(lq[r] - ln[r], 0.0f)), near[s]);
+							}
 						}
 					}
 					// the state the chunk begins with (`between` now spans all earlier blocks of the chunk)
@@ -1193,47 +1309,10 @@ namespace litenn_hip
 					for (int r = 0; r < 4; ++r)
 					{
 						const float qi = qb[r] * exp2_f32(between[r]);
-						const int d = min(d0 + c + r, dim - 1); // qi is zero beyond
-						const float* sr = state + static_cast<size_t>(d) * pitch;
 #pragma unroll
-						for (int n = 0; n < NC; ++n)
+						for (int b = 0; b < 4; ++b)
 						{
-							const int e = 64 * n + 4 * j;
-							const floatx4 sv = e < pitch ? *reinterpret_cast<const floatx4*>(sr + e) : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
-#pragma unroll
-							for (int b = 0; b < 4; ++b)
-							{
-								o[n][b] = __builtin_amdgcn_mfma_f32_16x16x4f32(sv[b], qi, o[n][b], 0, 0, 0);
-							}
-						}
-					}
-					// own block, earlier quarters: pass u pairs the tokens of quarter u with all tokens before it
-					const floatx4 kv = *reinterpret_cast<const floatx4*>(&ks[16 * wave + j][c]);
-					const floatx4 lk = *reinterpret_cast<const floatx4*>(&ls[16 * wave + j][c]);
-					floatx4 sc = scores[0];
-#pragma unroll
-					for (int u = 1; u < 4; ++u)
-					{
-						const floatx4 lu = *reinterpret_cast<const floatx4*>(&ls[16 * wave + 4 * u - 1][c]);
-#pragma unroll
-						for (int r = 0; r < 4; ++r)
-						{
-							const float kf = quarter < u ? kv[r] * exp2_f32(lu[r] - lk[r]) : 0.0f;
-							const float qf = quarter == u ? qv[r] * exp2_f32(lq[r] - lu[r]) : 0.0f;
-							sc = __builtin_amdgcn_mfma_f32_16x16x4f32(kf, qf, sc, 0, 0, 0);
-						}
-					}
-					scores[0] = sc;
-					// inside the quarter, pair by pair
-#pragma unroll
-					for (int s = 0; s < 4; ++s)
-					{
-						const floatx4 kn = *reinterpret_cast<const floatx4*>(&ks[16 * wave + 4 * quarter + s][c]);
-						const floatx4 ln = *reinterpret_cast<const floatx4*>(&ls[16 * wave + 4 * quarter + s][c]);
-#pragma unroll
-						for (int r = 0; r < 4; ++r)
-						{
-							near[s] = fmaf(qv[r] * kn[r], exp2_f32(fminf(lq[r] - ln[r], 0.0f)), near[s]);
+							o[b] = __builtin_amdgcn_mfma_f32_16x16x4f32(sv[r][b], qi, o[b], 0, 0, 0);
 						}
 					}
 				}
@@ -1245,27 +1324,56 @@ namespace litenn_hip
 				near[s] += __shfl_xor(near[s], 32, 64);
 				scores[0][s] += g == quarter && s <= (j & 3) ? near[s] : 0.0f;
 			}
+			if constexpr (NC > 1)
+			{
+				// the shares, added in a fixed order
+				const int first = block * (block + 1) / 2;
+				__syncthreads();
+#pragma unroll
+				for (int back = 0; back < 4; ++back)
+				{
+					if (back <= block)
+					{
+						*reinterpret_cast<floatx4*>(lds + ((col * kTiles + first + back) * 64 + lane) * 4) = scores[back];
+					}
+				}
+				__syncthreads();
+#pragma unroll
+				for (int back = 0; back < 4; ++back)
+				{
+					if (back <= block)
+					{
+						floatx4 t = { 0.0f, 0.0f, 0.0f, 0.0f };
+#pragma unroll
+						for (int n = 0; n < NC; ++n)
+						{
+							t += *reinterpret_cast<const floatx4*>(lds + ((n * kTiles + first + back) * 64 + lane) * 4);
+						}
+						scores[back] = t;
+					}
+				}
+			}
 			// o += scores . v
 #pragma unroll
 			for (int back = 0; back < 4; ++back)
 			{
-				const int b = wave - back;
+				const int b = block - back;
 				if (b >= 0)
 				{
+					floatx4 vv[4];
 #pragma unroll
 					for (int r = 0; r < 4; ++r)
 					{
 						const int s = min(16 * b + 4 * g + r, count - 1); // scores are zero beyond
-						const float* v = a.v + static_cast<size_t>(row0 + s) * a.ld + h * vdim;
+						vv[r] = load_columns(a.v + static_cast<size_t>(row0 + s) * a.ld + h * vdim, e0, vdim);
+					}
 #pragma unroll
-						for (int n = 0; n < NC; ++n)
+					for (int r = 0; r < 4; ++r)
+					{
+#pragma unroll
+						for (int x = 0; x < 4; ++x)
 						{
-							const floatx4 vv = load_columns(v, 64 * n + 4 * j, vdim);
-#pragma unroll
-							for (int x = 0; x < 4; ++x)
-							{
-								o[n][x] = __builtin_amdgcn_mfma_f32_16x16x4f32(vv[x], scores[back][r], o[n][x], 0, 0, 0);
-							}
+							o[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(vv[r][x], scores[back][r], o[x], 0, 0, 0);
 						}
 					}
 				}
@@ -1273,21 +1381,31 @@ namespace litenn_hip
 			// head norm and gate (columns past vdim are zero)
 			float ss = 0.0f;
 #pragma unroll
-			for (int n = 0; n < NC; ++n)
+			for (int b = 0; b < 4; ++b)
 			{
 #pragma unroll
-				for (int b = 0; b < 4; ++b)
+				for (int r = 0; r < 4; ++r)
 				{
-#pragma unroll
-					for (int r = 0; r < 4; ++r)
-					{
-						ss = fmaf(o[n][b][r], o[n][b][r], ss);
-					}
+					ss = fmaf(o[b][r], o[b][r], ss);
 				}
 			}
 			ss += __shfl_xor(ss, 16, 64);
 			ss += __shfl_xor(ss, 32, 64);
-			const int row = 16 * wave + j;
+			if constexpr (NC > 1)
+			{
+				if (g == 0)
+				{
+					squares[block][col][j] = ss;
+				}
+				__syncthreads();
+				ss = 0.0f;
+#pragma unroll
+				for (int n = 0; n < NC; ++n)
+				{
+					ss += squares[block][n][j];
+				}
+			}
+			const int row = 16 * block + j;
 			if (row >= count)
 			{
 				return;
@@ -1296,34 +1414,30 @@ namespace litenn_hip
 			const float* gate = a.gate + static_cast<size_t>(row0 + row) * a.ld + h * vdim;
 			T* out = static_cast<T*>(a.out) + static_cast<size_t>(row0 + row) * a.ldo + h * vdim;
 #pragma unroll
-			for (int n = 0; n < NC; ++n)
+			for (int r = 0; r < 4; ++r)
 			{
-#pragma unroll
-				for (int r = 0; r < 4; ++r)
+				const int e = 64 * col + 16 * g + 4 * r;
+				if (e < vdim)
 				{
-					const int e = 64 * n + 16 * g + 4 * r;
-					if (e < vdim)
+					const floatx4 z = load_columns(gate, e, vdim), w = load_columns(a.norm_w, e, vdim);
+					floatx4 y;
+#pragma unroll
+					for (int b = 0; b < 4; ++b)
 					{
-						const floatx4 z = load_columns(gate, e, vdim), w = load_columns(a.norm_w, e, vdim);
-						floatx4 y;
+						y[b] = o[b][r] * scale * w[b] * (z[b] * sigmoid_f32(z[b]));
+					}
+					if (sizeof(T) == 2 && (vdim & 3) == 0 && (a.ldo & 3) == 0)
+					{
+						*reinterpret_cast<uint2*>(out + e) = make_uint2(pack_bf16(y[0], y[1]), pack_bf16(y[2], y[3]));
+					}
+					else
+					{
 #pragma unroll
 						for (int b = 0; b < 4; ++b)
 						{
-							y[b] = o[n][b][r] * scale * w[b] * (z[b] * sigmoid_f32(z[b]));
-						}
-						if (sizeof(T) == 2 && (vdim & 3) == 0 && (a.ldo & 3) == 0)
-						{
-							*reinterpret_cast<uint2*>(out + e) = make_uint2(pack_bf16(y[0], y[1]), pack_bf16(y[2], y[3]));
-						}
-						else
-						{
-#pragma unroll
-							for (int b = 0; b < 4; ++b)
+							if (e + b < vdim)
 							{
-								if (e + b < vdim)
-								{
-									operand_store(out + e + b, y[b]);
-								}
+								operand_store(out + e + b, y[b]);
 							}
 						}
 					}
@@ -1361,16 +1475,16 @@ namespace litenn_hip
 		void launch_gla_chunks(const Gla& a, int chunks, hipStream_t s)
 		{
 			const int slabs = (a.shape.dim + kSlab - 1) / kSlab;
-			gla_state_kernel<NC><<<dim3(a.shape.heads * slabs, chunks), dim3(256), 0, s>>>(a);
+			gla_state_kernel<NC><<<dim3(a.shape.heads * slabs, chunks), dim3(256 * NC), 0, s>>>(a);
 			const int quads = a.shape.heads * a.shape.dim * (gla_state_pitch(a.shape.vdim) >> 2);
 			gla_scan_kernel<<<dim3((quads + 255) / 256), dim3(256), 0, s>>>(a, chunks);
 			if (a.f32)
 			{
-				gla_out_kernel<NC, float><<<dim3(a.shape.heads, chunks), dim3(256), 0, s>>>(a);
+				gla_out_kernel<NC, float><<<dim3(a.shape.heads, chunks), dim3(256 * NC), 0, s>>>(a);
 			}
 			else
 			{
-				gla_out_kernel<NC, uint16_t><<<dim3(a.shape.heads, chunks), dim3(256), 0, s>>>(a);
+				gla_out_kernel<NC, uint16_t><<<dim3(a.shape.heads, chunks), dim3(256 * NC), 0, s>>>(a);
 			}
 		}
 
