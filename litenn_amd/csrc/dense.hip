@@ -339,8 +339,8 @@ namespace litenn_hip
 
 		// ------------------------------------------------------------------
 		// Many rows, bfloat16 operands: BM activation rows x BN weight rows per workgroup of four
-		// wavefronts, K in tiles of 64 double-buffered in LDS (global -> registers while the previous tile
-		// is multiplied -> LDS), v_mfma_f32_16x16x32_bf16 with the weights as the A operand, so that a lane
+		// wavefronts, K in tiles of 64 double-buffered in LDS (global -> registers two tiles ahead -> LDS
+		// while the previous tile is multiplied), v_mfma_f32_16x16x32_bf16 with the weights as the A operand, so that a lane
 		// ends up with four consecutive outputs of one activation row.  The 16-byte pieces of a 128-byte
 		// LDS row are permuted by the row's low three bits: the 16 rows a fragment read touches then fall
 		// on different banks.
@@ -422,7 +422,7 @@ namespace litenn_hip
 				}
 				return;
 			}
-			float* c = static_cast<float*>(d.c) + static_cast<size_t>(m) * d.ldc + n;
+			float* c = static_cast<float*>(d.c) + blockIdx.y * d.split_stride + static_cast<size_t>(m) * d.ldc + n;
 			if (n + 3 < d.w.n && (d.ldc & 3) == 0)
 			{
 				*reinterpret_cast<float4*>(c) = make_float4(f[0], f[1], f[2], f[3]);
@@ -456,7 +456,10 @@ namespace litenn_hip
 			const int wm = wave / WN, wn = wave % WN;
 			const int m0 = tm * BM, n0 = tn * BN;
 			const int k = d.w.k;
-			const int steps = d.w.pitch / kTileK;
+			// this workgroup's share of K
+			const int all_steps = d.w.pitch / kTileK, part = static_cast<int>(blockIdx.y);
+			const int first_step = all_steps * part / d.splits;
+			const int steps = all_steps * (part + 1) / d.splits - first_step;
 
 			const int ch = tid & 7, row = tid >> 3; // this thread's piece column and first row
 			const uint16_t* xp[LA];
@@ -471,20 +474,21 @@ namespace litenn_hip
 			{
 				wp[i] = d.w.w + static_cast<size_t>(min(n0 + row + 32 * i, d.w.n - 1)) * d.w.pitch + ch * 8;
 			}
-			u32x4 rx[LA], rw[LW];
-			const auto request = [&](int step) {
+			// two K tiles travel at any time: tile t in register set t & 1 until it is staged
+			u32x4 rx[2][LA], rw[2][LW];
+			const auto request = [&](int step, int set) {
 #pragma unroll
 				for (int i = 0; i < LA; ++i)
 				{
-					rx[i] = *reinterpret_cast<const u32x4*>(xp[i] + step * kTileK);
+					rx[set][i] = *reinterpret_cast<const u32x4*>(xp[i] + step * kTileK);
 				}
 #pragma unroll
 				for (int i = 0; i < LW; ++i)
 				{
-					rw[i] = *reinterpret_cast<const u32x4*>(wp[i] + step * kTileK);
+					rw[set][i] = *reinterpret_cast<const u32x4*>(wp[i] + step * kTileK);
 				}
 			};
-			const auto stage = [&](int step, int buf) {
+			const auto stage = [&](int step, int set) {
 				const int left = k - step * kTileK - ch * 8; // valid elements of this thread's pieces
 				if (left < 8)
 				{
@@ -496,7 +500,7 @@ namespace litenn_hip
 						for (int e = 0; e < 4; ++e)
 						{
 							const uint32_t keep = left >= 2 * e + 2 ? 0xffffffffu : left == 2 * e + 1 ? 0xffffu : 0u;
-							rx[i][e] &= keep;
+							rx[set][i][e] &= keep;
 						}
 					}
 				}
@@ -504,12 +508,12 @@ namespace litenn_hip
 #pragma unroll
 				for (int i = 0; i < LA; ++i)
 				{
-					*reinterpret_cast<u32x4*>(&xs[buf][(row + 32 * i) * kTileK + slot]) = rx[i];
+					*reinterpret_cast<u32x4*>(&xs[set][(row + 32 * i) * kTileK + slot]) = rx[set][i];
 				}
 #pragma unroll
 				for (int i = 0; i < LW; ++i)
 				{
-					*reinterpret_cast<u32x4*>(&ws[buf][(row + 32 * i) * kTileK + slot]) = rw[i];
+					*reinterpret_cast<u32x4*>(&ws[set][(row + 32 * i) * kTileK + slot]) = rw[set][i];
 				}
 			};
 
@@ -523,16 +527,7 @@ namespace litenn_hip
 					acc[a][b] = floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
 				}
 			}
-			request(0);
-			stage(0, 0);
-			__syncthreads();
-			for (int step = 0; step < steps; ++step)
-			{
-				const int buf = step & 1;
-				if (step + 1 < steps)
-				{
-					request(step + 1);
-				}
+			const auto multiply = [&](int buf) {
 #pragma unroll
 				for (int ks = 0; ks < 2; ++ks)
 				{
@@ -559,11 +554,35 @@ namespace litenn_hip
 						}
 					}
 				}
-				if (step + 1 < steps)
+			};
+			// past the last tile it is requested and staged again: a branch around the loads would make every
+			// wait behind it a wait for all of them
+			request(first_step, 0);
+			request(first_step + min(1, steps - 1), 1);
+			stage(first_step, 0);
+			__syncthreads();
+			// tile `step` is in LDS buffer `set`, tile step + 1 in the other register set
+			const auto advance = [&](int step, int set) {
+				request(first_step + min(step + 2, steps - 1), set);
+				if constexpr (BM * BN < 128 * 128)
 				{
-					stage(step + 1, buf ^ 1);
+					// on their way before the products, not behind them (the largest tile, whose products take
+					// longer than the loads, runs better scheduled freely)
+					__builtin_amdgcn_sched_barrier(0);
 				}
+				multiply(set);
+				stage(first_step + min(step + 1, steps - 1), set ^ 1);
 				__syncthreads();
+			};
+			int step = 0;
+			for (; step + 1 < steps; step += 2)
+			{
+				advance(step, 0);
+				advance(step + 1, 1);
+			}
+			if (step < steps)
+			{
+				advance(step, 0);
 			}
 #pragma unroll
 			for (int b = 0; b < TM; ++b)
@@ -719,11 +738,22 @@ namespace litenn_hip
 			args.m_tiles = (args.d.m + BM - 1) / BM;
 			args.n_tiles = (args.d.w.n + BN - 1) / BN;
 			const int per = (args.m_tiles * args.n_tiles + 7) / 8;
-			dense_tile_kernel<BM, BN, WM, WN><<<dim3(8 * per), dim3(256), 0, s>>>(args);
+			dense_tile_kernel<BM, BN, WM, WN><<<dim3(8 * per, args.d.splits), dim3(256), 0, s>>>(args);
 		}
 
 		int tiles(const DenseRows& d, int bm, int bn) { return ((d.m + bm - 1) / bm) * ((d.w.n + bn - 1) / bn); }
 	} // namespace
+
+	// Few tiles: K is walked in up to four ranges at once, enough for about two workgroups per CU and none
+	// shorter than 16 tiles of K.
+	int dense_rows_splits(const DenseMatrix& w, int m)
+	{
+		DenseRows d;
+		d.w = w;
+		d.m = m;
+		const int t = m <= 32 ? tiles(d, 32, 64) : tiles(d, 64, 64);
+		return std::max(1, std::min({ kDenseMaxSplits, (512 + t / 2) / t, w.pitch / kTileK / 16 }));
+	}
 
 	size_t dense_row_max_k() { return kRowLdsLimit / sizeof(float) / (kFlight * kRowBlock) * (kFlight * kRowBlock); }
 

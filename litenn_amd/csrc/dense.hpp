@@ -67,9 +67,15 @@ namespace litenn_hip
 		void* c = nullptr;
 		int ldc = 0; // a multiple of 4 for the operand types
 		int out = kOutF32;
+		// kOutF32 with bfloat16 operands: the products of `splits` ranges of K, split_stride floats apart, to be
+		// added by the reader (see dense_rows_splits)
+		int splits = 1;
+		size_t split_stride = 0;
 		bool f32 = false; // Float32 operands (the bfloat16 weights widened exactly), f32 matrix instructions
 		ClampedGlu act;
 	};
+	constexpr int kDenseMaxSplits = 4;
+	int dense_rows_splits(const DenseMatrix& w, int m);
 	void launch_dense_rows(const DenseRows& a, hipStream_t s);
 } // namespace litenn_hip
 

@@ -29,6 +29,7 @@ namespace litenn_hip
 		constexpr int kRowsMin = 4;        // from here on a pass runs on the matrix cores
 		constexpr int kExpandMin = 16;     // from here on attention expands the cached latents
 		constexpr int kPassRows = 4096;    // most tokens of a pass (LITENN_HIP_PASS_ROWS)
+		constexpr int kSplitRows = 1024;   // up to here a sublayer's last product may walk K in several ranges at once
 		constexpr int kAlignRows = 8;      // first row of every part of a concatenated matrix
 
 		struct LayerState
@@ -389,7 +390,7 @@ namespace litenn_hip
 			struct { void** p; size_t bytes; } bufs[] = {
 				{ reinterpret_cast<void**>(&x), 4 * rows * desc.width },
 				{ reinterpret_cast<void**>(&proj), 4 * rows * ld_proj },
-				{ reinterpret_cast<void**>(&y), 4 * rows * ld_y },
+				{ reinterpret_cast<void**>(&y), 4 * rows * ld_y * (rows <= kSplitRows ? kDenseMaxSplits : 1) },
 				{ reinterpret_cast<void**>(&q), 4 * rows * ld_q },
 				{ reinterpret_cast<void**>(&absorbed), 4 * absorbed_floats },
 				{ reinterpret_cast<void**>(&partial), 4 * partial_floats },
@@ -596,6 +597,8 @@ namespace litenn_hip
 			const Position pos{ d_counters, 0 };
 			launch_embed_rows(embed, ids, rows, turns, pos, x, d_err, stream);
 			const float* pending = nullptr;
+			int parts = 1; // y is the sum of so many buffers
+			const size_t part_stride = static_cast<size_t>(rows) * ld_y;
 			// x += norm(y) if a sublayer's output is pending, then h = norm(x) norm_w, of rows first ..
 			const auto enter = [&](const float* norm_w, int first, int count) {
 				AddNorm a;
@@ -605,6 +608,8 @@ namespace litenn_hip
 				{
 					a.sub = y + static_cast<size_t>(first) * ld_y;
 					a.ldsub = ld_y;
+					a.sub_parts = parts;
+					a.sub_stride = part_stride;
 					a.sub_w = pending;
 					a.x_out = x + static_cast<size_t>(first) * desc.width;
 				}
@@ -617,6 +622,20 @@ namespace litenn_hip
 				a.f32 = f32;
 				launch_add_norm(a, stream);
 				pending = nullptr;
+			};
+			const auto leave = [&](const DenseMatrix& w, const float* after) {
+				DenseRows d;
+				d.w = w;
+				d.a = mid;
+				d.lda = ld_mid;
+				d.m = rows;
+				d.c = y;
+				d.ldc = ld_y;
+				d.f32 = f32;
+				d.splits = parts = !f32 && rows <= kSplitRows ? dense_rows_splits(w, rows) : 1;
+				d.split_stride = part_stride;
+				launch_dense_rows(d, stream);
+				pending = after;
 			};
 			for (LayerState& L : layers)
 			{
@@ -638,14 +657,12 @@ namespace litenn_hip
 					g.chunk_states = chunk_states;
 					launch_gla_rows(g, stream);
 				}
-				product(L.out, mid, ld_mid, rows, y, ld_y, kOutF32);
-				pending = L.norm1b;
+				leave(L.out, L.norm1b);
 				if (L.desc.ff > 0)
 				{
 					enter(L.norm2, 0, rows);
 					product(L.gate_up, h, ld_h, rows, mid, ld_mid, kOutGlu, L.desc.act);
-					product(L.down, mid, ld_mid, rows, y, ld_y, kOutF32);
-					pending = L.norm2b;
+					leave(L.down, L.norm2b);
 				}
 			}
 			enter(final_norm, rows - logit_rows, logit_rows);

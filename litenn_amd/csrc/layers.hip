@@ -77,7 +77,9 @@ namespace litenn_hip
 		}
 
 		// ---------------- residual and norms -------------------------------------------------
-		template <typename T>
+		// PARTS: how many buffers `sub` may be the sum of (with fewer the last one is loaded again and dropped:
+		// the loads must not hang on branches)
+		template <typename T, int PARTS>
 		__global__ __launch_bounds__(256) void add_norm_kernel(const AddNorm a)
 		{
 			__shared__ float red[4];
@@ -87,13 +89,23 @@ namespace litenn_hip
 			float kept[kKept], added[kKept], sub_w[kKept], norm_w[kKept];
 			float scale_sub = 0.0f;
 			const float* sub = a.sub ? a.sub + static_cast<size_t>(row) * a.ldsub : nullptr;
+			const auto summed = [&](int i) {
+				float v = sub[i];
+#pragma unroll
+				for (int p = 1; p < PARTS; ++p)
+				{
+					const float t = sub[min(p, a.sub_parts - 1) * a.sub_stride + i];
+					v += p < a.sub_parts ? t : 0.0f;
+				}
+				return v;
+			};
 			// every load of the kept part is on its way before the first one is needed
 #pragma unroll
 			for (int e = 0; e < kKept; ++e)
 			{
 				const int i = threadIdx.x + 256 * e;
 				kept[e] = i < a.width ? x[i] : 0.0f;
-				added[e] = sub && i < a.width ? sub[i] : 0.0f;
+				added[e] = sub && i < a.width ? summed(i) : 0.0f;
 				sub_w[e] = sub && i < a.width ? a.sub_w[i] : 0.0f;
 				norm_w[e] = i < a.width ? a.norm_w[i] : 0.0f;
 			}
@@ -107,11 +119,12 @@ namespace litenn_hip
 				}
 				for (int i = threadIdx.x + 256 * kKept; i < a.width; i += 256)
 				{
-					ss = fmaf(sub[i], sub[i], ss);
+					const float v = summed(i);
+					ss = fmaf(v, v, ss);
 				}
 				scale_sub = 1.0f / sqrtf(block_sum256(ss, red) / static_cast<float>(a.width) + a.eps);
 			}
-			const auto value = [&](int i) { return sub ? x[i] + sub[i] * scale_sub * a.sub_w[i] : x[i]; };
+			const auto value = [&](int i) { return sub ? x[i] + summed(i) * scale_sub * a.sub_w[i] : x[i]; };
 			float ss = 0.0f;
 #pragma unroll
 			for (int e = 0; e < kKept; ++e)
@@ -259,7 +272,7 @@ namespace litenn_hip
 		// A workgroup takes four heads (one per wavefront) over one split of the visible positions, in tiles
 		// of kLatentTile cached rows staged in LDS as Float32; per split and head it leaves the running
 		// maximum, the sum of weights and the weighted sum of latents.
-		constexpr int kLatentTile = 32, kLatentHeads = 4, kLatentMaxRank = 1024;
+		constexpr int kLatentTile = 16, kLatentHeads = 4, kLatentMaxRank = 1024, kLatentMaxSplits = 64;
 
 		template <typename T>
 		__global__ __launch_bounds__(256) void latent_step_kernel(const LatentStep a)
@@ -279,10 +292,10 @@ namespace litenn_hip
 			const int per = (tiles + a.splits - 1) / a.splits;
 			const int t0 = split * per, t1 = min(tiles, t0 + per);
 			const T* const cache = static_cast<const T*>(a.cache.rows);
-			// eight threads per row of a tile, 16 bytes each at a time (the pitch is a multiple of 64); a row's
-			// first kAhead pieces per thread are requested before anything waits
-			constexpr int E = 16 / sizeof(T), kAhead = 8;
-			const int my_key = threadIdx.x >> 3, c0 = (threadIdx.x & 7) * E;
+			// kPer threads per row of a tile, 16 bytes each at a time; a row's first kAhead pieces per thread are
+			// requested before anything waits
+			constexpr int E = 16 / sizeof(T), kAhead = 4, kPer = 256 / kLatentTile, kStep = kPer * E;
+			const int my_key = threadIdx.x / kPer, c0 = (threadIdx.x % kPer) * E;
 			const auto row_of = [&](int base) {
 				const int count = min(kLatentTile, last - base + 1);
 				return cache + static_cast<size_t>((base + min(my_key, count - 1)) % a.cache.ring) * pitch + c0;
@@ -293,7 +306,7 @@ namespace litenn_hip
 #pragma unroll
 				for (int i = 0; i < kAhead; ++i)
 				{
-					ahead[i] = *reinterpret_cast<const u32x4*>(p + (8 * E * i < pitch ? 8 * E * i : 0));
+					ahead[i] = *reinterpret_cast<const u32x4*>(p + (c0 + kStep * i < pitch ? kStep * i : -c0));
 				}
 			};
 			if (t0 < t1)
@@ -338,13 +351,13 @@ namespace litenn_hip
 #pragma unroll
 					for (int i = 0; i < kAhead; ++i)
 					{
-						if (8 * E * i < pitch)
+						if (c0 + kStep * i < pitch)
 						{
-							store(8 * E * i, ahead[i]);
+							store(kStep * i, ahead[i]);
 						}
 					}
 					const T* p = row_of(base);
-					for (int c = 8 * E * kAhead; c < pitch; c += 8 * E)
+					for (int c = kStep * kAhead; c0 + c < pitch; c += kStep)
 					{
 						store(c, *reinterpret_cast<const u32x4*>(p + c));
 					}
@@ -354,15 +367,16 @@ namespace litenn_hip
 					}
 				}
 				__syncthreads();
-				// scores: two lanes per key, each half of the latent
-				const int key = lane & 31, part = lane >> 5;
+				// scores: kParts lanes per key, each a share of the latent
+				constexpr int kParts = 64 / kLatentTile;
+				const int key = lane % kLatentTile, part = lane / kLatentTile;
 				float acc = 0.0f;
 				{
 					const float* kr = &tile[key * stride];
 					const float* qr = &qa[wave * pitch];
-					const int half = pitch >> 1;
+					const int share = pitch / kParts; // the pitch is a multiple of 64
 #pragma unroll 8
-					for (int c = part * half; c < (part + 1) * half; c += 4)
+					for (int c = part * share; c < (part + 1) * share; c += 4)
 					{
 						const floatx4 kv = *reinterpret_cast<const floatx4*>(kr + c);
 						const floatx4 qv = *reinterpret_cast<const floatx4*>(qr + c);
@@ -372,12 +386,16 @@ namespace litenn_hip
 						acc = fmaf(kv.w, qv.w, acc);
 					}
 				}
-				acc += __shfl_xor(acc, 32, 64);
+#pragma unroll
+				for (int off = kLatentTile; off < 64; off *= 2)
+				{
+					acc += __shfl_xor(acc, off, 64);
+				}
 				const float score = key < count ? acc : -INFINITY;
 				const float new_m = fmaxf(run_m, wave_max(score));
 				const float corr = run_m == -INFINITY ? 0.0f : expf(run_m - new_m);
 				const float p = expf(score - new_m);
-				run_l = run_l * corr + 0.5f * wave_sum(p); // every key is held by two lanes
+				run_l = run_l * corr + wave_sum(part == 0 ? p : 0.0f);
 				run_m = new_m;
 				if (part == 0)
 				{
@@ -435,7 +453,8 @@ namespace litenn_hip
 		__global__ __launch_bounds__(256) void latent_value_kernel(const LatentStep a)
 		{
 			__shared__ __attribute__((aligned(16))) float o[kLatentMaxRank];
-			__shared__ float weight[64], sum;
+			__shared__ float weight[kLatentMaxSplits], sum;
+			__shared__ __attribute__((aligned(16))) float shares[1024];
 			const int pitch = a.cache.pitch;
 			const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
 			const int slices = (a.shape.vdim + kValueSlice - 1) / kValueSlice;
@@ -453,7 +472,8 @@ namespace litenn_hip
 			}
 			const size_t step = static_cast<size_t>(a.shape.heads) * (pitch + 4);
 			const float* part = a.partial + (static_cast<size_t>(row) * a.splits * a.shape.heads + h) * (pitch + 4);
-			// weights of the splits (at most 64; one without a visible position has maximum -inf and weight 0)
+			static_assert(kLatentMaxSplits == 64, "one lane per split");
+			// weights of the splits (one without a visible position has maximum -inf and weight 0)
 			if (wave == 0)
 			{
 				const float sink = a.shape.sink ? a.shape.sink[h] : -INFINITY;
@@ -469,27 +489,29 @@ namespace litenn_hip
 				}
 			}
 			__syncthreads();
-			const float total = sum;
-			float v[kLatentMaxRank / 256];
-#pragma unroll
-			for (int c = 0; c < kLatentMaxRank / 256; ++c)
+			// four latent columns per thread; the threads left over by one row of columns share out the splits
+			const int quads = pitch >> 2, groups = 256 / quads;
+			const int quad = static_cast<int>(threadIdx.x) % quads, group = static_cast<int>(threadIdx.x) / quads;
+			if (group < groups)
 			{
-				v[c] = 0.0f;
-				const int col = c * 256 + static_cast<int>(threadIdx.x);
-				if (col < a.cache.rank)
-				{
+				floatx4 v = { 0.0f, 0.0f, 0.0f, 0.0f };
 #pragma unroll 8
-					for (int s = 0; s < a.splits; ++s)
-					{
-						v[c] = fmaf(weight[s], part[s * step + col], v[c]);
-					}
+				for (int s = group; s < a.splits; s += groups)
+				{
+					v += weight[s] * *reinterpret_cast<const floatx4*>(part + s * step + 4 * quad);
 				}
+				*reinterpret_cast<floatx4*>(&shares[(group * quads + quad) * 4]) = v;
 			}
-			const float inv = 1.0f / total;
-#pragma unroll
-			for (int c = 0; c < kLatentMaxRank / 256; ++c)
+			__syncthreads();
+			const float inv = 1.0f / sum;
+			for (int c = threadIdx.x; c < pitch; c += 256)
 			{
-				o[c * 256 + threadIdx.x] = v[c] * inv;
+				float t = 0.0f;
+				for (int i = 0; i < groups; ++i)
+				{
+					t += shares[i * pitch + c];
+				}
+				o[c] = c < a.cache.rank ? t * inv : 0.0f;
 			}
 			__syncthreads();
 #pragma unroll
@@ -1510,13 +1532,18 @@ namespace litenn_hip
 		{
 			return;
 		}
+		const dim3 grid(a.rows), threads(256);
 		if (a.f32)
 		{
-			add_norm_kernel<float><<<dim3(a.rows), dim3(256), 0, s>>>(a);
+			add_norm_kernel<float, 1><<<grid, threads, 0, s>>>(a);
+		}
+		else if (!a.sub || a.sub_parts == 1)
+		{
+			add_norm_kernel<uint16_t, 1><<<grid, threads, 0, s>>>(a);
 		}
 		else
 		{
-			add_norm_kernel<uint16_t><<<dim3(a.rows), dim3(256), 0, s>>>(a);
+			add_norm_kernel<uint16_t, kDenseMaxSplits><<<grid, threads, 0, s>>>(a);
 		}
 	}
 
@@ -1544,7 +1571,7 @@ namespace litenn_hip
 	{
 		const int groups = (heads + kLatentHeads - 1) / kLatentHeads * rows;
 		const int tiles = (window + kLatentTile - 1) / kLatentTile;
-		return std::max(1, std::min({ tiles, 512 / std::max(1, groups), 64 }));
+		return std::max(1, std::min({ tiles, 512 / std::max(1, groups), kLatentMaxSplits }));
 	}
 
 	size_t latent_step_partial_floats(int heads, int rows, int pitch, int splits)

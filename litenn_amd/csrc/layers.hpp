@@ -25,6 +25,8 @@ namespace litenn_hip
 		int ldx = 0;
 		const float* sub = nullptr;
 		int ldsub = 0;
+		int sub_parts = 1; // sub is the sum of so many buffers, sub_stride floats apart
+		size_t sub_stride = 0;
 		const float* sub_w = nullptr;
 		float* x_out = nullptr; // may be x; rows ldx apart
 		const float* norm_w = nullptr;
