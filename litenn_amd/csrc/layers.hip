@@ -447,41 +447,58 @@ namespace litenn_hip
 
 		// Merges the splits (and the sink), takes the result through W_uv, applies the gate.  A workgroup
 		// makes kValueSlice outputs of one head.
-		constexpr int kValueSlice = 32;
+		constexpr int kValueSlice = 32, kValueThreads = 512;
 
 		template <typename T>
-		__global__ __launch_bounds__(256) void latent_value_kernel(const LatentStep a)
+		__global__ __launch_bounds__(kValueThreads) void latent_value_kernel(const LatentStep a)
 		{
 			__shared__ __attribute__((aligned(16))) float o[kLatentMaxRank];
 			__shared__ float weight[kLatentMaxSplits], sum;
-			__shared__ __attribute__((aligned(16))) float shares[1024];
+			__shared__ __attribute__((aligned(16))) float shares[4 * kValueThreads];
 			const int pitch = a.cache.pitch;
 			const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
 			const int slices = (a.shape.vdim + kValueSlice - 1) / kValueSlice;
 			const int h = static_cast<int>(blockIdx.x) / slices, slice = static_cast<int>(blockIdx.x) % slices;
 			const int row = blockIdx.y;
-			// this wavefront's first rows of W_uv (a rank of up to 512 is one piece per lane), ahead of the merge
-			constexpr int kRows = kValueSlice / 4;
+			const size_t step = static_cast<size_t>(a.shape.heads) * (pitch + 4);
+			const float* part = a.partial + (static_cast<size_t>(row) * a.splits * a.shape.heads + h) * (pitch + 4);
+			// Everything this workgroup reads is requested before anything waits: the splits' maxima and sums, its
+			// first latents (four columns per thread; the threads left over by one row of columns share out the
+			// splits), this wavefront's rows of W_uv (a rank of up to 512 is one piece per lane) and its gates.
+			static_assert(kLatentMaxSplits == 64, "one lane per split");
+			const float split_m = lane < a.splits ? part[lane * step + pitch] : -INFINITY;
+			const float split_l = lane < a.splits ? part[lane * step + pitch + 1] : 0.0f;
+			const int quads = pitch >> 2, groups = kValueThreads / quads;
+			const int quad = static_cast<int>(threadIdx.x) % quads, group = static_cast<int>(threadIdx.x) / quads;
+			constexpr int kAhead = 16;
+			floatx4 ahead[kAhead];
+#pragma unroll
+			for (int i = 0; i < kAhead; ++i)
+			{
+				ahead[i] = *reinterpret_cast<const floatx4*>(part + min(group + i * groups, a.splits - 1) * step + 4 * quad);
+			}
+			constexpr int kWaves = kValueThreads / 64, kRows = kValueSlice / kWaves;
 			u32x4 first[kRows];
 #pragma unroll
 			for (int i = 0; i < kRows; ++i)
 			{
-				const int e = min(slice * kValueSlice + wave + 4 * i, a.shape.vdim - 1);
+				const int e = min(slice * kValueSlice + wave + kWaves * i, a.shape.vdim - 1);
 				first[i] = *reinterpret_cast<const u32x4*>(a.uv.w + static_cast<size_t>(h * a.shape.vdim + e) * a.uv.pitch +
 				                                           (lane * 8 < pitch ? lane * 8 : 0));
 			}
-			const size_t step = static_cast<size_t>(a.shape.heads) * (pitch + 4);
-			const float* part = a.partial + (static_cast<size_t>(row) * a.splits * a.shape.heads + h) * (pitch + 4);
-			static_assert(kLatentMaxSplits == 64, "one lane per split");
+			float gates = 0.0f; // lane i: row i
+			if (a.gate && lane < kRows)
+			{
+				const int e = min(slice * kValueSlice + wave + kWaves * lane, a.shape.vdim - 1);
+				gates = a.gate[static_cast<size_t>(row) * a.ldg + h * a.shape.vdim + e];
+			}
 			// weights of the splits (one without a visible position has maximum -inf and weight 0)
 			if (wave == 0)
 			{
 				const float sink = a.shape.sink ? a.shape.sink[h] : -INFINITY;
-				const float m = lane < a.splits ? part[lane * step + pitch] : -INFINITY;
-				const float l = lane < a.splits ? part[lane * step + pitch + 1] : 0.0f;
-				const float top = fmaxf(wave_max(m), sink);
-				const float w = expf(m - top);
-				const float all = wave_sum(w * l);
+				const float top = fmaxf(wave_max(split_m), sink);
+				const float w = expf(split_m - top);
+				const float all = wave_sum(w * split_l);
 				weight[lane] = w;
 				if (lane == 0)
 				{
@@ -489,14 +506,16 @@ namespace litenn_hip
 				}
 			}
 			__syncthreads();
-			// four latent columns per thread; the threads left over by one row of columns share out the splits
-			const int quads = pitch >> 2, groups = 256 / quads;
-			const int quad = static_cast<int>(threadIdx.x) % quads, group = static_cast<int>(threadIdx.x) / quads;
 			if (group < groups)
 			{
 				floatx4 v = { 0.0f, 0.0f, 0.0f, 0.0f };
-#pragma unroll 8
-				for (int s = group; s < a.splits; s += groups)
+#pragma unroll
+				for (int i = 0; i < kAhead; ++i)
+				{
+					const int s = group + i * groups;
+					v += (s < a.splits ? weight[min(s, kLatentMaxSplits - 1)] : 0.0f) * ahead[i];
+				}
+				for (int s = group + kAhead * groups; s < a.splits; s += groups)
 				{
 					v += weight[s] * *reinterpret_cast<const floatx4*>(part + s * step + 4 * quad);
 				}
@@ -504,7 +523,7 @@ namespace litenn_hip
 			}
 			__syncthreads();
 			const float inv = 1.0f / sum;
-			for (int c = threadIdx.x; c < pitch; c += 256)
+			for (int c = threadIdx.x; c < pitch; c += kValueThreads)
 			{
 				float t = 0.0f;
 				for (int i = 0; i < groups; ++i)
@@ -517,7 +536,7 @@ namespace litenn_hip
 #pragma unroll
 			for (int i = 0; i < kRows; ++i)
 			{
-				const int e = slice * kValueSlice + wave + 4 * i;
+				const int e = slice * kValueSlice + wave + kWaves * i;
 				if (e >= a.shape.vdim)
 				{
 					break;
@@ -539,14 +558,14 @@ namespace litenn_hip
 					acc = fmaf(__uint_as_float(x.w & 0xffff0000u), o1.w, acc);
 				}
 				acc = wave_sum(acc);
+				const float gate = __shfl(gates, i, 64);
 				if (lane == 0)
 				{
-					const int col = h * a.shape.vdim + e;
 					if (a.gate)
 					{
-						acc *= sigmoid_f32(a.gate[static_cast<size_t>(row) * a.ldg + col]);
+						acc *= sigmoid_f32(gate);
 					}
-					operand_store(static_cast<T*>(a.out) + static_cast<size_t>(row) * a.ldo + col, acc);
+					operand_store(static_cast<T*>(a.out) + static_cast<size_t>(row) * a.ldo + h * a.shape.vdim + e, acc);
 				}
 			}
 		}
@@ -1600,11 +1619,11 @@ namespace litenn_hip
 		const dim3 value(a.shape.heads * ((a.shape.vdim + kValueSlice - 1) / kValueSlice), a.rows);
 		if (a.out_f32)
 		{
-			latent_value_kernel<float><<<value, dim3(256), 0, s>>>(a);
+			latent_value_kernel<float><<<value, dim3(kValueThreads), 0, s>>>(a);
 		}
 		else
 		{
-			latent_value_kernel<uint16_t><<<value, dim3(256), 0, s>>>(a);
+			latent_value_kernel<uint16_t><<<value, dim3(kValueThreads), 0, s>>>(a);
 		}
 	}
 

@@ -260,13 +260,18 @@ def test_clamped_feed_forward(hip, dtype):
     model.close()
 
 
+def lively(w):
+    """Small embeddings under full-size sublayers: the tied head then does not answer every token with itself."""
+    w["embed"] *= 0.1
+
+
 def test_greedy_generation(hip):
     """generate(): the prompt in passes, then the captured step, against the plain form's greedy tokens; again
     after other work on the same model (replays of the same captured step), and continued."""
-    model, plain = pair(hip, MIXED, 71, "float32")
-    prompt = ku.tokens(MIXED, 45, 13)
+    model, plain = pair(hip, MIXED, 71, "float32", edit=lively)
+    prompt = ku.tokens(MIXED, 45, 12)
     want, margins = plain.greedy(prompt, 40)
-    assert min(margins) > 1e-4  # no near-tie in this sequence
+    assert min(margins) > 2e-3 and len(set(want)) > 15  # no near-tie in this sequence, no single repeated token
     for _ in range(3):
         model.reset()
         got, _, _ = model.generate(prompt, 40)
@@ -283,7 +288,7 @@ def test_greedy_generation(hip):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_the_captured_step_equals_the_eager_one(hip, dtype, monkeypatch):
-    w = ku.random_weights(MIXED, 72)
+    w = ku.random_weights(MIXED, 72, edit=lively)
     prompt = ku.tokens(MIXED, 37, 15)
     got = []
     for graph in ("1", "0"):
@@ -297,8 +302,8 @@ def test_the_captured_step_equals_the_eager_one(hip, dtype, monkeypatch):
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_generation_in_portions_of_the_prompt(hip, dtype):
     """The prompt fed ahead in portions, or all by generate() itself: the same tokens."""
-    model, plain = pair(hip, MIXED, 73, dtype)
-    prompt = ku.tokens(MIXED, 90, 16)
+    model, plain = pair(hip, MIXED, 73, dtype, edit=lively)
+    prompt = ku.tokens(MIXED, 90, 15)
     whole, _, _ = model.generate(prompt, 12)
     model.reset()
     model.eval(prompt[:50], want=[])
