@@ -15,7 +15,7 @@ LIB_PATH = os.path.join(LIB_DIR, "liblitenn_hip.so")
 TRACE_LIB_PATH = os.path.join(LIB_DIR, "liblitenn_hip_trace.so")
 
 SOURCES = ["api.hip", "gemv.hip", "gemm.hip", "glue.hip", "attn_tile.hip", "primitives.hip", "decoder.hip", "llama.hip", "gguf.hip",
-           "checkpoint.hip", "dense.hip", "layers.hip", "layer_ops.hip", "layered.hip", "registry.hip"]
+           "checkpoint.hip", "dense.hip", "layers.hip", "mixers.hip", "layer_ops.hip", "layered.hip", "registry.hip"]
 # gemv.hip: the dispatcher hands the first six kernel arguments over in registers (the streaming
 # kernel's activation pointer, K and first-row addressing), see gemv_stream_kernel
 # glue.hip: the attention step's pointers, among them the device-resident position it loads first

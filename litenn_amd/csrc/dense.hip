@@ -135,7 +135,7 @@ namespace litenn_hip
 					x[e] = load_piece(d.x, i, k);
 					sub[e] = d.sub ? load_piece(d.sub, i, k) : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
 					subw[e] = d.sub ? load_piece(d.sub_w, i, k) : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f };
-					nw[e] = load_piece(d.norm_w, i, k);
+					nw[e] = d.norm_w ? load_piece(d.norm_w, i, k) : floatx4{ 1.0f, 1.0f, 1.0f, 1.0f };
 				}
 				float scale_sub = 0.0f;
 				if (d.sub)
@@ -180,9 +180,10 @@ namespace litenn_hip
 				for (int p = threadIdx.x + kRowThreads * kKept; p < pieces; p += kRowThreads)
 				{
 					put(p, enter(p, load_piece(d.x, 4 * p, k), d.sub ? load_piece(d.sub, 4 * p, k) : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f },
-					             d.sub ? load_piece(d.sub_w, 4 * p, k) : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f }, load_piece(d.norm_w, 4 * p, k)));
+					             d.sub ? load_piece(d.sub_w, 4 * p, k) : floatx4{ 0.0f, 0.0f, 0.0f, 0.0f },
+					             d.norm_w ? load_piece(d.norm_w, 4 * p, k) : floatx4{ 1.0f, 1.0f, 1.0f, 1.0f }));
 				}
-				const float scale = 1.0f / sqrtf(block_sum(ss, red) / static_cast<float>(k) + d.eps);
+				const float scale = d.norm_w ? 1.0f / sqrtf(block_sum(ss, red) / static_cast<float>(k) + d.eps) : 1.0f;
 #pragma unroll
 				for (int e = 0; e < kKept; ++e)
 				{
@@ -308,7 +309,7 @@ namespace litenn_hip
 							{
 								if (rg * R + r < n)
 								{
-									d.y[rg * R + r] = acc[r];
+									d.y[rg * R + r] = soft_cap(acc[r], d.softcap);
 								}
 							}
 						}
@@ -392,7 +393,7 @@ namespace litenn_hip
 			{
 				return;
 			}
-			const float f[4] = { v.x, v.y, v.z, v.w };
+			float f[4] = { v.x, v.y, v.z, v.w };
 			if (d.out == kOutGlu)
 			{
 				T* c = static_cast<T*>(d.c) + static_cast<size_t>(m) * d.ldc + (n >> 1);
@@ -421,6 +422,14 @@ namespace litenn_hip
 					}
 				}
 				return;
+			}
+			if (d.softcap > 0.0f)
+			{
+#pragma unroll
+				for (int i = 0; i < 4; ++i)
+				{
+					f[i] = soft_cap(f[i], d.softcap);
+				}
 			}
 			float* c = static_cast<float*>(d.c) + blockIdx.y * d.split_stride + static_cast<size_t>(m) * d.ldc + n;
 			if (n + 3 < d.w.n && (d.ldc & 3) == 0)

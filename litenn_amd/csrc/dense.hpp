@@ -17,7 +17,8 @@ namespace litenn_hip
 		int n = 0, k = 0, pitch = 0;
 	};
 
-	// y = g sigmoid(alpha g) (u + shift) with g = min(g, limit), u = clamp(u, -limit, limit)
+	// y = g sigmoid(alpha g) (u + shift) with g = min(g, limit), u = clamp(u, -limit, limit); an infinite limit,
+	// alpha 1 and shift 0 make it silu(g) u
 	struct ClampedGlu
 	{
 		float limit = 0.0f, alpha = 0.0f, shift = 0.0f;
@@ -27,7 +28,7 @@ namespace litenn_hip
 	enum DensePrologue
 	{
 		kRowPlain = 0,    // x as it is
-		kRowAddNorm = 1,  // x' = x + norm(sub) sub_w (sub may be null), then norm(x') norm_w; x' -> x_out if given
+		kRowAddNorm = 1,  // x' = x + norm(sub) sub_w (sub may be null); x' -> x_out if given; norm(x') norm_w, or x' without norm_w
 		kRowHeadGate = 2, // per head of `vdim`: norm(x) norm_w, then times silu(gate)
 	};
 	struct DenseRow
@@ -45,6 +46,7 @@ namespace litenn_hip
 		float eps = 0.0f;
 		bool glu = false; // rows 2i and 2i + 1 are gate and up of output i
 		ClampedGlu act;
+		float softcap = 0.0f; // > 0: y becomes softcap tanh(y / softcap)
 	};
 	// false, with nothing launched, when k does not fit the workgroup's LDS
 	bool launch_dense_row(const DenseRow& a, hipStream_t s);
@@ -73,6 +75,7 @@ namespace litenn_hip
 		size_t split_stride = 0;
 		bool f32 = false; // Float32 operands (the bfloat16 weights widened exactly), f32 matrix instructions
 		ClampedGlu act;
+		float softcap = 0.0f; // kOutF32: > 0: c becomes softcap tanh(c / softcap)
 	};
 	constexpr int kDenseMaxSplits = 4;
 	int dense_rows_splits(const DenseMatrix& w, int m);
@@ -101,6 +104,8 @@ namespace litenn_hip
 	__device__ __forceinline__ void operand_store(float* p, float v) { *p = v; }
 
 	__device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+	__device__ __forceinline__ float soft_cap(float v, float cap) { return cap > 0.0f ? cap * tanhf(v / cap) : v; }
 
 	__device__ __forceinline__ float clamped_glu(float g, float u, const ClampedGlu& c)
 	{

@@ -107,6 +107,8 @@ extern "C" int litenn_hip_window_attn(int dev, const void* q, const void* kv, in
 	a.kv = kv;
 	a.ldkv = static_cast<int>(heads * (dim + vdim));
 	a.v_first = static_cast<int>(heads * dim);
+	a.k_head = dim;
+	a.v_head = vdim;
 	a.keys = static_cast<int>(keys);
 	a.key_base = static_cast<int>(o->key_position);
 	a.rows = static_cast<int>(m);

@@ -2,9 +2,11 @@
 //
 // Memory: weights stay in bfloat16; projections that read the same input are one matrix (their rows
 // concatenated, so a layer's first product is one launch), gate and up rows of a feed-forward are
-// interleaved so that the launch forms their product.  A latent-attention layer keeps a ring of
-// normalised latents, long enough for its window plus one pass of tokens, a gated linear attention
-// layer its Float32 state: what a sequence holds does not grow with its length beyond the window.
+// interleaved so that the launch forms their product.  Mixers that run side by side share the input
+// projection and, with their weights folded into what it reads, the output projection.  An attention layer
+// keeps a ring of normalised latents, or of keys and values, long enough for its window plus one pass of tokens, a
+// recurrent layer its Float32 state: what a sequence holds does not grow with its length beyond the window.
+// Layers that use another's weights hold a cache and state of their own.
 //
 // A pass of kRowsMin tokens and more runs on the matrix cores, fewer tokens go one by one through the
 // single-row form, whose launches read their position from device memory (so that one can be
@@ -32,13 +34,11 @@ namespace litenn_hip
 		constexpr int kSplitRows = 1024;   // up to here a sublayer's last product may walk K in several ranges at once
 		constexpr int kAlignRows = 8;      // first row of every part of a concatenated matrix
 
-		struct LayerState
+		struct MixerState
 		{
-			LayerDesc desc;
-			const float *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr;
-			DenseMatrix in, out; // concatenated input projections, output projection
-			// first columns of the parts of `in`'s product
-			int at_q = 0, at_k = 0, at_v = 0, at_gate = 0, at_low = 0, at_latent = 0;
+			MixerDesc desc;
+			// first columns of the parts of the input projections' product, and of its share of the output projection's input
+			int at_q = 0, at_k = 0, at_v = 0, at_gate = 0, at_low = 0, at_latent = 0, at_in = 0, at_mid = 0;
 			// latent attention
 			DenseMatrix uq, uk, uv, ukv; // uk and uv are rows of ukv
 			int v_first = 0;
@@ -49,6 +49,23 @@ namespace litenn_hip
 			DenseMatrix a2;
 			const float *a2_bias = nullptr, *head_norm = nullptr;
 			float* state = nullptr;
+			// grouped attention
+			const float* k_norm = nullptr; // beside q_norm
+			const double* turns = nullptr;
+			HeadCache heads;
+			// state space
+			const float *conv_w = nullptr, *conv_b = nullptr, *dt_bias = nullptr, *a_log = nullptr, *skip = nullptr,
+			            *group_norm = nullptr;
+			float* ring = nullptr; // the convolution's last inputs
+		};
+
+		struct LayerState
+		{
+			LayerDesc desc;
+			// norms ahead of the sublayers (null where there are none) and behind them
+			const float *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr;
+			DenseMatrix in, out; // concatenated input projections, output projection
+			std::vector<MixerState> mixers;
 			// feed-forward
 			DenseMatrix gate_up, down;
 		};
@@ -57,7 +74,7 @@ namespace litenn_hip
 		struct Slot
 		{
 			uint16_t* matrix = nullptr; // bfloat16 rows, `stride` elements apart
-			float* vector = nullptr;    // Float32 [rows]
+			float* vector = nullptr;    // Float32 [rows], or [cols, rows] of a tensor [rows, cols]
 			size_t rows = 0, cols = 0, stride = 0;
 			bool filled = false;
 		};
@@ -67,9 +84,9 @@ namespace litenn_hip
 	{
 		LayeredDesc desc;
 		bool f32 = false;
-		DenseMatrix embed;
+		DenseMatrix embed, head;
 		const float* final_norm = nullptr;
-		double* turns = nullptr;
+		const double* turns = nullptr;
 		std::vector<LayerState> layers;
 		std::map<std::string, Slot> slots;
 		int max_pass = kPassRows;
@@ -77,11 +94,11 @@ namespace litenn_hip
 		// scratch for cap_rows tokens
 		size_t cap_rows = 0;
 		float *x = nullptr, *proj = nullptr, *y = nullptr, *q = nullptr, *absorbed = nullptr, *partial = nullptr,
-		      *log_decay = nullptr, *chunk_states = nullptr;
+		      *log_decay = nullptr, *chunk_states = nullptr, *xbc = nullptr;
 		void *h = nullptr, *mid = nullptr, *kv = nullptr;
 		int ld_proj = 0, ld_y = 0, ld_q = 0, ld_h = 0, ld_mid = 0, ld_kv = 0;
 		// single-row form
-		float *xt[2] = { nullptr, nullptr }, *row_mid = nullptr;
+		float *xt[2] = { nullptr, nullptr }, *row_mid = nullptr, *row_ssm = nullptr;
 
 		~LayeredModel() override { free_scratch(); }
 
@@ -89,7 +106,8 @@ namespace litenn_hip
 		{
 			void** bufs[] = { reinterpret_cast<void**>(&x),       reinterpret_cast<void**>(&proj), reinterpret_cast<void**>(&y),
 				              reinterpret_cast<void**>(&q),       reinterpret_cast<void**>(&absorbed), reinterpret_cast<void**>(&partial),
-				              reinterpret_cast<void**>(&log_decay), reinterpret_cast<void**>(&chunk_states), &h, &mid, &kv };
+				              reinterpret_cast<void**>(&log_decay), reinterpret_cast<void**>(&chunk_states),
+				              reinterpret_cast<void**>(&xbc), &h, &mid, &kv };
 			for (void** b : bufs)
 			{
 				if (*b)
@@ -175,6 +193,51 @@ namespace litenn_hip
 			return m;
 		}
 
+		// the tensors' columns one behind the other: their products, added
+		DenseMatrix side_by_side(const std::vector<std::pair<std::string, int>>& parts, int rows)
+		{
+			int cols = 0;
+			for (const auto& p : parts)
+			{
+				cols += p.second;
+			}
+			DenseMatrix m = matrix({ { parts[0].first, rows, nullptr } }, cols);
+			const Slot whole = slots[parts[0].first];
+			int at = 0;
+			for (const auto& p : parts)
+			{
+				Slot s = whole;
+				s.matrix = whole.matrix + at;
+				s.cols = static_cast<size_t>(p.second);
+				slots[p.first] = s;
+				at += p.second;
+			}
+			return m;
+		}
+
+		const double* turns_per_position(double base, int dims)
+		{
+			std::vector<double> f((static_cast<size_t>(dims) + 1) / 2);
+			for (size_t i = 0; i < f.size(); ++i)
+			{
+				f[i] = std::pow(base, -2.0 * static_cast<double>(i) / dims) / (2.0 * M_PI);
+			}
+			double* p = static_cast<double*>(allocate(sizeof(double) * f.size()));
+			copy_in(p, f.data(), sizeof(double) * f.size());
+			return p;
+		}
+
+		// a tensor [rows, cols], kept column by column
+		const float* columns(const std::string& name, int rows, int cols)
+		{
+			Slot s;
+			s.vector = static_cast<float*>(allocate(sizeof(float) * static_cast<size_t>(rows) * cols));
+			s.rows = static_cast<size_t>(rows);
+			s.cols = static_cast<size_t>(cols);
+			slots[name] = s;
+			return s.vector;
+		}
+
 		const float* vector(const std::string& name, int n)
 		{
 			Slot s;
@@ -184,73 +247,193 @@ namespace litenn_hip
 			return s.vector;
 		}
 
+		// weights of one mixer: its input projections join `parts`, its output projection `outs`
+		void build_mixer(const std::string& mix, MixerState& M, std::vector<Part>& parts, std::vector<std::pair<std::string, int>>& outs)
+		{
+			const MixerDesc& m = M.desc;
+			const int values = m.heads * m.vdim, keys = m.heads * m.dim;
+			switch (m.kind)
+			{
+			case MixerKind::LatentAttention: {
+				parts.insert(parts.end(), { { mix + "dq", m.q_rank, &M.at_q }, { mix + "dkv", m.kv_rank, &M.at_latent }, { mix + "g", values, &M.at_gate } });
+				M.q_norm = vector(mix + "dq.norm", m.q_rank);
+				M.latent_norm = vector(mix + "dkv.norm", m.kv_rank);
+				M.sink = vector(mix + "sink", m.heads);
+				M.uq = matrix({ { mix + "uq", keys, nullptr } }, m.q_rank);
+				int uv_at = 0;
+				M.ukv = matrix({ { mix + "uk", keys, nullptr }, { mix + "uv", values, &uv_at } }, m.kv_rank);
+				M.v_first = uv_at;
+				M.uk = M.uv = M.ukv;
+				M.uk.n = keys;
+				M.uv.n = values;
+				M.uv.w = M.ukv.w + static_cast<size_t>(uv_at) * M.ukv.pitch;
+				break;
+			}
+			case MixerKind::GatedLinearAttention:
+				parts.insert(parts.end(), { { mix + "q", keys, &M.at_q }, { mix + "k", keys, &M.at_k }, { mix + "v", values, &M.at_v },
+				                            { mix + "g", values, &M.at_gate }, { mix + "a1", m.decay_rank, &M.at_low } });
+				M.a2 = matrix({ { mix + "a2", keys, nullptr } }, m.decay_rank);
+				M.a2_bias = vector(mix + "a2.b", keys);
+				M.head_norm = vector(mix + "norm", m.vdim);
+				break;
+			case MixerKind::GroupedAttention:
+				parts.insert(parts.end(), { { mix + "q", keys, &M.at_q }, { mix + "k", m.kv_heads * m.dim, &M.at_k } });
+				if (!m.values_are_keys)
+				{
+					parts.push_back({ mix + "v", m.kv_heads * m.vdim, &M.at_v });
+				}
+				if (m.projection_norm)
+				{
+					M.q_norm = vector(mix + "q.norm", keys);
+					M.k_norm = vector(mix + "k.norm", m.kv_heads * m.dim);
+				}
+				if (m.rot_dims > 0)
+				{
+					M.turns = turns_per_position(m.rot_base, m.rot_dims);
+				}
+				break;
+			case MixerKind::StateSpace: {
+				const int channels = values + 2 * m.groups * m.state;
+				parts.push_back({ mix + "in", values + channels + m.heads, &M.at_in });
+				M.conv_w = columns(mix + "conv", channels, m.taps);
+				M.conv_b = vector(mix + "conv.b", channels);
+				M.dt_bias = vector(mix + "dt_bias", m.heads);
+				M.a_log = vector(mix + "A_log", m.heads);
+				M.skip = vector(mix + "D", m.heads);
+				M.group_norm = vector(mix + "norm", values);
+				break;
+			}
+			}
+			outs.emplace_back(mix + "o", values);
+		}
+
+		void build_weights(const std::string& p, LayerState& L)
+		{
+			const int width = desc.width;
+			const bool around = desc.norms == NormPlacement::Around;
+			(around ? L.norm1 : L.norm1b) = vector(p + "norm1", width);
+			if (around)
+			{
+				L.norm1b = vector(p + "norm1b", width);
+			}
+			std::vector<Part> parts;
+			std::vector<std::pair<std::string, int>> outs;
+			L.mixers.resize(L.desc.mixers.size()); // before their members' addresses go into `parts`
+			for (size_t i = 0; i < L.mixers.size(); ++i)
+			{
+				MixerState& M = L.mixers[i];
+				M.desc = L.desc.mixers[i];
+				for (const auto& before : outs)
+				{
+					M.at_mid += before.second;
+				}
+				build_mixer(p + "mix." + M.desc.name, M, parts, outs);
+			}
+			L.in = matrix(parts, width);
+			for (MixerState& M : L.mixers)
+			{
+				if (M.desc.kind == MixerKind::GroupedAttention && M.desc.values_are_keys)
+				{
+					M.at_v = M.at_k;
+				}
+			}
+			L.out = side_by_side(outs, width);
+			if (L.desc.ff > 0)
+			{
+				const int ff = L.desc.ff;
+				(around ? L.norm2 : L.norm2b) = vector(p + "norm2", width);
+				if (around)
+				{
+					L.norm2b = vector(p + "norm2b", width);
+				}
+				L.gate_up = interleaved(p + "mlp.gate", p + "mlp.up", ff, width);
+				L.down = matrix({ { p + "mlp.down", width, nullptr } }, ff);
+			}
+		}
+
+		// what a sequence holds in one mixer
+		void build_state(MixerState& M)
+		{
+			MixerDesc& m = M.desc;
+			m.window = m.window > 0 ? std::min(m.window, context_length) : context_length;
+			// a pass appends before it reads: the window behind its first token must survive
+			const int ring = static_cast<int>(std::min<long long>(context_length, static_cast<long long>(m.window) - 1 + max_pass));
+			switch (m.kind)
+			{
+			case MixerKind::LatentAttention:
+				M.cache.ring = ring;
+				M.cache.rank = m.kv_rank;
+				M.cache.pitch = M.ukv.pitch;
+				M.cache.f32 = f32;
+				M.cache.rows = allocate((f32 ? 4 : 2) * static_cast<size_t>(ring) * M.cache.pitch);
+				M.splits = latent_step_splits(m.heads, 1, m.window);
+				break;
+			case MixerKind::GatedLinearAttention:
+				M.state = static_cast<float*>(allocate(sizeof(float) * state_floats(m)));
+				break;
+			case MixerKind::GroupedAttention:
+				M.heads.ring = ring;
+				M.heads.heads = m.kv_heads;
+				M.heads.dim = m.dim;
+				M.heads.vdim = m.vdim;
+				M.heads.f32 = f32;
+				M.heads.rows = allocate((f32 ? 4 : 2) * M.heads.elements());
+				M.splits = grouped_step_splits(m.heads, m.kv_heads, m.dim, m.vdim, m.window);
+				break;
+			case MixerKind::StateSpace:
+				M.state = static_cast<float*>(allocate(sizeof(float) * state_floats(m)));
+				M.ring = static_cast<float*>(allocate(sizeof(float) * m.taps * static_cast<size_t>(ssm_args(M).channels())));
+				break;
+			}
+		}
+
 		void build()
 		{
 			const int width = desc.width;
 			embed = matrix({ { "embed", desc.vocab, nullptr } }, width);
+			head = desc.tied_head ? embed : matrix({ { "head", desc.vocab, nullptr } }, width);
 			final_norm = vector("final.norm", width);
-			int widest_mid = std::max(width, 64), proj_cols = 0, q_cols = 4, kv_cols = 0;
-			for (size_t i = 0; i < desc.layers.size(); ++i)
+			layers.resize(desc.layers.size());
+			for (size_t i = 0; i < layers.size(); ++i)
 			{
-				layers.emplace_back();
-				LayerState& L = layers.back();
-				L.desc = desc.layers[i];
-				const MixerDesc& m = L.desc.mixer;
-				const std::string p = "l" + std::to_string(i) + ".", mix = p + "mix.";
-				L.norm1 = vector(p + "norm1", width);
-				L.norm1b = vector(p + "norm1b", width);
-				const int values = m.heads * m.vdim, keys = m.heads * m.dim;
-				if (m.kind == MixerKind::LatentAttention)
+				layers[i].desc = desc.layers[i];
+				if (layers[i].desc.weights_of < 0)
 				{
-					L.in = matrix({ { mix + "dq", m.q_rank, &L.at_q }, { mix + "dkv", m.kv_rank, &L.at_latent }, { mix + "g", values, &L.at_gate } },
-					              width);
-					L.q_norm = vector(mix + "dq.norm", m.q_rank);
-					L.latent_norm = vector(mix + "dkv.norm", m.kv_rank);
-					L.sink = vector(mix + "sink", m.heads);
-					L.uq = matrix({ { mix + "uq", keys, nullptr } }, m.q_rank);
-					int uv_at = 0;
-					L.ukv = matrix({ { mix + "uk", keys, nullptr }, { mix + "uv", values, &uv_at } }, m.kv_rank);
-					L.v_first = uv_at;
-					L.uk = L.uv = L.ukv;
-					L.uk.n = keys;
-					L.uv.n = values;
-					L.uv.w = L.ukv.w + static_cast<size_t>(uv_at) * L.ukv.pitch;
-					const int window = m.window > 0 ? std::min(m.window, context_length) : context_length;
-					L.desc.mixer.window = window;
-					// a pass appends before it reads: the window behind its first token must survive
-					const long long ring = std::min<long long>(context_length, static_cast<long long>(window) - 1 + max_pass);
-					L.cache.ring = static_cast<int>(ring);
-					L.cache.rank = m.kv_rank;
-					L.cache.pitch = L.ukv.pitch;
-					L.cache.f32 = f32;
-					L.cache.rows = allocate((f32 ? 4 : 2) * static_cast<size_t>(ring) * L.cache.pitch);
-					L.splits = latent_step_splits(m.heads, 1, window);
-					q_cols = std::max(q_cols, keys);
-					kv_cols = std::max(kv_cols, L.ukv.n);
-					widest_mid = std::max({ widest_mid, values, m.q_rank });
+					build_weights("l" + std::to_string(i) + ".", layers[i]);
 				}
-				else
+			}
+			int widest_mid = std::max(width, 64), proj_cols = 0, q_cols = 4, kv_cols = 0, ssm_cols = 4;
+			for (LayerState& L : layers)
+			{
+				if (L.desc.weights_of >= 0)
 				{
-					L.in = matrix({ { mix + "q", keys, &L.at_q }, { mix + "k", keys, &L.at_k }, { mix + "v", values, &L.at_v },
-					                { mix + "g", values, &L.at_gate }, { mix + "a1", m.decay_rank, &L.at_low } },
-					              width);
-					L.a2 = matrix({ { mix + "a2", keys, nullptr } }, m.decay_rank);
-					L.a2_bias = vector(mix + "a2.b", keys);
-					L.head_norm = vector(mix + "norm", m.vdim);
-					L.state = static_cast<float*>(allocate(sizeof(float) * state_floats(m)));
-					widest_mid = std::max(widest_mid, values);
+					L = LayerState(layers[static_cast<size_t>(L.desc.weights_of)]);
 				}
+			}
+			for (LayerState& L : layers)
+			{
+				int mid_cols = 0;
+				for (MixerState& M : L.mixers)
+				{
+					build_state(M);
+					const MixerDesc& m = M.desc;
+					mid_cols += m.heads * m.vdim;
+					if (m.kind == MixerKind::LatentAttention)
+					{
+						kv_cols = std::max(kv_cols, M.ukv.n);
+						widest_mid = std::max(widest_mid, m.q_rank);
+					}
+					if (m.kind == MixerKind::StateSpace)
+					{
+						ssm_cols = std::max(ssm_cols, m.heads * m.vdim);
+					}
+					else
+					{
+						q_cols = std::max(q_cols, m.heads * m.dim);
+					}
+				}
+				widest_mid = std::max({ widest_mid, mid_cols, L.desc.ff });
 				proj_cols = std::max(proj_cols, L.in.n);
-				L.out = matrix({ { mix + "o", width, nullptr } }, values);
-				if (L.desc.ff > 0)
-				{
-					const int ff = L.desc.ff;
-					L.norm2 = vector(p + "norm2", width);
-					L.norm2b = vector(p + "norm2b", width);
-					L.gate_up = interleaved(p + "mlp.gate", p + "mlp.up", ff, width);
-					L.down = matrix({ { p + "mlp.down", width, nullptr } }, ff);
-					widest_mid = std::max(widest_mid, ff);
-				}
 			}
 			const auto up4 = [](int n) { return (n + 3) & ~3; };
 			ld_proj = up4(proj_cols);
@@ -261,22 +444,18 @@ namespace litenn_hip
 			ld_kv = (std::max(kv_cols, 8) + 7) & ~7;
 			if (desc.sinusoid_base > 0.0)
 			{
-				std::vector<double> f((static_cast<size_t>(width) + 1) / 2);
-				for (size_t i = 0; i < f.size(); ++i)
-				{
-					f[i] = std::pow(desc.sinusoid_base, -2.0 * static_cast<double>(i) / width) / (2.0 * M_PI);
-				}
-				turns = static_cast<double*>(allocate(sizeof(double) * f.size()));
-				copy_in(turns, f.data(), sizeof(double) * f.size());
+				turns = turns_per_position(desc.sinusoid_base, width);
 			}
 			xt[0] = static_cast<float*>(allocate(sizeof(float) * static_cast<size_t>(width)));
 			xt[1] = static_cast<float*>(allocate(sizeof(float) * static_cast<size_t>(width)));
 			row_mid = static_cast<float*>(allocate(sizeof(float) * static_cast<size_t>(ld_mid)));
+			row_ssm = static_cast<float*>(allocate(sizeof(float) * static_cast<size_t>(ssm_cols)));
 		}
 
 		static size_t state_floats(const MixerDesc& m)
 		{
-			return static_cast<size_t>(m.heads) * m.dim * gla_state_pitch(m.vdim);
+			return m.kind == MixerKind::StateSpace ? static_cast<size_t>(m.heads) * m.state * ssm_state_pitch(m.vdim)
+			                                       : static_cast<size_t>(m.heads) * m.dim * gla_state_pitch(m.vdim);
 		}
 
 		static void copy_in(void* dst, const void* src, size_t bytes)
@@ -296,8 +475,8 @@ namespace litenn_hip
 				throw std::runtime_error(std::string("the configuration has no place for tensor '") + t.name + "'");
 			}
 			Slot& s = it->second;
-			const bool shaped = s.matrix ? t.rank == 2 && t.shape[0] == s.rows && t.shape[1] == s.cols
-			                             : t.rank == 1 && t.shape[0] == s.rows;
+			const bool shaped = s.cols ? t.rank == 2 && t.shape[0] == s.rows && t.shape[1] == s.cols
+			                           : t.rank == 1 && t.shape[0] == s.rows;
 			if (!shaped || !t.data)
 			{
 				throw std::runtime_error(std::string("tensor '") + t.name + "' has another shape than the configuration gives it");
@@ -316,19 +495,21 @@ namespace litenn_hip
 			}
 			else
 			{
-				std::vector<float> v(s.rows);
-				for (size_t i = 0; i < s.rows; ++i)
+				const size_t cols = std::max<size_t>(s.cols, 1);
+				std::vector<float> v(s.rows * cols);
+				for (size_t i = 0; i < v.size(); ++i)
 				{
+					float& to = v[i % cols * s.rows + i / cols];
 					if (t.dtype == LITENN_BF16)
 					{
 						uint16_t b;
 						memcpy(&b, static_cast<const uint8_t*>(t.data) + 2 * i, 2);
 						const uint32_t w = static_cast<uint32_t>(b) << 16;
-						memcpy(&v[i], &w, 4);
+						memcpy(&to, &w, 4);
 					}
 					else if (t.dtype == LITENN_F32)
 					{
-						memcpy(&v[i], static_cast<const uint8_t*>(t.data) + 4 * i, 4);
+						memcpy(&to, static_cast<const uint8_t*>(t.data) + 4 * i, 4);
 					}
 					else
 					{
@@ -366,24 +547,38 @@ namespace litenn_hip
 			LITENN_HIP_TRY(action, hipStreamSynchronize(stream));
 			free_scratch();
 			const int n = static_cast<int>(rows);
-			size_t absorbed_floats = 0, partial_floats = 0, decay_floats = 0, chunk_floats = 0, kv_rows = 0;
+			size_t absorbed_floats = 0, partial_floats = 0, decay_floats = 0, chunk_floats = 0, kv_rows = 0, xbc_floats = 0;
 			for (const LayerState& L : layers)
 			{
-				const MixerDesc& m = L.desc.mixer;
-				if (m.kind == MixerKind::LatentAttention)
+				for (const MixerState& M : L.mixers)
 				{
-					for (int r = 1; r < kExpandMin; ++r)
+					const MixerDesc& m = M.desc;
+					switch (m.kind)
 					{
-						absorbed_floats = std::max(absorbed_floats, static_cast<size_t>(r) * m.heads * L.cache.pitch);
-						partial_floats = std::max(partial_floats, latent_step_partial_floats(m.heads, r, L.cache.pitch,
-						                                                                     latent_step_splits(m.heads, r, m.window)));
+					case MixerKind::LatentAttention:
+						for (int r = 1; r < kExpandMin; ++r)
+						{
+							absorbed_floats = std::max(absorbed_floats, static_cast<size_t>(r) * m.heads * M.cache.pitch);
+							partial_floats = std::max(partial_floats, latent_step_partial_floats(m.heads, r, M.cache.pitch,
+							                                                                     latent_step_splits(m.heads, r, m.window)));
+						}
+						kv_rows = std::max(kv_rows, std::min<size_t>(static_cast<size_t>(context_length), static_cast<size_t>(m.window) - 1 + rows));
+						break;
+					case MixerKind::GatedLinearAttention:
+						decay_floats = std::max(decay_floats, rows * m.heads * m.dim);
+						chunk_floats = std::max(chunk_floats, gla_chunk_floats(n, m.heads, m.dim, m.vdim));
+						break;
+					case MixerKind::GroupedAttention:
+						partial_floats = std::max(partial_floats, grouped_step_partial_floats(m.heads, m.vdim, M.splits));
+						break;
+					case MixerKind::StateSpace: {
+						const Ssm shape = ssm_args(M);
+						decay_floats = std::max(decay_floats, 2 * rows * m.heads);
+						xbc_floats = std::max(xbc_floats, rows * shape.ldx());
+						chunk_floats = std::max(chunk_floats, ssm_chunk_floats(n, shape));
+						break;
 					}
-					kv_rows = std::max(kv_rows, std::min<size_t>(static_cast<size_t>(context_length), static_cast<size_t>(m.window) - 1 + rows));
-				}
-				else
-				{
-					decay_floats = std::max(decay_floats, rows * m.heads * m.dim);
-					chunk_floats = std::max(chunk_floats, gla_chunk_floats(n, m.heads, m.dim, m.vdim));
+					}
 				}
 			}
 			const size_t operand = f32 ? 4 : 2;
@@ -396,6 +591,7 @@ namespace litenn_hip
 				{ reinterpret_cast<void**>(&partial), 4 * partial_floats },
 				{ reinterpret_cast<void**>(&log_decay), 4 * decay_floats },
 				{ reinterpret_cast<void**>(&chunk_states), 4 * chunk_floats },
+				{ reinterpret_cast<void**>(&xbc), 4 * xbc_floats },
 				{ &h, operand * rows * ld_h },
 				{ &mid, operand * rows * ld_mid },
 				{ &kv, operand * kv_rows * ld_kv },
@@ -412,9 +608,12 @@ namespace litenn_hip
 		{
 			for (const LayerState& L : layers)
 			{
-				if (L.state)
+				for (const MixerState& M : L.mixers)
 				{
-					launch_zero_ints(reinterpret_cast<int*>(L.state), state_floats(L.desc.mixer), stream);
+					if (M.state)
+					{
+						launch_zero_ints(reinterpret_cast<int*>(M.state), state_floats(M.desc), stream);
+					}
 				}
 			}
 			LITENN_HIP_TRY(action, hipGetLastError());
@@ -436,40 +635,167 @@ namespace litenn_hip
 		}
 
 		// ---- single row ---------------------------------------------------------------------
-		LatentShape latent_shape(const LayerState& L) const
+		LatentShape latent_shape(const MixerState& M) const
 		{
-			const MixerDesc& m = L.desc.mixer;
+			const MixerDesc& m = M.desc;
 			LatentShape s;
 			s.heads = m.heads;
 			s.dim = m.dim;
 			s.vdim = m.vdim;
 			s.window = m.window;
 			s.scale = m.scale;
-			s.sink = L.sink;
+			s.sink = M.sink;
 			return s;
 		}
 
-		Gla gla_args(const LayerState& L) const
+		Gla gla_args(const MixerState& M) const
 		{
-			const MixerDesc& m = L.desc.mixer;
+			const MixerDesc& m = M.desc;
 			Gla g;
 			g.shape.heads = m.heads;
 			g.shape.dim = m.dim;
 			g.shape.vdim = m.vdim;
 			g.shape.q_scale = static_cast<float>(1.0 / std::sqrt(static_cast<double>(m.dim)));
 			g.shape.inv_tau = static_cast<float>(1.0 / static_cast<double>(m.tau));
-			g.q = proj + L.at_q;
-			g.k = proj + L.at_k;
-			g.v = proj + L.at_v;
-			g.gate = proj + L.at_gate;
-			g.a1 = proj + L.at_low;
+			g.q = proj + M.at_q;
+			g.k = proj + M.at_k;
+			g.v = proj + M.at_v;
+			g.gate = proj + M.at_gate;
+			g.a1 = proj + M.at_low;
 			g.ld = ld_proj;
-			g.a2 = L.a2;
-			g.a2_bias = L.a2_bias;
-			g.state = L.state;
-			g.norm_w = L.head_norm;
+			g.a2 = M.a2;
+			g.a2_bias = M.a2_bias;
+			g.state = M.state;
+			g.norm_w = M.head_norm;
 			g.eps = desc.eps;
 			return g;
+		}
+
+		GroupedAttn grouped_args(const MixerState& M) const
+		{
+			const MixerDesc& m = M.desc;
+			GroupedAttn a;
+			a.heads = m.heads;
+			a.window = m.window;
+			a.scale = m.scale;
+			a.rot.dims = m.rot_dims;
+			a.rot.turns = M.turns;
+			a.q_norm = M.q_norm;
+			a.k_norm = M.k_norm;
+			a.eps = desc.eps;
+			a.cache = M.heads;
+			a.q = proj + M.at_q;
+			a.k = proj + M.at_k;
+			a.v = proj + M.at_v;
+			a.ld = ld_proj;
+			a.q_out = q;
+			a.ldq = ld_q;
+			a.partial = partial;
+			a.splits = M.splits;
+			return a;
+		}
+
+		Ssm ssm_args(const MixerState& M) const
+		{
+			const MixerDesc& m = M.desc;
+			Ssm a;
+			a.heads = m.heads;
+			a.vdim = m.vdim;
+			a.state = m.state;
+			a.groups = m.groups;
+			a.taps = m.taps;
+			a.conv_w = M.conv_w;
+			a.conv_b = M.conv_b;
+			a.dt_bias = M.dt_bias;
+			a.a_log = M.a_log;
+			a.d = M.skip;
+			a.in = proj + M.at_in;
+			a.ld = ld_proj;
+			a.states = M.state;
+			a.ring = M.ring;
+			a.y = row_ssm;
+			a.xbc = xbc;
+			a.steps = log_decay;
+			a.chunk_states = chunk_states;
+			return a;
+		}
+
+		// the recurrence's output on its way to the output projection
+		GatedNorm gated_norm_args(const MixerState& M) const
+		{
+			GatedNorm g;
+			g.width = M.desc.heads * M.desc.vdim;
+			g.parts = M.desc.norm_groups;
+			g.norm_w = M.group_norm;
+			g.eps = desc.eps;
+			g.scale = M.desc.weight;
+			return g;
+		}
+
+		// grouped attention and state space, alone or side by side, on one token: from proj to row_mid
+		void mix_token(const LayerState& L, const Position& pos)
+		{
+			GroupedAttn attn;
+			Ssm ssm;
+			GatedNorm norm;
+			const MixerState *a = nullptr, *b = nullptr;
+			for (const MixerState& M : L.mixers)
+			{
+				if (M.desc.kind == MixerKind::GroupedAttention)
+				{
+					a = &M;
+					attn = grouped_args(M);
+					attn.pos = pos;
+				}
+				else
+				{
+					b = &M;
+					ssm = ssm_args(M);
+					ssm.pos = pos;
+					norm = gated_norm_args(M);
+					norm.y = row_ssm;
+					norm.z = ssm.in;
+					norm.out = row_mid + M.at_mid;
+				}
+			}
+			launch_mixer_step(a ? &attn : nullptr, b ? &ssm : nullptr, stream);
+			launch_mixer_finish(a ? &attn : nullptr, a ? a->desc.weight : 1.0f, a ? row_mid + a->at_mid : nullptr, b ? &norm : nullptr, stream);
+		}
+
+		// the same for a prompt's rows: from proj to mid
+		void mix_rows(const LayerState& L, int rows, int past, const Position& pos)
+		{
+			for (const MixerState& M : L.mixers)
+			{
+				void* out = static_cast<uint8_t*>(mid) + (f32 ? 4 : 2) * static_cast<size_t>(M.at_mid);
+				if (M.desc.kind == MixerKind::GroupedAttention)
+				{
+					GroupedAttn a = grouped_args(M);
+					a.rows = rows;
+					a.pos = pos;
+					launch_grouped_append(a, stream);
+					WindowAttn w = grouped_window(a, past);
+					w.out_scale = M.desc.weight;
+					w.out = out;
+					w.ldo = ld_mid;
+					launch_window_attn(w, stream);
+				}
+				else
+				{
+					Ssm a = ssm_args(M);
+					a.rows = rows;
+					a.pos = pos;
+					launch_ssm_rows(a, stream);
+					GatedNorm g = gated_norm_args(M);
+					g.y = a.in;
+					g.ldy = ld_proj;
+					g.out = out;
+					g.ldo = ld_mid;
+					g.rows = rows;
+					g.f32 = f32;
+					launch_gated_norm(g, stream);
+				}
+			}
 		}
 
 		// the token at position counters[0] + offset; logits to `out` unless null
@@ -480,12 +806,13 @@ namespace litenn_hip
 			int at = 0;                // xt[at] is the residual stream, `pending` still to be added
 			const float* pending = nullptr; // norm weight of the sublayer output in y
 			// norm(x + norm(y)) norm_w through `w`
-			const auto enter = [&](const DenseMatrix& w, const float* norm_w, float* dst, bool glu, const ClampedGlu& act) {
+			const auto enter = [&](const DenseMatrix& w, const float* norm_w, float* dst, bool glu, const ClampedGlu& act, float softcap = 0.0f) {
 				DenseRow r;
 				r.w = w;
 				r.x = xt[at];
 				r.y = dst;
-				r.prologue = kRowAddNorm;
+				r.softcap = softcap;
+				r.prologue = pending || norm_w ? kRowAddNorm : kRowPlain;
 				r.norm_w = norm_w;
 				r.eps = desc.eps;
 				r.glu = glu;
@@ -510,30 +837,31 @@ namespace litenn_hip
 			};
 			for (LayerState& L : layers)
 			{
-				const MixerDesc& m = L.desc.mixer;
+				const MixerState& M = L.mixers[0];
+				const MixerDesc& m = M.desc;
 				enter(L.in, L.norm1, proj, false, ClampedGlu{});
 				if (m.kind == MixerKind::LatentAttention)
 				{
 					DenseRow r;
-					r.w = L.uq;
-					r.x = proj + L.at_q;
+					r.w = M.uq;
+					r.x = proj + M.at_q;
 					r.y = q;
 					r.prologue = kRowAddNorm;
-					r.norm_w = L.q_norm;
+					r.norm_w = M.q_norm;
 					r.eps = desc.eps;
 					launch_dense_row(r, stream);
 					LatentStep a;
-					a.shape = latent_shape(L);
-					a.cache = L.cache;
-					a.uk = L.uk;
-					a.uv = L.uv;
+					a.shape = latent_shape(M);
+					a.cache = M.cache;
+					a.uk = M.uk;
+					a.uv = M.uv;
 					a.q = q;
 					a.ldq = ld_q;
-					a.latent = proj + L.at_latent;
+					a.latent = proj + M.at_latent;
 					a.ldl = ld_proj;
-					a.latent_w = L.latent_norm;
+					a.latent_w = M.latent_norm;
 					a.eps = desc.eps;
-					a.gate = proj + L.at_gate;
+					a.gate = proj + M.at_gate;
 					a.ldg = ld_proj;
 					a.out = row_mid;
 					a.ldo = ld_mid;
@@ -542,13 +870,13 @@ namespace litenn_hip
 					a.pos = pos;
 					a.absorbed = absorbed;
 					a.partial = partial;
-					a.splits = L.splits;
+					a.splits = M.splits;
 					launch_latent_step(a, stream);
 					leave(L.out, row_mid, L.norm1b);
 				}
-				else
+				else if (m.kind == MixerKind::GatedLinearAttention)
 				{
-					Gla g = gla_args(L);
+					Gla g = gla_args(M);
 					g.o = row_mid;
 					launch_gla_step(g, stream);
 					DenseRow r;
@@ -556,12 +884,17 @@ namespace litenn_hip
 					r.x = row_mid;
 					r.y = y;
 					r.prologue = kRowHeadGate;
-					r.norm_w = L.head_norm;
-					r.gate = proj + L.at_gate;
+					r.norm_w = M.head_norm;
+					r.gate = proj + M.at_gate;
 					r.vdim = m.vdim;
 					r.eps = desc.eps;
 					launch_dense_row(r, stream);
 					pending = L.norm1b;
+				}
+				else
+				{
+					mix_token(L, pos);
+					leave(L.out, row_mid, L.norm1b);
 				}
 				if (L.desc.ff > 0)
 				{
@@ -571,7 +904,7 @@ namespace litenn_hip
 			}
 			if (out)
 			{
-				enter(embed, final_norm, out, false, ClampedGlu{});
+				enter(head, final_norm, out, false, ClampedGlu{}, desc.logit_softcap);
 			}
 		}
 
@@ -639,16 +972,16 @@ namespace litenn_hip
 			};
 			for (LayerState& L : layers)
 			{
-				const MixerDesc& m = L.desc.mixer;
+				const MixerState& M = L.mixers[0];
 				enter(L.norm1, 0, rows);
 				product(L.in, h, ld_h, rows, proj, ld_proj, kOutF32);
-				if (m.kind == MixerKind::LatentAttention)
+				if (M.desc.kind == MixerKind::LatentAttention)
 				{
-					attend(L, rows, past, pos);
+					attend(M, rows, past, pos);
 				}
-				else
+				else if (M.desc.kind == MixerKind::GatedLinearAttention)
 				{
-					Gla g = gla_args(L);
+					Gla g = gla_args(M);
 					g.rows = rows;
 					g.out = mid;
 					g.ldo = ld_mid;
@@ -656,6 +989,10 @@ namespace litenn_hip
 					g.log_decay = log_decay;
 					g.chunk_states = chunk_states;
 					launch_gla_rows(g, stream);
+				}
+				else
+				{
+					mix_rows(L, rows, past, pos);
 				}
 				leave(L.out, L.norm1b);
 				if (L.desc.ff > 0)
@@ -667,23 +1004,24 @@ namespace litenn_hip
 			}
 			enter(final_norm, rows - logit_rows, logit_rows);
 			DenseRows d;
-			d.w = embed;
+			d.w = head;
 			d.a = h;
 			d.lda = ld_h;
 			d.m = logit_rows;
 			d.c = logits;
 			d.ldc = vocab;
 			d.f32 = f32;
+			d.softcap = desc.logit_softcap;
 			launch_dense_rows(d, stream);
 		}
 
-		void attend(LayerState& L, int rows, int past, const Position& pos)
+		void attend(const MixerState& M, int rows, int past, const Position& pos)
 		{
-			const MixerDesc& m = L.desc.mixer;
+			const MixerDesc& m = M.desc;
 			AddNorm n; // queries' latent
-			n.x = proj + L.at_q;
+			n.x = proj + M.at_q;
 			n.ldx = ld_proj;
-			n.norm_w = L.q_norm;
+			n.norm_w = M.q_norm;
 			n.out = mid;
 			n.ldo = ld_mid;
 			n.rows = rows;
@@ -691,18 +1029,18 @@ namespace litenn_hip
 			n.eps = desc.eps;
 			n.f32 = f32;
 			launch_add_norm(n, stream);
-			product(L.uq, mid, ld_mid, rows, q, ld_q, kOutF32);
-			launch_latent_append(proj + L.at_latent, ld_proj, L.latent_norm, desc.eps, rows, pos, L.cache, stream);
+			product(M.uq, mid, ld_mid, rows, q, ld_q, kOutF32);
+			launch_latent_append(proj + M.at_latent, ld_proj, M.latent_norm, desc.eps, rows, pos, M.cache, stream);
 			if (rows < kExpandMin)
 			{
 				LatentStep a;
-				a.shape = latent_shape(L);
-				a.cache = L.cache;
-				a.uk = L.uk;
-				a.uv = L.uv;
+				a.shape = latent_shape(M);
+				a.cache = M.cache;
+				a.uk = M.uk;
+				a.uv = M.uv;
 				a.q = q;
 				a.ldq = ld_q;
-				a.gate = proj + L.at_gate;
+				a.gate = proj + M.at_gate;
 				a.ldg = ld_proj;
 				a.out = mid;
 				a.ldo = ld_mid;
@@ -718,11 +1056,11 @@ namespace litenn_hip
 			const int base = std::max(0, past - m.window + 1);
 			const int keys = past + rows - base;
 			DenseRows d;
-			d.w = L.ukv;
-			d.a = L.cache.rows;
-			d.lda = L.cache.pitch;
-			d.a_first = base % L.cache.ring;
-			d.a_ring = L.cache.ring;
+			d.w = M.ukv;
+			d.a = M.cache.rows;
+			d.lda = M.cache.pitch;
+			d.a_first = base % M.cache.ring;
+			d.a_ring = M.cache.ring;
 			d.m = keys;
 			d.c = kv;
 			d.ldc = ld_kv;
@@ -730,17 +1068,19 @@ namespace litenn_hip
 			d.f32 = f32;
 			launch_dense_rows(d, stream);
 			WindowAttn w;
-			w.shape = latent_shape(L);
+			w.shape = latent_shape(M);
 			w.q = q;
 			w.ldq = ld_q;
 			w.kv = kv;
 			w.ldkv = ld_kv;
-			w.v_first = L.v_first;
+			w.v_first = M.v_first;
+			w.k_head = static_cast<size_t>(m.dim);
+			w.v_head = static_cast<size_t>(m.vdim);
 			w.keys = keys;
 			w.key_base = base;
 			w.rows = rows;
 			w.q_base = past;
-			w.gate = proj + L.at_gate;
+			w.gate = proj + M.at_gate;
 			w.ldg = ld_proj;
 			w.out = mid;
 			w.ldo = ld_mid;

@@ -4,7 +4,7 @@
 // (recurrent step, and a chunked form whose contractions run on the Float32 matrix instructions).
 // Norms, positions, scores, softmax and everything inside a recurrence are Float32.  The reference
 // has no counterpart of these layers.
-#include "layers.hpp"
+#include "layer_device.hpp"
 
 #include <algorithm>
 #include <cmath>
@@ -13,33 +13,6 @@ namespace litenn_hip
 {
 	namespace
 	{
-		typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
-		typedef float floatx4 __attribute__((ext_vector_type(4)));
-		typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
-		typedef floatx4 floatx4_a4 __attribute__((aligned(4))); // global loads and stores take any 4-byte address
-
-		constexpr float kLog2e = 1.44269504088896340736f;
-
-		__device__ __forceinline__ float exp2_f32(float x) { return __builtin_amdgcn_exp2f(x); }
-
-		__device__ __forceinline__ int row_position(const Position& p, int row)
-		{
-			return (p.dev ? *p.dev : 0) + p.add + row;
-		}
-
-		// sum over a workgroup of 256
-		__device__ __forceinline__ float block_sum256(float v, float* red)
-		{
-			v = wave_sum(v);
-			__syncthreads();
-			if ((threadIdx.x & 63) == 0)
-			{
-				red[threadIdx.x >> 6] = v;
-			}
-			__syncthreads();
-			return (red[0] + red[1]) + (red[2] + red[3]);
-		}
-
 		// ---------------- embedding ----------------------------------------------------------
 		__global__ __launch_bounds__(256) void embed_rows_kernel(DenseMatrix table, const int32_t* __restrict__ ids,
 		                                                         const double* __restrict__ turns, Position pos,
@@ -107,7 +80,7 @@ namespace litenn_hip
 				kept[e] = i < a.width ? x[i] : 0.0f;
 				added[e] = sub && i < a.width ? summed(i) : 0.0f;
 				sub_w[e] = sub && i < a.width ? a.sub_w[i] : 0.0f;
-				norm_w[e] = i < a.width ? a.norm_w[i] : 0.0f;
+				norm_w[e] = i < a.width ? (a.norm_w ? a.norm_w[i] : 1.0f) : 0.0f;
 			}
 			if (sub)
 			{
@@ -137,7 +110,7 @@ namespace litenn_hip
 				const float v = value(i);
 				ss = fmaf(v, v, ss);
 			}
-			const float scale = 1.0f / sqrtf(block_sum256(ss, red) / static_cast<float>(a.width) + a.eps);
+			const float scale = a.norm_w ? 1.0f / sqrtf(block_sum256(ss, red) / static_cast<float>(a.width) + a.eps) : 1.0f;
 			float* x_out = a.x_out ? a.x_out + static_cast<size_t>(row) * a.ldx : nullptr;
 			T* out = static_cast<T*>(a.out) + static_cast<size_t>(row) * a.ldo;
 			const auto put = [&](int i, float v, float w) {
@@ -158,7 +131,7 @@ namespace litenn_hip
 			}
 			for (int i = threadIdx.x + 256 * kKept; i < a.width; i += 256)
 			{
-				put(i, value(i), a.norm_w[i]);
+				put(i, value(i), a.norm_w ? a.norm_w[i] : 1.0f);
 			}
 		}
 
@@ -571,6 +544,13 @@ namespace litenn_hip
 		}
 
 		// ---------------- windowed attention over expanded keys and values -----------------------
+		// the row of the buffer that holds key row r
+		__device__ __forceinline__ int window_row(const WindowAttn& a, int r)
+		{
+			r += a.kv_first;
+			return a.kv_ring > 0 && r >= a.kv_ring ? r - a.kv_ring : r;
+		}
+
 		// One wavefront per (query row, head), any head size up to 1024; Float32 arithmetic.
 		constexpr int kRowAttnMaxDim = 1024;
 
@@ -581,6 +561,7 @@ namespace litenn_hip
 			__shared__ float ws[64];
 			const int row = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
 			const int dim = a.shape.dim, vdim = a.shape.vdim;
+			const size_t k_at = h / a.shape.share * a.k_head, v_at = a.v_first + h / a.shape.share * a.v_head;
 			for (int d = lane; d < dim; d += 64)
 			{
 				qs[d] = a.q[static_cast<size_t>(row) * a.ldq + h * dim + d];
@@ -603,7 +584,7 @@ namespace litenn_hip
 				float score = -INFINITY;
 				if (key <= last)
 				{
-					const T* k = kv + static_cast<size_t>(key - a.key_base) * a.ldkv + h * dim;
+					const T* k = kv + static_cast<size_t>(window_row(a, key - a.key_base)) * a.ldkv + k_at;
 					float acc = 0.0f;
 					for (int d = 0; d < dim; ++d)
 					{
@@ -627,10 +608,10 @@ namespace litenn_hip
 					if (e < vdim)
 					{
 						float t = o[c] * corr;
-						const T* v = kv + static_cast<size_t>(base - a.key_base) * a.ldkv + a.v_first + h * vdim + e;
+						const T* v = kv + v_at + e;
 						for (int i = 0; i < count; ++i)
 						{
-							t = fmaf(ws[i], operand_load(v + static_cast<size_t>(i) * a.ldkv), t);
+							t = fmaf(ws[i], operand_load(v + static_cast<size_t>(window_row(a, base - a.key_base + i)) * a.ldkv), t);
 						}
 						o[c] = t;
 					}
@@ -650,7 +631,7 @@ namespace litenn_hip
 				const int e = c * 64 + lane;
 				if (e < vdim)
 				{
-					float v = o[c] * weight / total;
+					float v = o[c] * weight / total * a.out_scale;
 					if (a.gate)
 					{
 						v *= sigmoid_f32(a.gate[static_cast<size_t>(row) * a.ldg + h * vdim + e]);
@@ -687,7 +668,8 @@ namespace litenn_hip
 			// key rows (relative to key_base) any query of the tile sees
 			const int lo = max(0, a.q_base + q_first - a.shape.window + 1 - a.key_base);
 			const int hi = min(a.keys, a.q_base + min(q_first + kWinQ, a.rows) - a.key_base);
-			const uint16_t* const kv = static_cast<const uint16_t*>(a.kv);
+			const uint16_t* const keys = static_cast<const uint16_t*>(a.kv) + h / a.shape.share * a.k_head;
+			const uint16_t* const values = static_cast<const uint16_t*>(a.kv) + a.v_first + h / a.shape.share * a.v_head;
 			const float scale2 = a.shape.scale * kLog2e; // scores in units of log 2
 
 			bf16x8 q_frag[DK / 32];
@@ -700,8 +682,8 @@ namespace litenn_hip
 #pragma unroll
 					for (int e = 0; e < 4; ++e)
 					{
-						const int d = 32 * st + 8 * g + 2 * e; // dim is a multiple of 8
-						w[e] = d < dim ? pack_bf16(q[d], q[d + 1]) : 0u;
+						const int d = 32 * st + 8 * g + 2 * e;
+						w[e] = d < dim ? pack_bf16(q[d], d + 1 < dim ? q[d + 1] : 0.0f) : 0u;
 					}
 					q_frag[st] = __builtin_bit_cast(bf16x8, u32x4{ w[0], w[1], w[2], w[3] });
 				}
@@ -722,10 +704,10 @@ namespace litenn_hip
 				for (int i = 0; i < KN; ++i)
 				{
 					const int c = tid + 256 * i, key = min(base + c / KP, hi - 1), d = (c % KP) * 8;
-					kr[i] = d < dim ? *reinterpret_cast<const u32x4*>(kv + static_cast<size_t>(key) * a.ldkv + h * dim + d)
+					kr[i] = d < dim ? *reinterpret_cast<const u32x4*>(keys + static_cast<size_t>(window_row(a, key)) * a.ldkv + d)
 					                : u32x4{ 0u, 0u, 0u, 0u };
 				}
-				const uint16_t* v = kv + static_cast<size_t>(min(base + v_key, hi - 1)) * a.ldkv + a.v_first + h * vdim;
+				const uint16_t* v = values + static_cast<size_t>(window_row(a, min(base + v_key, hi - 1))) * a.ldkv;
 #pragma unroll
 				for (int i = 0; i < VN; ++i)
 				{
@@ -844,13 +826,13 @@ namespace litenn_hip
 				weight = exp2_f32(run_m - all_m);
 				total = run_l * weight + exp2_f32(sink - all_m);
 			}
-			const float inv = weight / total;
+			const float inv = weight / total * a.out_scale;
 			uint16_t* out = static_cast<uint16_t*>(a.out) + static_cast<size_t>(my_q) * a.ldo + static_cast<size_t>(h) * vdim;
 			const float* gate = a.gate ? a.gate + static_cast<size_t>(my_q) * a.ldg + static_cast<size_t>(h) * vdim : nullptr;
 #pragma unroll
 			for (int b = 0; b < DV / 16; ++b)
 			{
-				const int e = 16 * b + 4 * g; // vdim is a multiple of 8
+				const int e = 16 * b + 4 * g;
 				if (e < vdim)
 				{
 					floatx4 v = o[b] * inv;
@@ -859,10 +841,24 @@ namespace litenn_hip
 #pragma unroll
 						for (int r = 0; r < 4; ++r)
 						{
-							v[r] *= sigmoid_f32(gate[e + r]);
+							v[r] *= e + r < vdim ? sigmoid_f32(gate[e + r]) : 0.0f;
 						}
 					}
-					*reinterpret_cast<uint2*>(out + e) = make_uint2(pack_bf16(v.x, v.y), pack_bf16(v.z, v.w));
+					if ((vdim & 3) == 0 && (reinterpret_cast<size_t>(a.out) & 7) == 0)
+					{
+						*reinterpret_cast<uint2*>(out + e) = make_uint2(pack_bf16(v.x, v.y), pack_bf16(v.z, v.w));
+					}
+					else
+					{
+#pragma unroll
+						for (int r = 0; r < 4; ++r)
+						{
+							if (e + r < vdim)
+							{
+								out[e + r] = to_bf16(v[r]);
+							}
+						}
+					}
 				}
 			}
 		}
@@ -1017,25 +1013,6 @@ namespace litenn_hip
 		{
 			return a.chunk_states +
 			       static_cast<size_t>(chunks) * a.shape.heads * a.shape.dim * gla_state_pitch(a.shape.vdim);
-		}
-
-		// four columns from column e of a row of `n`, zero beyond
-		__device__ __forceinline__ floatx4 load_columns(const float* row, int e, int n)
-		{
-			floatx4 v = { 0.0f, 0.0f, 0.0f, 0.0f };
-			if (e + 3 < n)
-			{
-				v = *reinterpret_cast<const floatx4_a4*>(row + e);
-			}
-			else
-			{
-#pragma unroll
-				for (int i = 0; i < 3; ++i)
-				{
-					v[i] = e + i < n ? row[e + i] : 0.0f;
-				}
-			}
-			return v;
 		}
 
 		// NC: groups of 64 value columns, each the work of four wavefronts (which share out the channels or the
@@ -1640,8 +1617,8 @@ namespace litenn_hip
 			return;
 		}
 		// whole 16-byte pieces of a head's keys and values
-		const bool pieces = a.shape.dim % 8 == 0 && a.shape.vdim % 8 == 0 && a.ldkv % 8 == 0 && a.v_first % 8 == 0 &&
-		                    a.ldo % 4 == 0 && a.shape.dim <= 256 && a.shape.vdim <= 256;
+		const bool pieces = a.k_head % 8 == 0 && a.v_head % 8 == 0 && a.ldkv % 8 == 0 && a.v_first % 8 == 0 &&
+		                    (a.ldo % 4 == 0 || a.shape.vdim % 4 != 0) && a.shape.dim <= 256 && a.shape.vdim <= 256;
 		if (!pieces)
 		{
 			window_attn_row_kernel<uint16_t><<<rows, dim3(64), 0, s>>>(a);

@@ -13,6 +13,23 @@ namespace litenn_hip
 		constexpr int kMaxSize = 1 << 24;
 		constexpr int kDefaultContext = 32768;
 
+		// the layer's feed-forward, if it has one; its constants are the design's
+		const Json* dense_feed_forward(const Json& layer, LayerDesc& L)
+		{
+			const Json* mlp = layer.find("mlp");
+			if (!mlp || mlp->is_null())
+			{
+				return nullptr;
+			}
+			const std::string& kind = mlp->string("kind");
+			if (kind != "dense")
+			{
+				throw std::runtime_error("configuration: unknown feed-forward kind '" + kind + "'");
+			}
+			L.ff = mlp->integer("ff", 1, kMaxSize);
+			return mlp;
+		}
+
 		// ---- Kulurax -------------------------------------------------------------------------
 		// Sinusoidal positions; layers of latent attention or gated linear attention, each optionally
 		// followed by a clamped gated feed-forward; norms on both sides of every sublayer; tied head.
@@ -34,7 +51,7 @@ namespace litenn_hip
 				const Json& mix = in.at("mixer");
 				const std::string& type = in.string("type");
 				LayerDesc L;
-				MixerDesc& m = L.mixer;
+				MixerDesc m;
 				m.heads = mix.integer("heads", 1, 32768);
 				if (type == "latent_attention")
 				{
@@ -68,15 +85,9 @@ namespace litenn_hip
 				{
 					throw std::runtime_error("configuration: unknown layer type '" + type + "'");
 				}
-				const Json* mlp = in.find("mlp");
-				if (mlp && !mlp->is_null())
+				L.mixers.push_back(m);
+				if (const Json* mlp = dense_feed_forward(in, L))
 				{
-					const std::string& kind = mlp->string("kind");
-					if (kind != "dense")
-					{
-						throw std::runtime_error("configuration: unknown feed-forward kind '" + kind + "'");
-					}
-					L.ff = mlp->integer("ff", 1, kMaxSize);
 					L.act.limit = static_cast<float>(mlp->real("limit"));
 					L.act.alpha = 1.702f;
 					L.act.shift = 1.0f;
@@ -86,8 +97,131 @@ namespace litenn_hip
 			return d;
 		}
 
+		// ---- Degedra -------------------------------------------------------------------------
+		// Layers of windowed attention and a state-space recurrence side by side, each optionally followed by a
+		// gated feed-forward; only what a sublayer returns is normalised; soft-capped logits.  A layer may use
+		// an earlier or later layer's weights.
+		MixerDesc degedra_attention(const Json& c)
+		{
+			MixerDesc m;
+			m.kind = MixerKind::GroupedAttention;
+			m.name = "left.";
+			m.heads = c.integer("heads", 1, 32768);
+			m.kv_heads = c.integer("kv_heads", 1, m.heads);
+			m.dim = c.integer("dim", 1, grouped_max_dim());
+			m.vdim = c.integer("vdim", 1, grouped_max_dim());
+			m.scale = static_cast<float>(c.real("scale"));
+			const Json* mask = c.find("mask");
+			m.window = mask && !mask->is_null() ? mask->integer("size", 1, 1 << 30) : 0;
+			const Json* rot = c.find("rot");
+			if (rot && !rot->is_null())
+			{
+				m.rot_dims = rot->integer("dims", 0, m.dim);
+				m.rot_base = rot->real("base");
+			}
+			m.projection_norm = true;
+			m.values_are_keys = true;
+			if (m.heads % m.kv_heads != 0)
+			{
+				throw std::runtime_error("configuration: 'heads' is not a multiple of 'kv_heads'");
+			}
+			if (m.vdim != m.dim)
+			{
+				throw std::runtime_error("configuration: the values are the keys, but 'vdim' is not 'dim'");
+			}
+			if (m.rot_dims % 2 != 0 || (m.rot_dims > 0 && !(m.rot_base > 0.0)))
+			{
+				throw std::runtime_error("configuration: the rotation takes an even number of dimensions and a base greater than zero");
+			}
+			return m;
+		}
+
+		MixerDesc degedra_state_space(const Json& c)
+		{
+			MixerDesc m;
+			m.kind = MixerKind::StateSpace;
+			m.name = "right.";
+			m.heads = c.integer("heads", 1, 32768);
+			m.vdim = c.integer("vdim", 1, 32768);
+			m.state = c.integer("state", 1, ssm_max_state());
+			m.groups = c.integer("groups", 1, m.heads);
+			m.norm_groups = c.integer("norm_groups", 1, kMaxSize);
+			m.taps = c.integer("conv", 1, 1024);
+			if (m.heads % m.groups != 0)
+			{
+				throw std::runtime_error("configuration: 'heads' is not a multiple of 'groups'");
+			}
+			if (static_cast<long long>(m.heads) * m.vdim > kMaxSize || m.heads * m.vdim % m.norm_groups != 0)
+			{
+				throw std::runtime_error("configuration: 'norm_groups' does not divide heads times 'vdim'");
+			}
+			return m;
+		}
+
+		LayeredDesc describe_degedra(const Json& c, const ShapeOf&)
+		{
+			LayeredDesc d;
+			d.vocab = c.integer("vocab", 1, kMaxSize);
+			d.width = c.integer("width", 1, kMaxSize);
+			d.eps = static_cast<float>(c.at("norm").real("eps"));
+			d.norms = NormPlacement::Output;
+			d.tied_head = false;
+			const Json* cap = c.find("logit_softcap");
+			if (cap && !cap->is_null())
+			{
+				d.logit_softcap = static_cast<float>(c.real("logit_softcap"));
+				if (!(d.logit_softcap > 0.0f))
+				{
+					throw std::runtime_error("configuration: 'logit_softcap' must be greater than zero");
+				}
+			}
+			const Json& layers = c.at("layers");
+			if (layers.kind != Json::Array || layers.items.empty())
+			{
+				throw std::runtime_error("configuration: 'layers' is not a list of layers");
+			}
+			const int count = static_cast<int>(layers.items.size());
+			for (int i = 0; i < count; ++i)
+			{
+				// the owner of the layer's weights describes the layer
+				int owner = i;
+				for (int hops = 0; const Json* of = layers.items[owner].find("weights_of"); ++hops)
+				{
+					if (of->is_null())
+					{
+						break;
+					}
+					owner = layers.items[owner].integer("weights_of", 0, count - 1);
+					if (hops == count)
+					{
+						throw std::runtime_error("configuration: 'weights_of' leads round in a circle");
+					}
+				}
+				const Json& in = layers.items[owner];
+				const std::string& type = in.string("type");
+				if (type != "parallel" || layers.items[i].string("type") != type)
+				{
+					throw std::runtime_error("configuration: unknown layer type '" + layers.items[i].string("type") + "'");
+				}
+				const Json& mix = in.at("mixer");
+				LayerDesc L;
+				L.weights_of = owner == i ? -1 : owner;
+				L.mixers = { degedra_attention(mix.at("left")), degedra_state_space(mix.at("right")) };
+				L.mixers[0].weight = static_cast<float>(mix.real("left_scale"));
+				L.mixers[1].weight = static_cast<float>(mix.real("right_scale"));
+				if (dense_feed_forward(in, L))
+				{
+					L.act.limit = INFINITY;
+					L.act.alpha = 1.0f;
+				}
+				d.layers.push_back(L);
+			}
+			return d;
+		}
+
 		constexpr Architecture kArchitectures[] = {
 			{ "Kulurax", describe_kulurax },
+			{ "Degedra", describe_degedra },
 		};
 
 		int dtype_of(const std::string& name)
