@@ -749,39 +749,46 @@ def bench_gemv_configs(ln, hiprt, steps=1600, warmup=64):
     return out
 
 
-KULURAX_SHAPES = {
-    # width, ff, heads, kv_rank, q_rank, gla heads; the LLaMA model beside it has the same width, ff, heads of 128
-    # (a quarter of them KV heads), layers and vocabulary
-    "2048": dict(width=2048, ff=5632, heads=16, kv_rank=256, q_rank=768, gla_heads=8, layers=8),
-    "4096": dict(width=4096, ff=14336, heads=32, kv_rank=512, q_rank=1536, gla_heads=16, layers=8),
+# width, ff, layers and heads are every side's; beside the layered decoders stands a LLaMA model of the same width,
+# ff, heads of 128 (a quarter of them KV heads), layers and vocabulary
+LAYERED_SHAPES = {
+    "2048": {"common": dict(width=2048, ff=5632, heads=16, layers=8), "kulurax": dict(kv_rank=256, q_rank=768, gla_heads=8),
+             "degedra": dict(kv_heads=4, ssm_heads=32)},
+    "4096": {"common": dict(width=4096, ff=14336, heads=32, layers=8), "kulurax": dict(kv_rank=512, q_rank=1536, gla_heads=16),
+             "degedra": dict(kv_heads=8, ssm_heads=64)},
 }
 
 
-def bench_kulurax(ln, names, prompts, n_new=128, window=1024, vocab=32000, repeats=3, which=("kulurax", "llama")):
-    """Prefill and decode of a layered decoder (linear and latent attention alternating, bfloat16 weights) beside
-    a LLaMA decoder of the same width, feed-forward, depth and vocabulary in Q8_0, the block format nearest to
-    16 bits.  Random weights; the best of `repeats` runs after one warm-up, model sides in turn."""
+# design -> the model it is measured beside
+LAYERED_SIDES = {"kulurax": "llama", "degedra": "kulurax"}
+
+
+def bench_layered(ln, which, names, prompts, n_new=128, window=1024, vocab=32000, repeats=3):
+    """Prefill and decode of layered decoders (bfloat16 weights) beside each other, and beside a LLaMA decoder of the same
+    width, feed-forward, depth and vocabulary in Q8_0, the block format nearest to 16 bits.  Random weights; the best of
+    `repeats` runs after one warm-up, model sides in turn."""
     from litenn_amd import synth
     from litenn_amd.formats import DT_F16, Q8_0
+    makers = {"kulurax": synth.kulurax_config, "degedra": synth.degedra_config}
     out = []
     for name in names:
-        shape = KULURAX_SHAPES[name]
-        cfg = synth.kulurax_config(vocab=vocab, window=window, **shape)
+        shape = LAYERED_SHAPES[name]
+        common = shape["common"]
         context = max(prompts) + n_new + 8
         t0 = time.perf_counter()
-        sides = {}
-        if "kulurax" in which:
-            sides["kulurax"] = ln.create_model(cfg, synth.kulurax_large_tensors(cfg, 7), context_length=context)
-        if "llama" in which:
-            lcfg = synth.LLaMAConfig(f"llama-{name}-q8_0", shape["layers"], shape["width"], shape["heads"],
-                                     shape["heads"] // 4, shape["ff"], vocab, context, formats={"default": Q8_0})
-            l_model = ln.LLaMA.from_config(lcfg, kv_dtype=DT_F16)
-            for item in synth.llama_tensors(lcfg, 3):
-                l_model.set_tensor(*item)
-            sides["llama"] = l_model
+        sides, cfgs = {}, {}
+        for side in which:
+            if side == "llama":
+                lcfg = synth.LLaMAConfig(f"llama-{name}-q8_0", common["layers"], common["width"], common["heads"],
+                                         common["heads"] // 4, common["ff"], vocab, context, formats={"default": Q8_0})
+                sides[side] = ln.LLaMA.from_config(lcfg, kv_dtype=DT_F16)
+                for item in synth.llama_tensors(lcfg, 3):
+                    sides[side].set_tensor(*item)
+            else:
+                cfgs[side] = makers[side](vocab=vocab, window=window, **common, **shape[side])
+                sides[side] = ln.create_model(cfgs[side], synth.layered_large_tensors(cfgs[side], 7), context_length=context)
         log(f"[bench] models of width {name} resident after {time.perf_counter() - t0:.1f} s")
-        entry = {"width": shape["width"], "ff": shape["ff"], "layers": shape["layers"], "vocab": vocab, "window": window,
-                 "shape": shape, "runs": []}
+        entry = {"vocab": vocab, "window": window, **common, "shape": {s: shape[s] for s in which if s in shape}, "runs": []}
         for n_prompt in prompts:
             prompt = np.random.default_rng(5).integers(0, vocab, n_prompt).astype(np.int32)
             best = {}
@@ -796,9 +803,9 @@ def bench_kulurax(ln, names, prompts, n_new=128, window=1024, vocab=32000, repea
                     b[0], b[1] = min(b[0], pre), min(b[1], dec)
             run = {"prompt": n_prompt, "new_tokens": n_new}
             for side, (pre, dec) in best.items():
-                if side == "kulurax":
-                    w_bytes = synth.kulurax_decode_weight_bytes(cfg)
-                    flops = synth.kulurax_prefill_flops(cfg, n_prompt)
+                if side in cfgs:
+                    w_bytes = synth.layered_decode_weight_bytes(cfgs[side])
+                    flops = synth.layered_prefill_flops(cfgs[side], n_prompt)
                 else:
                     w_bytes = lcfg.matmul_weight_bytes_per_token()
                     per_token = sum(2.0 * s[0] * s[1] for kind, s in lcfg.tensor_shapes().items()
@@ -847,12 +854,15 @@ def main() -> int:
                     help="also measure an empty kernel, a read-only kernel and the GEMV's in-kernel timeline")
     ap.add_argument("--block-timeline", action="store_true",
                     help="print the decoder-block kernel's in-kernel timeline (timeline build of the library) and exit")
-    ap.add_argument("--kulurax", action="store_true",
-                    help="measure the layered decoder (Kulurax) beside a LLaMA model of equal size, print that and exit")
-    ap.add_argument("--kulurax-widths", default="2048,4096", help="model widths of --kulurax")
-    ap.add_argument("--kulurax-prompts", default="128,512,2048", help="prompt lengths of --kulurax")
-    ap.add_argument("--kulurax-new", type=int, default=128, help="generated tokens of --kulurax")
-    ap.add_argument("--kulurax-sides", default="kulurax,llama", help="which of the two models --kulurax runs (profiler runs take one)")
+    for design, beside in LAYERED_SIDES.items():
+        ap.add_argument(f"--{design}", action="store_true",
+                        help=f"measure the layered decoder ({design.capitalize()}) beside a {beside.capitalize()} model of "
+                             "equal size, print that and exit")
+        ap.add_argument(f"--{design}-widths", default="2048,4096", help=f"model widths of --{design}")
+        ap.add_argument(f"--{design}-prompts", default="128,512,2048", help=f"prompt lengths of --{design}")
+        ap.add_argument(f"--{design}-new", type=int, default=128, help=f"generated tokens of --{design}")
+        ap.add_argument(f"--{design}-sides", default=f"{design},{beside}",
+                        help=f"which of kulurax, degedra, llama --{design} runs (profiler runs take one)")
     ap.add_argument("--traffic-probe", action="store_true",
                     help="also launch a known-size streaming kernel (profiler counter calibration)")
     args = ap.parse_args()
@@ -874,11 +884,14 @@ def main() -> int:
         return 1
     log("[bench]", ln.DeviceTraits.Info(ln.HIP(0)))
 
-    if args.kulurax:
-        result = bench_kulurax(ln, args.kulurax_widths.split(","), [int(p) for p in args.kulurax_prompts.split(",")],
-                               n_new=args.kulurax_new, repeats=3 if "," in args.kulurax_sides else 1, which=args.kulurax_sides.split(","))
-        print(json.dumps({"kulurax": result, "dtype": "bf16 weights, f32 residual", "data": "synthetic"}), flush=True)
-        return 0
+    for design in LAYERED_SIDES:
+        if getattr(args, design):
+            sides = getattr(args, f"{design}_sides").split(",")
+            result = bench_layered(ln, sides, getattr(args, f"{design}_widths").split(","),
+                                   [int(p) for p in getattr(args, f"{design}_prompts").split(",")],
+                                   n_new=getattr(args, f"{design}_new"), repeats=3 if len(sides) > 1 else 1)
+            print(json.dumps({design: result, "dtype": "bf16 weights, f32 residual", "data": "synthetic"}), flush=True)
+            return 0
 
     if args.traffic_probe:
         traffic_probe(ln)

@@ -235,11 +235,60 @@ def kulurax_tensor_shapes(cfg: dict, decay_rank: int = 16) -> dict:
     return out
 
 
-def kulurax_large_tensors(cfg: dict, seed) -> dict:
+def degedra_attention(heads: int, kv_heads: int, dim: int, window: int, scale: float | None = None, rot_dims: int | None = None,
+                      rot_base: float = 10000.0) -> dict:
+    return {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5 if scale is None else scale,
+            "mask": {"size": window}, "rot": {"dims": dim if rot_dims is None else rot_dims, "base": rot_base}}
+
+
+def degedra_state_space(heads: int, vdim: int, state: int, groups: int = 1, norm_groups: int = 1, conv: int = 4) -> dict:
+    return {"heads": heads, "vdim": vdim, "state": state, "groups": groups, "norm_groups": norm_groups, "conv": conv}
+
+
+def degedra_layer(left: dict, right: dict, ff: int | None, left_scale: float = 1.0, right_scale: float = 1.0) -> dict:
+    return {"type": "parallel", "mlp": None if ff is None else {"kind": "dense", "ff": ff},
+            "mixer": {"left": left, "right": right, "left_scale": left_scale, "right_scale": right_scale}}
+
+
+def degedra_config(width: int, ff: int, layers: int, heads: int, kv_heads: int, vocab: int, window: int, dim: int = 128,
+                   ssm_heads: int = 64, ssm_vdim: int = 64, state: int = 128, groups: int = 2) -> dict:
+    """A Degedra decoder of equal layers, every one with a feed-forward."""
+    layer = degedra_layer(degedra_attention(heads, kv_heads, dim, window),
+                          degedra_state_space(ssm_heads, ssm_vdim, state, groups, groups), ff)
+    return {"architecture": "Degedra", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+            "layers": [layer] * layers}
+
+
+def degedra_tensor_shapes(cfg: dict) -> dict:
+    w = cfg["width"]
+    out = {"embed": (cfg["vocab"], w), "head": (cfg["vocab"], w), "final.norm": (w,)}
+    for i, layer in enumerate(cfg["layers"]):
+        if layer.get("weights_of") is not None:
+            continue
+        p, a, r = f"l{i}.", layer["mixer"]["left"], layer["mixer"]["right"]
+        keys, cached, inner = a["heads"] * a["dim"], a["kv_heads"] * a["dim"], r["heads"] * r["vdim"]
+        channels = inner + 2 * r["groups"] * r["state"]
+        left = {"q": (keys, w), "k": (cached, w), "q.norm": (keys,), "k.norm": (cached,), "o": (w, keys)}
+        right = {"in": (inner + channels + r["heads"], w), "conv": (channels, r["conv"]), "conv.b": (channels,),
+                 "dt_bias": (r["heads"],), "A_log": (r["heads"],), "D": (r["heads"],), "norm": (inner,), "o": (w, inner)}
+        out[p + "norm1"] = (w,)
+        out.update({p + "mix.left." + k: s for k, s in left.items()})
+        out.update({p + "mix.right." + k: s for k, s in right.items()})
+        if layer["mlp"]:
+            ff = layer["mlp"]["ff"]
+            out[p + "norm2"] = (w,)
+            out.update({p + "mlp.gate": (ff, w), p + "mlp.up": (ff, w), p + "mlp.down": (w, ff)})
+    return out
+
+
+TENSOR_SHAPES = {"Kulurax": kulurax_tensor_shapes, "Degedra": degedra_tensor_shapes}
+
+
+def layered_large_tensors(cfg: dict, seed) -> dict:
     """bfloat16 bits for a large model: every matrix is a window into one pool of N(0, 1/64) values, so that
     gigabytes of weights take a second to make and little host memory."""
     rng = _rng(seed)
-    shapes = kulurax_tensor_shapes(cfg)
+    shapes = TENSOR_SHAPES[cfg["architecture"]](cfg)
     size = max(int(np.prod(s)) for s in shapes.values()) + 65536
     pool = (rng.standard_normal(size, dtype=np.float32) * np.float32(1.0 / 64.0)).view(np.uint32)
     pool = ((pool + 0x8000) >> 16).astype(np.uint16)
@@ -254,22 +303,29 @@ def kulurax_large_tensors(cfg: dict, seed) -> dict:
     return out
 
 
-def kulurax_decode_weight_bytes(cfg: dict) -> int:
-    """Weight bytes a single-token step reads: every matrix once (the tied table as the head)."""
-    return 2 * sum(int(np.prod(s)) for s in kulurax_tensor_shapes(cfg).values() if len(s) == 2)
+def layered_decode_weight_bytes(cfg: dict) -> int:
+    """Weight bytes a single-token step reads: every matrix once (an embedding table only where it is the head)."""
+    shapes = TENSOR_SHAPES[cfg["architecture"]](cfg)
+    return 2 * sum(int(np.prod(s)) for n, s in shapes.items() if len(s) == 2 and not (n == "embed" and "head" in shapes))
 
 
-def kulurax_prefill_flops(cfg: dict, rows: int) -> float:
+def window_pairs(rows: int, window: int) -> float:
+    """Query-key pairs of `rows` tokens from an empty sequence."""
+    return rows * (rows + 1) / 2 if rows <= window else window * (window + 1) / 2 + (rows - window) * window
+
+
+def layered_prefill_flops(cfg: dict, rows: int) -> float:
     """Matrix-product operations of a prompt pass of `rows` tokens from an empty sequence: linears, window attention's
     visible scores and values, the recurrence (state update and read)."""
-    shapes = kulurax_tensor_shapes(cfg)
-    total = sum(2.0 * rows * np.prod(s) for n, s in shapes.items() if len(s) == 2 and n != "embed")
+    shapes = TENSOR_SHAPES[cfg["architecture"]](cfg)
+    total = sum(2.0 * rows * np.prod(s) for n, s in shapes.items() if len(s) == 2 and n not in ("embed", "head"))
     for layer in cfg["layers"]:
         m = layer["mixer"]
         if layer["type"] == "gla":
             total += 4.0 * rows * m["heads"] * m["dim"] * m["vdim"]
-        else:
-            w = m["mask"]["size"]
-            seen = rows * (rows + 1) / 2 if rows <= w else w * (w + 1) / 2 + (rows - w) * w
-            total += 2.0 * seen * m["heads"] * (m["dim"] + m["vdim"])
+        elif layer["type"] == "parallel":
+            r, m = m["right"], m["left"]
+            total += 4.0 * rows * r["heads"] * r["state"] * r["vdim"]
+        if "mask" in m:
+            total += 2.0 * window_pairs(rows, m["mask"]["size"]) * m["heads"] * (m["dim"] + m["vdim"])
     return float(total + 2.0 * cfg["vocab"] * cfg["width"])
