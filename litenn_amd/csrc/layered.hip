@@ -241,7 +241,7 @@ namespace litenn_hip
 		const float* vector(const std::string& name, int n)
 		{
 			Slot s;
-			s.vector = static_cast<float*>(allocate(sizeof(float) * static_cast<size_t>(n)));
+			s.vector = static_cast<float*>(allocate(sizeof(float) * ((static_cast<size_t>(n) + 3) & ~size_t{ 3 }))); // whole pieces
 			s.rows = static_cast<size_t>(n);
 			slots[name] = s;
 			return s.vector;

@@ -170,10 +170,11 @@ namespace litenn_hip
 		int window = 0;            // positions a query sees, itself included
 		float scale = 1.0f;
 		Rotary rot;
-		const float *q_norm = nullptr, *k_norm = nullptr; // [heads dim], [cache.heads dim], or null
+		const float *q_norm = nullptr, *k_norm = nullptr; // [heads dim], [cache.heads dim], or both null
 		float eps = 0.0f;
 		HeadCache cache;
-		const float *q = nullptr, *k = nullptr, *v = nullptr; // columns of one buffer; v may be k
+		// columns of one buffer; v may be k.  These and the norms start on 16-byte pieces and are readable up to whole ones.
+		const float *q = nullptr, *k = nullptr, *v = nullptr;
 		int ld = 0;
 		int rows = 1;
 		Position pos;

@@ -22,7 +22,7 @@ namespace litenn_hip
 			for (int i = threadIdx.x; i < rot.dims / 2; i += 256)
 			{
 				const double t = static_cast<double>(position) * rot.turns[i];
-				sincosf(static_cast<float>((t - rint(t)) * 6.283185307179586476925), sn + i, cs + i);
+				sincospif(static_cast<float>(2.0 * (t - rint(t))), sn + i, cs + i);
 			}
 		}
 
@@ -58,37 +58,159 @@ namespace litenn_hip
 			return 1.0f / sqrtf(block_sum256(ss, red) / static_cast<float>(n) + eps);
 		}
 
-		template <typename T>
+		// four elements from element e (a multiple of 4) of n, zero beyond; the row must be readable up to a whole piece
+		__device__ __forceinline__ floatx4 load_whole(const float* row, int e, int n)
+		{
+			floatx4 v = *reinterpret_cast<const floatx4*>(row + min(e, (n - 1) & ~3));
+#pragma unroll
+			for (int i = 0; i < 4; ++i)
+			{
+				v[i] = e + i < n ? v[i] : 0.0f;
+			}
+			return v;
+		}
+
+		// the same over two rows, one behind the other, the second one from element up4(n0)
+		__device__ __forceinline__ floatx4 load_either(const float* a, int n0, const float* b, int n1, int e)
+		{
+			const int first = (n0 + 3) & ~3;
+			return e < first ? load_whole(a, e, n0) : load_whole(b, e - first, n1);
+		}
+
+		// both sums over a workgroup of 256
+		__device__ __forceinline__ float2 block_sums256(float2 v, float* red)
+		{
+			v.x = wave_sum(v.x);
+			v.y = wave_sum(v.y);
+			__syncthreads();
+			if ((threadIdx.x & 63) == 0)
+			{
+				red[threadIdx.x >> 6] = v.x;
+				red[4 + (threadIdx.x >> 6)] = v.y;
+			}
+			__syncthreads();
+			return make_float2((red[0] + red[1]) + (red[2] + red[3]), (red[4] + red[5]) + (red[6] + red[7]));
+		}
+
+		__device__ __forceinline__ float sum_squares(const floatx4& v) { return (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]); }
+
+		__device__ __forceinline__ void store_piece(uint16_t* p, const floatx4& v)
+		{
+			*reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3]));
+		}
+		__device__ __forceinline__ void store_piece(float* p, const floatx4& v) { *reinterpret_cast<floatx4*>(p) = v; }
+
+		// KEPT > 0: queries and keys of up to 1024 KEPT elements pass through LDS, read once; 0: any number
+		template <typename T, int KEPT>
 		__global__ __launch_bounds__(256) void grouped_append_kernel(const GroupedAttn a)
 		{
-			__shared__ float red[4];
-			__shared__ float cs[kGroupedMaxDim / 2], sn[kGroupedMaxDim / 2];
-			const int row = blockIdx.x, position = row_position(a.pos, row);
+			__shared__ float red[8];
+			__shared__ __attribute__((aligned(16))) float cs[kGroupedMaxDim / 2], sn[kGroupedMaxDim / 2];
+			__shared__ __attribute__((aligned(16))) float lds[KEPT > 0 ? 1024 * KEPT : 4];
+			const int row = blockIdx.x, position = row_position(a.pos, row), tid = threadIdx.x;
 			const HeadCache& c = a.cache;
 			const float* q = a.q + static_cast<size_t>(row) * a.ld;
 			const float* k = a.k + static_cast<size_t>(row) * a.ld;
 			const float* v = a.v + static_cast<size_t>(row) * a.ld;
 			const int q_cols = a.heads * c.dim, k_cols = c.heads * c.dim, v_cols = c.heads * c.vdim;
-			rotary_angles(a.rot, position, cs, sn);
-			const float q_scale = projection_scale(q, a.q_norm, q_cols, a.eps, red);
-			const float k_scale = projection_scale(k, a.k_norm, k_cols, a.eps, red);
-			__syncthreads();
+			const int k_at = (q_cols + 3) & ~3, half = a.rot.dims >> 1;
 			float* q_out = a.q_out + static_cast<size_t>(row) * a.ldq;
-#pragma unroll 4
-			for (int e = threadIdx.x; e < q_cols; e += 256)
-			{
-				const int d = e % c.dim;
-				q_out[e] = rotated(q, a.q_norm, q_scale, e - d, d, a.rot, cs, sn);
-			}
 			T* rows = static_cast<T*>(c.rows) + static_cast<size_t>(position % c.ring) * c.row_pitch();
-			for (int e = threadIdx.x; e < k_cols; e += 256)
+			if constexpr (KEPT > 0)
 			{
-				const int d = e % c.dim;
-				operand_store(rows + e / c.dim * c.head_stride() + d, rotated(k, a.k_norm, k_scale, e - d, d, a.rot, cs, sn));
+				floatx4 x[KEPT], w[KEPT];
+#pragma unroll
+				for (int i = 0; i < KEPT; ++i)
+				{
+					x[i] = load_either(q, q_cols, k, k_cols, 4 * (tid + 256 * i));
+				}
+#pragma unroll
+				for (int i = 0; i < KEPT; ++i)
+				{
+					w[i] = a.q_norm ? load_either(a.q_norm, q_cols, a.k_norm, k_cols, 4 * (tid + 256 * i)) : floatx4{ 1.0f, 1.0f, 1.0f, 1.0f };
+				}
+				rotary_angles(a.rot, position, cs, sn);
+				float2 ss = make_float2(0.0f, 0.0f);
+#pragma unroll
+				for (int i = 0; i < KEPT; ++i)
+				{
+					const int e = 4 * (tid + 256 * i);
+					(e < k_at ? ss.x : ss.y) += sum_squares(x[i]);
+					*reinterpret_cast<floatx4*>(lds + e) = x[i] * w[i];
+				}
+				ss = block_sums256(ss, red);
+				const float q_scale = a.q_norm ? 1.0f / sqrtf(ss.x / static_cast<float>(q_cols) + a.eps) : 1.0f;
+				const float k_scale = a.q_norm ? 1.0f / sqrtf(ss.y / static_cast<float>(k_cols) + a.eps) : 1.0f;
+				if (c.dim % 4 == 0 && half % 4 == 0)
+				{
+					// four elements lie in one head and in one half of its pairs
+					const auto turned = [&](int at, int d, float scale) {
+						floatx4 x0 = *reinterpret_cast<const floatx4*>(lds + at + d);
+						if (d < 2 * half)
+						{
+							const bool lower = d < half;
+							const int i = lower ? d : d - half;
+							const floatx4 x1 = *reinterpret_cast<const floatx4*>(lds + at + (lower ? d + half : i));
+							const floatx4 co = *reinterpret_cast<const floatx4*>(cs + i), si = *reinterpret_cast<const floatx4*>(sn + i);
+							x0 = lower ? x0 * co - x1 * si : x0 * co + x1 * si;
+						}
+						return x0 * scale;
+					};
+					for (int e = 4 * tid; e < q_cols; e += 1024)
+					{
+						const int d = e % c.dim;
+						*reinterpret_cast<floatx4*>(q_out + e) = turned(e - d, d, q_scale);
+					}
+					for (int e = 4 * tid; e < k_cols; e += 1024)
+					{
+						const int d = e % c.dim;
+						store_piece(rows + e / c.dim * c.head_stride() + d, turned(k_at + e - d, d, k_scale));
+					}
+				}
+				else
+				{
+					for (int e = tid; e < q_cols; e += 256)
+					{
+						const int d = e % c.dim;
+						q_out[e] = rotated(lds, nullptr, q_scale, e - d, d, a.rot, cs, sn);
+					}
+					for (int e = tid; e < k_cols; e += 256)
+					{
+						const int d = e % c.dim;
+						operand_store(rows + e / c.dim * c.head_stride() + d, rotated(lds + k_at, nullptr, k_scale, e - d, d, a.rot, cs, sn));
+					}
+				}
 			}
-			for (int e = threadIdx.x; e < v_cols; e += 256)
+			else
 			{
-				operand_store(rows + e / c.vdim * c.head_stride() + c.key_pitch() + e % c.vdim, v[e]);
+				rotary_angles(a.rot, position, cs, sn);
+				const float q_scale = projection_scale(q, a.q_norm, q_cols, a.eps, red);
+				const float k_scale = projection_scale(k, a.k_norm, k_cols, a.eps, red);
+				__syncthreads();
+				for (int e = tid; e < q_cols; e += 256)
+				{
+					const int d = e % c.dim;
+					q_out[e] = rotated(q, a.q_norm, q_scale, e - d, d, a.rot, cs, sn);
+				}
+				for (int e = tid; e < k_cols; e += 256)
+				{
+					const int d = e % c.dim;
+					operand_store(rows + e / c.dim * c.head_stride() + d, rotated(k, a.k_norm, k_scale, e - d, d, a.rot, cs, sn));
+				}
+			}
+			if (c.vdim % 4 == 0)
+			{
+				for (int e = 4 * tid; e < v_cols; e += 1024)
+				{
+					store_piece(rows + e / c.vdim * c.head_stride() + c.key_pitch() + e % c.vdim, *reinterpret_cast<const floatx4*>(v + e));
+				}
+			}
+			else
+			{
+				for (int e = tid; e < v_cols; e += 256)
+				{
+					operand_store(rows + e / c.vdim * c.head_stride() + c.key_pitch() + e % c.vdim, v[e]);
+				}
 			}
 		}
 
@@ -110,7 +232,7 @@ namespace litenn_hip
 		size_t grouped_step_lds(const GroupedAttn& a)
 		{
 			const HeadCache& c = a.cache;
-			const size_t floats = ((a.rot.dims + 3) & ~3) + kStepHeads * (c.key_pitch() + KT);
+			const size_t floats = ((a.rot.dims + 3) & ~3) + (kStepHeads + 1) * c.key_pitch() + c.value_pitch() + kStepHeads * KT;
 			return sizeof(float) * floats + sizeof(T) * KT * static_cast<size_t>(key_stride<T>(c.key_pitch()) + c.value_pitch());
 		}
 
@@ -167,8 +289,10 @@ namespace litenn_hip
 			const int kp = c.key_pitch(), vp = c.value_pitch(), rp = c.row_pitch(), ks = key_stride<T>(kp);
 			float* const cs = lds;
 			float* const sn = cs + a.rot.dims / 2;
-			float* const qs = lds + ((a.rot.dims + 3) & ~3); // [kStepHeads][kp]
-			float* const weights = qs + kStepHeads * kp;     // [kStepHeads][KT]
+			float* const qs = lds + ((a.rot.dims + 3) & ~3); // [kStepHeads][kp], and the token's own key behind them
+			float* const own_key = qs + kStepHeads * kp;
+			float* const own_value = own_key + kp;     // [vp]
+			float* const weights = own_value + vp;     // [kStepHeads][KT]
 			T* const k_tile = reinterpret_cast<T*>(weights + kStepHeads * KT); // [KT][ks]
 			T* const v_tile = k_tile + KT * ks;                                // [KT][vp]
 
@@ -208,17 +332,89 @@ namespace litenn_hip
 			};
 			request(first + t0 * KT);
 
-			rotary_angles(a.rot, last, cs, sn);
-			const float q_scale = projection_scale(a.q, a.q_norm, a.heads * c.dim, a.eps, red);
-			const bool owns_last = t1 == tiles; // this split's last row is the token's own
-			const float k_scale = owns_last ? projection_scale(a.k, a.k_norm, c.heads * c.dim, a.eps, red) : 0.0f;
-			__syncthreads();
-			for (int i = tid; i < kStepHeads * kp; i += 256)
+			// this workgroup's queries and key as projected, times the norm's weights, and the value; what lies behind a
+			// head is zero.  All of it is requested before anything waits.
+			const int q_cols = a.heads * c.dim, k_cols = c.heads * c.dim;
+			constexpr int kQuads = 4;
+			float2 ss = make_float2(0.0f, 0.0f);
+			floatx4 all_q[kQuads], all_k;
+#pragma unroll
+			for (int i = 0; i < kQuads; ++i)
 			{
-				const int hq = i / kp, d = i % kp;
-				qs[i] = hq < heads && d < c.dim
-				            ? rotated(a.q, a.q_norm, q_scale, (head0 + hq) * c.dim, d, a.rot, cs, sn) * (a.scale * kLog2e)
-				            : 0.0f;
+				all_q[i] = load_whole(a.q, 4 * (tid + 256 * i), q_cols);
+			}
+			all_k = load_whole(a.k, 4 * tid, k_cols);
+			const int own = (kStepHeads + 1) * kp;
+			const auto own_index = [&](int i, bool& real) { // into the queries, or behind them into the keys
+				const int hq = i / kp, d = i - hq * kp;
+				real = d < c.dim && (hq < heads || (hq == kStepHeads && i < own));
+				return hq < kStepHeads ? (head0 + min(hq, heads - 1)) * c.dim + min(d, c.dim - 1)
+				                       : q_cols + kvh * c.dim + min(d, c.dim - 1);
+			};
+			for (int base = tid; base < own; base += 256 * 4)
+			{
+				float x[4], w[4];
+#pragma unroll
+				for (int u = 0; u < 4; ++u)
+				{
+					bool real;
+					const int at = own_index(min(base + 256 * u, own - 1), real);
+					x[u] = at < q_cols ? a.q[at] : a.k[at - q_cols];
+					w[u] = !a.q_norm ? 1.0f : at < q_cols ? a.q_norm[at] : a.k_norm[at - q_cols];
+				}
+#pragma unroll
+				for (int u = 0; u < 4; ++u)
+				{
+					const int i = base + 256 * u;
+					if (i < own)
+					{
+						bool real;
+						own_index(i, real);
+						qs[i] = real ? x[u] * w[u] : 0.0f;
+					}
+				}
+			}
+			for (int i = tid; i < vp; i += 256)
+			{
+				own_value[i] = i < c.vdim ? a.v[kvh * c.vdim + i] : 0.0f;
+			}
+			rotary_angles(a.rot, last, cs, sn);
+#pragma unroll
+			for (int i = 0; i < kQuads; ++i)
+			{
+				ss.x += sum_squares(all_q[i]);
+			}
+			ss.y = sum_squares(all_k);
+			for (int i = 4 * (tid + 256 * kQuads); i < q_cols; i += 1024)
+			{
+				ss.x += sum_squares(load_whole(a.q, i, q_cols));
+			}
+			for (int i = 4 * (tid + 256); i < k_cols; i += 1024)
+			{
+				ss.y += sum_squares(load_whole(a.k, i, k_cols));
+			}
+			ss = block_sums256(ss, red);
+			const float q_scale = (a.q_norm ? 1.0f / sqrtf(ss.x / static_cast<float>(q_cols) + a.eps) : 1.0f) * (a.scale * kLog2e);
+			const float k_scale = a.q_norm ? 1.0f / sqrtf(ss.y / static_cast<float>(k_cols) + a.eps) : 1.0f;
+			// scaled and rotated where they are: a thread owns a pair, or an element that passes unchanged
+			{
+				const int half = a.rot.dims >> 1, per_row = kp - half;
+				for (int i = tid; i < (kStepHeads + 1) * per_row; i += 256)
+				{
+					const int hq = i / per_row, m = i - hq * per_row;
+					const float by = hq < kStepHeads ? q_scale : k_scale;
+					float* const x = qs + hq * kp;
+					if (m < half)
+					{
+						const float u = x[m] * by, v = x[m + half] * by;
+						x[m] = u * cs[m] - v * sn[m];
+						x[m + half] = v * cs[m] + u * sn[m];
+					}
+					else
+					{
+						x[m + half] *= by;
+					}
+				}
 			}
 
 			// wavefront w works on heads w and w + 4 of the workgroup's
@@ -266,14 +462,9 @@ namespace litenn_hip
 					for (int i = tid; i < rp; i += 256)
 					{
 						const int e = i < kp ? i : i - kp;
-						const bool real = e < (i < kp ? c.dim : c.vdim);
-						float x = 0.0f;
-						if (real)
-						{
-							x = i < kp ? rotated(a.k, a.k_norm, k_scale, kvh * c.dim, e, a.rot, cs, sn) : a.v[kvh * c.vdim + e];
-						}
+						const float x = own_key[i]; // the value follows the key
 						operand_store(i < kp ? k_tile + (count - 1) * ks + e : v_tile + (count - 1) * vp + e, x);
-						if (real && chunk == 0)
+						if (e < (i < kp ? c.dim : c.vdim) && chunk == 0)
 						{
 							operand_store(row + i, x);
 						}
@@ -465,38 +656,85 @@ namespace litenn_hip
 			load_rows(0);
 			const int p = row_position(a.pos, 0);
 			const float* const raw = a.in + inner; // x | B | C
-			const float dt = softplus_f32(a.in[inner + channels + h] + a.dt_bias[h]);
-			const float decay = expf(-expf(a.a_log[h]) * dt);
-			const auto convolved = [&](int ch, bool keep) {
-				const float now = raw[ch];
-				float acc = fmaf(a.conv_w[static_cast<size_t>(a.taps - 1) * channels + ch], now, a.conv_b[ch]);
-				for (int back = 1; back < a.taps; ++back)
+			const float dt_raw = a.in[inner + channels + h] + a.dt_bias[h], rate = a.a_log[h];
+			// the last kNear taps of a channel and its input travel together
+			constexpr int kNear = 4;
+			struct Window
+			{
+				float w[kNear], x[kNear], bias;
+			};
+			int slot[kNear]; // ring rows, of tap 0 the token's own
+#pragma unroll
+			for (int back = 0; back < kNear; ++back)
+			{
+				const int at = min(back, a.taps - 1);
+				slot[back] = p >= at ? (p - at) % a.taps : 0;
+			}
+			const auto request = [&](int ch) {
+				Window t;
+#pragma unroll
+				for (int back = 0; back < kNear; ++back)
 				{
-					if (p >= back)
-					{
-						acc = fmaf(a.conv_w[static_cast<size_t>(a.taps - 1 - back) * channels + ch],
-						           a.ring[static_cast<size_t>((p - back) % a.taps) * channels + ch], acc);
-					}
+					t.w[back] = a.conv_w[static_cast<size_t>(a.taps - 1 - min(back, a.taps - 1)) * channels + ch];
+					t.x[back] = back ? a.ring[static_cast<size_t>(slot[back]) * channels + ch] : raw[ch];
+				}
+				t.bias = a.conv_b[ch];
+				return t;
+			};
+			const auto convolved = [&](const Window& t, int ch, bool keep) {
+				float acc = fmaf(t.w[0], t.x[0], t.bias);
+#pragma unroll
+				for (int back = 1; back < kNear; ++back)
+				{
+					acc = back < a.taps && p >= back ? fmaf(t.w[back], t.x[back], acc) : acc;
+				}
+				for (int back = kNear; back < a.taps && back <= p; ++back)
+				{
+					acc = fmaf(a.conv_w[static_cast<size_t>(a.taps - 1 - back) * channels + ch],
+					           a.ring[static_cast<size_t>((p - back) % a.taps) * channels + ch], acc);
 				}
 				if (keep)
 				{
-					a.ring[static_cast<size_t>(p % a.taps) * channels + ch] = now;
+					a.ring[static_cast<size_t>(slot[0]) * channels + ch] = t.x[0];
 				}
 				return silu_f32(acc);
 			};
-			// one workgroup of a group stores the group's inputs
+			// B and C of the group (one workgroup of a group stores their inputs), then this workgroup's columns of x
 			const bool keep = slice == 0 && h % (a.heads / a.groups) == 0;
-			for (int i = tid; i < 2 * a.state; i += 256)
-			{
-				const bool is_c = i >= a.state;
-				const int n = is_c ? i - a.state : i;
-				const float v = convolved(inner + (is_c ? a.groups * a.state : 0) + group * a.state + n, keep);
-				(is_c ? cs : bs)[n] = is_c ? v : v * dt;
-			}
+			const int total = 2 * a.state + kSsmCols;
+			const auto channel = [&](int i) {
+				i = min(i, total - 1);
+				return i < a.state       ? inner + group * a.state + i
+				       : i < 2 * a.state ? inner + (a.groups - 1 + group) * a.state + i
+				                         : h * a.vdim + min(slice * kSsmCols + i - 2 * a.state, a.vdim - 1);
+			};
 			const int col = slice * kSsmCols + tid;
-			if (tid < kSsmCols)
+			Window w0 = request(channel(tid)), w1 = request(channel(tid + 256));
+			const float dt = softplus_f32(dt_raw), decay = expf(-expf(rate) * dt);
+			for (int first = tid; first < total; first += 512)
 			{
-				xs[tid] = col < a.vdim ? convolved(h * a.vdim + col, true) : 0.0f;
+				if (first != tid)
+				{
+					w0 = request(channel(first));
+					w1 = request(channel(first + 256));
+				}
+#pragma unroll
+				for (int u = 0; u < 2; ++u)
+				{
+					const int i = first + 256 * u;
+					if (i < 2 * a.state)
+					{
+						const float v = convolved(u ? w1 : w0, channel(i), keep);
+						(i < a.state ? bs[i] : cs[i - a.state]) = i < a.state ? v * dt : v;
+					}
+					else if (i < total)
+					{
+						const int e2 = i - 2 * a.state;
+						const bool inside_head = slice * kSsmCols + e2 < a.vdim;
+						const float v = convolved(u ? w1 : w0, channel(i), inside_head);
+						xs[e2] = inside_head ? v : 0.0f;
+					}
+				}
 			}
 			__syncthreads();
 			const floatx4 x = *reinterpret_cast<const floatx4*>(xs + (tid & 7) * 4);
@@ -540,7 +778,7 @@ namespace litenn_hip
 		__global__ __launch_bounds__(256) void mixer_step_kernel(const GroupedAttn attn, int attn_blocks, const Ssm ssm)
 		{
 			extern __shared__ __attribute__((aligned(16))) float step_lds[];
-			__shared__ float red[4];
+			__shared__ float red[8];
 			if (static_cast<int>(blockIdx.x) < attn_blocks)
 			{
 				grouped_step_block<T, KT>(attn, static_cast<int>(blockIdx.x), step_lds, red);
@@ -639,7 +877,8 @@ namespace litenn_hip
 		constexpr int kConvRows = 8; // rows of a thread
 
 		// x | B | C behind convolution and silu, four channels per thread; the last column of workgroups makes the
-		// step sizes and log decays
+		// step sizes and log decays.  TAPS > 0: that many taps, channels a multiple of 4, every input read once; 0: any.
+		template <int TAPS>
 		__global__ __launch_bounds__(256) void ssm_conv_kernel(const Ssm a)
 		{
 			const int inner = a.inner(), channels = a.channels(), ldx = a.ldx();
@@ -680,13 +919,52 @@ namespace litenn_hip
 			{
 				acc[t] = bias;
 			}
-			for (int tap = 0; tap < a.taps; ++tap)
+			if constexpr (TAPS > 0)
 			{
-				const floatx4 w = load_columns(a.conv_w + static_cast<size_t>(tap) * channels, ch, channels);
+				floatx4 in[kConvRows + TAPS - 1], w[TAPS];
+				const float* const column = a.in + inner + ch;
+#pragma unroll
+				for (int i = 0; i < kConvRows + TAPS - 1; ++i)
+				{
+					const int row = min(max(row0 + i - (TAPS - 1), 0), a.rows - 1);
+					in[i] = *reinterpret_cast<const floatx4_a4*>(column + static_cast<size_t>(row) * a.ld);
+				}
+#pragma unroll
+				for (int tap = 0; tap < TAPS; ++tap)
+				{
+					w[tap] = *reinterpret_cast<const floatx4*>(a.conv_w + static_cast<size_t>(tap) * channels + ch);
+				}
+				if (row0 < TAPS - 1) // inputs from ahead of these rows
+				{
+#pragma unroll
+					for (int i = 0; i < TAPS - 1; ++i)
+					{
+						if (row0 + i < TAPS - 1)
+						{
+							in[i] = input(row0 + i - (TAPS - 1));
+						}
+					}
+				}
 #pragma unroll
 				for (int t = 0; t < kConvRows; ++t)
 				{
-					acc[t] += w * input(row0 + t - (a.taps - 1) + tap);
+#pragma unroll
+					for (int tap = 0; tap < TAPS; ++tap)
+					{
+						acc[t] += w[tap] * in[t + tap];
+					}
+				}
+			}
+			else
+			{
+				for (int tap = 0; tap < a.taps; ++tap)
+				{
+					const floatx4 w = load_columns(a.conv_w + static_cast<size_t>(tap) * channels, ch, channels);
+#pragma unroll
+					for (int t = 0; t < kConvRows; ++t)
+					{
+						acc[t] += w * input(row0 + t - (a.taps - 1) + tap);
+					}
 				}
 			}
 #pragma unroll
@@ -1025,6 +1303,28 @@ namespace litenn_hip
 
 		bool narrow_heads(const HeadCache& c) { return c.key_pitch() <= 256 && c.value_pitch() <= 256; }
 
+		template <typename T>
+		void launch_append(const GroupedAttn& a, hipStream_t s)
+		{
+			const size_t cols = ((static_cast<size_t>(a.heads) * a.cache.dim + 3) & ~size_t{ 3 }) + static_cast<size_t>(a.cache.heads) * a.cache.dim;
+			if (cols <= 2048)
+			{
+				grouped_append_kernel<T, 2><<<dim3(a.rows), dim3(256), 0, s>>>(a);
+			}
+			else if (cols <= 5120)
+			{
+				grouped_append_kernel<T, 5><<<dim3(a.rows), dim3(256), 0, s>>>(a);
+			}
+			else if (cols <= 10240)
+			{
+				grouped_append_kernel<T, 10><<<dim3(a.rows), dim3(256), 0, s>>>(a);
+			}
+			else
+			{
+				grouped_append_kernel<T, 0><<<dim3(a.rows), dim3(256), 0, s>>>(a);
+			}
+		}
+
 		template <typename T, int KT>
 		void launch_step(const GroupedAttn& attn, int attn_blocks, const Ssm& ssm, int ssm_blocks, hipStream_t s)
 		{
@@ -1045,11 +1345,11 @@ namespace litenn_hip
 		}
 		if (a.cache.f32)
 		{
-			grouped_append_kernel<float><<<dim3(a.rows), dim3(256), 0, s>>>(a);
+			launch_append<float>(a, s);
 		}
 		else
 		{
-			grouped_append_kernel<uint16_t><<<dim3(a.rows), dim3(256), 0, s>>>(a);
+			launch_append<uint16_t>(a, s);
 		}
 	}
 
@@ -1105,7 +1405,14 @@ namespace litenn_hip
 			return;
 		}
 		const int conv_blocks = (a.ldx() / 4 + 63) / 64;
-		ssm_conv_kernel<<<dim3(conv_blocks + 1, (a.rows + 4 * kConvRows - 1) / (4 * kConvRows)), dim3(256), 0, s>>>(a);
+		const dim3 conv_grid(conv_blocks + 1, (a.rows + 4 * kConvRows - 1) / (4 * kConvRows));
+		switch (a.channels() % 4 == 0 ? a.taps : 0)
+		{
+		case 2: ssm_conv_kernel<2><<<conv_grid, dim3(256), 0, s>>>(a); break;
+		case 3: ssm_conv_kernel<3><<<conv_grid, dim3(256), 0, s>>>(a); break;
+		case 4: ssm_conv_kernel<4><<<conv_grid, dim3(256), 0, s>>>(a); break;
+		default: ssm_conv_kernel<0><<<conv_grid, dim3(256), 0, s>>>(a); break;
+		}
 		const int chunks = (a.rows + kChunk - 1) / kChunk;
 		const int slabs = (a.state + kSlab - 1) / kSlab, slices = (a.vdim + kSlice - 1) / kSlice;
 		ssm_state_kernel<<<dim3(a.heads * slabs * slices, chunks), dim3(256), 0, s>>>(a);

@@ -60,6 +60,10 @@ SINGLE = {
     "attention_256": left_only(du.attention(4, 2, 256, 100, 0.05, 256)),
     "attention_beyond_tiles": left_only(du.attention(4, 1, 264, 40, 0.05, 130)),
     "attention_largest": left_only(du.attention(3, 1, 512, 20, 0.05, 512)),
+    "attention_many_queries": left_only(du.attention(32, 2, 128, 33, 0.09, 128)),
+    "attention_more_queries": left_only(du.attention(40, 2, 200, 33, 0.07, 96)),
+    "attention_most_queries": left_only(du.attention(48, 2, 256, 33, 0.06, 256)),
+    "attention_many_odd_queries": left_only(du.attention(90, 5, 33, 40, 0.2, 18)),
     "attention_sees_all": left_only(du.attention(4, 2, 32, 5000, 0.1, 32)),
     "ssm": right_only(du.state_space()),
     "ssm_ones": right_only(du.state_space(1, 1, 1, 1, 1, 1)),
