@@ -271,6 +271,9 @@ namespace litenn_hip
 			return acc;
 		}
 
+		// the least shift, up to 8, whose power of two is n or more
+		__device__ __forceinline__ int shift_over(int n) { return min(8, 32 - __clz(n - 1)); }
+
 		__host__ __device__ inline int grouped_chunks(int heads, int kv_heads)
 		{
 			return (heads / kv_heads + kStepHeads - 1) / kStepHeads;
@@ -311,23 +314,28 @@ namespace litenn_hip
 				}
 				return;
 			}
-			// a tile's rows in 16-byte pieces; a thread's first kAhead pieces are requested before anything waits
+			// Threads are dealt to rows by shifts (a kernel this short is bound by the instructions it fetches): a tile's
+			// rows in 16-byte pieces, one piece column per thread; its first kAhead pieces are requested before anything waits
 			constexpr int E = 16 / static_cast<int>(sizeof(T)), kAhead = 8;
-			const int row_pieces = rp / E;
-			const T* const cache = static_cast<const T*>(c.rows) + kvh * c.head_stride();
-			const auto piece_of = [&](int base, int p) {
-				const int count = min(KT, last - base + 1);
-				int r = base % c.ring + min(p / row_pieces, count - 1);
+			const int row_pieces = rp / E, piece_shift = shift_over(row_pieces);
+			const int piece_row = tid >> piece_shift, piece_step = 256 >> piece_shift, piece = tid & ((1 << piece_shift) - 1);
+			const int piece_col = min(piece, row_pieces - 1) * E;
+			const T* const cache = static_cast<const T*>(c.rows) + kvh * c.head_stride() + piece_col;
+			T* const piece_to = piece_col < kp ? k_tile + piece_col : v_tile + piece_col - kp;
+			const int piece_stride = piece_col < kp ? ks : vp;
+			int ring_at = (first + t0 * KT) % c.ring; // ring row of the tile's first position
+			const auto piece_of = [&](int count, int row) {
+				int r = ring_at + min(row, count - 1);
 				r -= r >= c.ring ? c.ring : 0;
-				return *reinterpret_cast<const u32x4*>(cache + static_cast<size_t>(r) * rp + p % row_pieces * E);
+				return *reinterpret_cast<const u32x4*>(cache + static_cast<size_t>(r) * rp);
 			};
-			const int pieces = KT * row_pieces;
 			u32x4 ahead[kAhead];
 			const auto request = [&](int base) {
+				const int count = min(KT, last - base + 1);
 #pragma unroll
 				for (int i = 0; i < kAhead; ++i)
 				{
-					ahead[i] = piece_of(base, min(tid + 256 * i, pieces - 1));
+					ahead[i] = piece_of(count, piece_row + i * piece_step);
 				}
 			};
 			request(first + t0 * KT);
@@ -344,33 +352,27 @@ namespace litenn_hip
 				all_q[i] = load_whole(a.q, 4 * (tid + 256 * i), q_cols);
 			}
 			all_k = load_whole(a.k, 4 * tid, k_cols);
-			const int own = (kStepHeads + 1) * kp;
-			const auto own_index = [&](int i, bool& real) { // into the queries, or behind them into the keys
-				const int hq = i / kp, d = i - hq * kp;
-				real = d < c.dim && (hq < heads || (hq == kStepHeads && i < own));
-				return hq < kStepHeads ? (head0 + min(hq, heads - 1)) * c.dim + min(d, c.dim - 1)
-				                       : q_cols + kvh * c.dim + min(d, c.dim - 1);
-			};
-			for (int base = tid; base < own; base += 256 * 4)
+			const int own_shift = shift_over(kp), own_d = tid & ((1 << own_shift) - 1);
+			const int own_row = tid >> own_shift, own_step = 256 >> own_shift; // a row longer than 256 takes all threads twice
+			for (int d = own_d; d < kp; d += 256)
 			{
-				float x[4], w[4];
-#pragma unroll
-				for (int u = 0; u < 4; ++u)
+				constexpr int kRows = 3;
+				for (int row = own_row; row <= heads; row += kRows * own_step)
 				{
-					bool real;
-					const int at = own_index(min(base + 256 * u, own - 1), real);
-					x[u] = at < q_cols ? a.q[at] : a.k[at - q_cols];
-					w[u] = !a.q_norm ? 1.0f : at < q_cols ? a.q_norm[at] : a.k_norm[at - q_cols];
-				}
+					float x[kRows], w[kRows];
 #pragma unroll
-				for (int u = 0; u < 4; ++u)
-				{
-					const int i = base + 256 * u;
-					if (i < own)
+					for (int u = 0; u < kRows; ++u)
 					{
-						bool real;
-						own_index(i, real);
-						qs[i] = real ? x[u] * w[u] : 0.0f;
+						const int hq = min(row + u * own_step, heads);
+						const int at = (hq < heads ? head0 + hq : kvh) * c.dim + min(d, c.dim - 1);
+						x[u] = (hq < heads ? a.q : a.k)[at];
+						w[u] = a.q_norm ? (hq < heads ? a.q_norm : a.k_norm)[at] : 1.0f;
+					}
+#pragma unroll
+					for (int u = 0; u < kRows; ++u)
+					{
+						const int hq = min(row + u * own_step, heads);
+						(hq < heads ? qs + hq * kp : own_key)[d] = d < c.dim ? x[u] * w[u] : 0.0f;
 					}
 				}
 			}
@@ -398,21 +400,23 @@ namespace litenn_hip
 			const float k_scale = a.q_norm ? 1.0f / sqrtf(ss.y / static_cast<float>(k_cols) + a.eps) : 1.0f;
 			// scaled and rotated where they are: a thread owns a pair, or an element that passes unchanged
 			{
-				const int half = a.rot.dims >> 1, per_row = kp - half;
-				for (int i = tid; i < (kStepHeads + 1) * per_row; i += 256)
+				const int half = a.rot.dims >> 1;
+				for (int m = own_d; m < kp - half; m += 256)
 				{
-					const int hq = i / per_row, m = i - hq * per_row;
-					const float by = hq < kStepHeads ? q_scale : k_scale;
-					float* const x = qs + hq * kp;
-					if (m < half)
+					for (int row = own_row; row <= heads; row += own_step)
 					{
-						const float u = x[m] * by, v = x[m + half] * by;
-						x[m] = u * cs[m] - v * sn[m];
-						x[m + half] = v * cs[m] + u * sn[m];
-					}
-					else
-					{
-						x[m + half] *= by;
+						const float by = row < heads ? q_scale : k_scale;
+						float* const x = row < heads ? qs + row * kp : own_key;
+						if (m < half)
+						{
+							const float u = x[m] * by, v = x[m + half] * by;
+							x[m] = u * cs[m] - v * sn[m];
+							x[m + half] = v * cs[m] + u * sn[m];
+						}
+						else
+						{
+							x[m + half] *= by;
+						}
 					}
 				}
 			}
@@ -436,25 +440,24 @@ namespace litenn_hip
 				const int base = first + t * KT;
 				const int count = min(KT, last - base + 1);
 				__syncthreads(); // the previous tile has been consumed
-				const auto stage = [&](int p, u32x4 w) {
-					const int r = p / row_pieces, col = p % row_pieces * E;
-					if (p < pieces && base + r != last)
+				const auto stage = [&](int row, u32x4 w) {
+					if (row < KT && piece < row_pieces && base + row != last)
 					{
-						if (r >= count)
+						if (row >= count)
 						{
 							w = u32x4{ 0u, 0u, 0u, 0u };
 						}
-						*reinterpret_cast<u32x4*>(col < kp ? k_tile + r * ks + col : v_tile + r * vp + col - kp) = w;
+						*reinterpret_cast<u32x4*>(piece_to + row * piece_stride) = w;
 					}
 				};
 #pragma unroll
 				for (int i = 0; i < kAhead; ++i)
 				{
-					stage(tid + 256 * i, ahead[i]);
+					stage(piece_row + i * piece_step, ahead[i]);
 				}
-				for (int p = tid + 256 * kAhead; p < pieces; p += 256)
+				for (int row = piece_row + kAhead * piece_step; row < KT; row += piece_step)
 				{
-					stage(p, piece_of(base, p));
+					stage(row, piece_of(count, row));
 				}
 				if (base + count - 1 == last)
 				{
@@ -472,6 +475,8 @@ namespace litenn_hip
 				}
 				if (t + 1 < t1)
 				{
+					ring_at += KT; // there is another tile: the ring is longer than this one
+					ring_at -= ring_at >= c.ring ? c.ring : 0;
 					request(base + KT);
 				}
 				__syncthreads();
@@ -532,10 +537,9 @@ namespace litenn_hip
 #pragma unroll
 						for (int i = 0; i < kCols; ++i)
 						{
-							const int col = 2 * lane + 128 * i;
-							if (col < vp)
+							if (128 * i < vp) // uniform; what lies behind the last column is not stored
 							{
-								const float2 x = unpack2(v_tile + (kk + e) * vp + col);
+								const float2 x = unpack2(v_tile + (kk + e) * vp + min(2 * lane + 128 * i, vp - 2));
 								o[0][i].x = fmaf(p0[e], x.x, o[0][i].x);
 								o[0][i].y = fmaf(p0[e], x.y, o[0][i].y);
 								o[1][i].x = fmaf(p1[e], x.x, o[1][i].x);
@@ -663,20 +667,15 @@ namespace litenn_hip
 			{
 				float w[kNear], x[kNear], bias;
 			};
-			int slot[kNear]; // ring rows, of tap 0 the token's own
-#pragma unroll
-			for (int back = 0; back < kNear; ++back)
-			{
-				const int at = min(back, a.taps - 1);
-				slot[back] = p >= at ? (p - at) % a.taps : 0;
-			}
+			const int slot0 = p % a.taps; // ring row of the token's own input
+			const auto slot = [&](int back) { return slot0 - back + (slot0 < back ? a.taps : 0); };
 			const auto request = [&](int ch) {
 				Window t;
 #pragma unroll
 				for (int back = 0; back < kNear; ++back)
 				{
 					t.w[back] = a.conv_w[static_cast<size_t>(a.taps - 1 - min(back, a.taps - 1)) * channels + ch];
-					t.x[back] = back ? a.ring[static_cast<size_t>(slot[back]) * channels + ch] : raw[ch];
+					t.x[back] = back ? a.ring[static_cast<size_t>(slot(min(back, a.taps - 1))) * channels + ch] : raw[ch];
 				}
 				t.bias = a.conv_b[ch];
 				return t;
@@ -691,11 +690,11 @@ namespace litenn_hip
 				for (int back = kNear; back < a.taps && back <= p; ++back)
 				{
 					acc = fmaf(a.conv_w[static_cast<size_t>(a.taps - 1 - back) * channels + ch],
-					           a.ring[static_cast<size_t>((p - back) % a.taps) * channels + ch], acc);
+					           a.ring[static_cast<size_t>(slot(back)) * channels + ch], acc);
 				}
 				if (keep)
 				{
-					a.ring[static_cast<size_t>(slot[0]) * channels + ch] = t.x[0];
+					a.ring[static_cast<size_t>(slot0) * channels + ch] = t.x[0];
 				}
 				return silu_f32(acc);
 			};
@@ -709,32 +708,28 @@ namespace litenn_hip
 				                         : h * a.vdim + min(slice * kSsmCols + i - 2 * a.state, a.vdim - 1);
 			};
 			const int col = slice * kSsmCols + tid;
-			Window w0 = request(channel(tid)), w1 = request(channel(tid + 256));
-			const float dt = softplus_f32(dt_raw), decay = expf(-expf(rate) * dt);
-			for (int first = tid; first < total; first += 512)
+			float dt = 0.0f, decay = 0.0f;
+			for (int first = 0; first < total; first += 512)
 			{
-				if (first != tid)
+				const int i0 = first + tid, i1 = i0 + 256;
+				const Window w0 = request(channel(i0)), w1 = request(channel(i1));
+				if (first == 0)
 				{
-					w0 = request(channel(first));
-					w1 = request(channel(first + 256));
+					dt = softplus_f32(dt_raw);
+					decay = expf(-expf(rate) * dt);
 				}
-#pragma unroll
-				for (int u = 0; u < 2; ++u)
-				{
-					const int i = first + 256 * u;
-					if (i < 2 * a.state)
+				const auto put = [&](int i, const Window& w) {
+					if (i >= total)
 					{
-						const float v = convolved(u ? w1 : w0, channel(i), keep);
-						(i < a.state ? bs[i] : cs[i - a.state]) = i < a.state ? v * dt : v;
+						return;
 					}
-					else if (i < total)
-					{
-						const int e2 = i - 2 * a.state;
-						const bool inside_head = slice * kSsmCols + e2 < a.vdim;
-						const float v = convolved(u ? w1 : w0, channel(i), inside_head);
-						xs[e2] = inside_head ? v : 0.0f;
-					}
-				}
+					const bool is_x = i >= 2 * a.state, inside_head = slice * kSsmCols + i - 2 * a.state < a.vdim;
+					const float v = convolved(w, channel(i), is_x ? inside_head : keep);
+					float* const to = is_x ? xs + i - 2 * a.state : i < a.state ? bs + i : cs + i - a.state;
+					*to = is_x && !inside_head ? 0.0f : i < a.state ? v * dt : v;
+				};
+				put(i0, w0);
+				put(i1, w1);
 			}
 			__syncthreads();
 			const floatx4 x = *reinterpret_cast<const floatx4*>(xs + (tid & 7) * 4);
