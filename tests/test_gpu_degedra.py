@@ -418,3 +418,46 @@ def test_trace_replay(hip, tmp_path, dtype):
             d = got - full[rid][places]
             d -= d.mean(axis=1, keepdims=True)
             assert np.sqrt((d * d).mean(axis=1)).max() <= LIMIT[dtype] * full[rid].std()
+
+
+def random_config(seed):
+    """Two or three layers of sizes drawn at random, one perhaps with another's weights."""
+    rng = np.random.default_rng([seed, 91])
+
+    def pick(*values):
+        return values[int(rng.integers(len(values)))]
+
+    layers = []
+    for _ in range(int(rng.integers(1, 4))):
+        kv_heads, dim = int(rng.integers(1, 5)), int(rng.integers(1, 100))
+        left = du.attention(kv_heads * int(rng.integers(1, 12)), kv_heads, dim, int(rng.integers(1, 150)),
+                            float(rng.uniform(0.3, 1.0) / np.sqrt(dim)), 2 * int(rng.integers(0, dim // 2 + 1)),
+                            float(rng.uniform(2.0, 1e5)))
+        groups, per_group, vdim = int(rng.integers(1, 4)), int(rng.integers(1, 5)), int(rng.integers(1, 100))
+        inner = groups * per_group * vdim
+        parts = pick(*[n for n in range(1, 9) if inner % n == 0 and inner // n >= 16] or [1])
+        right = du.state_space(groups * per_group, vdim, int(rng.integers(1, 150)), groups, parts, int(rng.integers(1, 7)))
+        layers.append(du.layer(left, right, pick(None, int(rng.integers(1, 300))), float(rng.uniform(0.3, 1.5)),
+                               float(rng.uniform(0.3, 1.5))))
+    if pick(0, 1):
+        layers.append(du.again(layers, int(rng.integers(len(layers)))))
+    return du.config(layers, int(rng.integers(2, 300)), int(rng.integers(8, 300)), 10.0 ** -int(rng.integers(3, 7)),
+                     float(rng.uniform(2.0, 50.0)))
+
+
+@pytest.mark.parametrize("seed", range(24))
+def test_random_configurations(hip, seed):
+    """Sizes nobody chose, in portions nobody chose; 16 bits beside 32 on the same tokens."""
+    cfg = random_config(seed)
+    rng = np.random.default_rng([seed, 92])
+    w = du.random_weights(cfg, seed)
+    plain = ref.NumpyDegedra(cfg, du.as_floats(w))
+    toks = du.tokens(cfg, int(rng.integers(100, 260)), seed)
+    want = plain.forward(toks)
+    cuts = [int(n) for n in rng.integers(1, rng.integers(4, 90), 40)] + [1]
+    for dtype in DTYPES:
+        model = hip.create_model(cfg, w, dtype=dtype, context_length=300)
+        errors = du.row_errors(feed(model, toks, cuts), want)
+        model.close()
+        # in 16 bits a token whose mixers nearly cancel may be far off
+        assert (errors.max() if dtype == "float32" else np.quantile(errors, 0.9)) <= LIMIT[dtype], (dtype, cfg, cuts)
